@@ -49,6 +49,10 @@ class ModelConfig:
     def validate(self) -> None:
         """Raise ConfigError for values no model can be built from."""
 
+    def sizes_from_weights(self, shapes: Dict[str, Any]) -> None:
+        """Take sizes that ``config.json`` leaves to the weight file: ``shapes`` is tensor name -> shape of what the files
+        hold.  Called by whoever builds a model from a folder, before the model is put together."""
+
     # dict / json -------------------------------------------------------
     @classmethod
     def preprocess_dict(cls, d: Dict[str, Any]) -> Dict[str, Any]:

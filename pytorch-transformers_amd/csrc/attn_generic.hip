@@ -19,7 +19,8 @@ __global__ void attn_generic_kernel(T* __restrict__ out, const T* __restrict__ q
                                     const T* __restrict__ v_pool, const int* __restrict__ block_table,
                                     int bt_stride, const int* __restrict__ token_seq,
                                     const int* __restrict__ token_pos, const float* __restrict__ slopes, int bias_mode, float bias_scale,
-                                    int nh, int nkv, int d, float scale, int window, int chunk) {
+                                    int nh, int nkv, int d, float scale, int window, int chunk,
+                                    const float* __restrict__ sink) {
     __shared__ float q_s[256];
     __shared__ float p_s[PTA_PAGE];
     const int m = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -74,7 +75,14 @@ __global__ void attn_generic_kernel(T* __restrict__ out, const T* __restrict__ q
         m_run = m_new;
     }
     T* orow = out + ((long)m * nh + h) * d;
-    const float inv = 1.0f / l_run;
+    // a learned number per head: its exponential joins the sum of the weights once, with no key and no value
+    float last = 1.f;
+    if (sink) {
+        const float m_new = fmaxf(m_run, sink[h]);
+        last = expf(m_run - m_new);
+        l_run = l_run * last + expf(sink[h] - m_new);
+    }
+    const float inv = last / l_run;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int dim = lane + r * PTA_WAVE;
@@ -95,8 +103,8 @@ extern "C" int pta_attention_sizes_ok(int nh, int nkv, int d, int rotated) {
 
 extern "C" int pta_attn_generic(void* out, const void* q, const void* k_pool, const void* v_pool,
                                 const int* block_table, int bt_stride, const int* token_seq, const int* token_pos,
-                                const PtaScoreBias* score_bias, int M, int nh, int nkv, int d, float scale, int window, int chunk, int dtype,
-                                void* stream) {
+                                const PtaScoreBias* score_bias, int M, int nh, int nkv, int d, float scale, int window, int chunk,
+                                const float* sink, int dtype, void* stream) {
     int bias_mode = 0;
     if (pta_score_bias_mode("attn_generic", score_bias, &bias_mode)) return 1;
     const float* slopes = score_bias ? score_bias->slopes : nullptr;
@@ -112,11 +120,11 @@ extern "C" int pta_attn_generic(void* out, const void* q, const void* k_pool, co
     if (dtype == PTA_F32)
         hipLaunchKernelGGL(attn_generic_kernel<float>, grid, dim3(PTA_WAVE), 0, s, (float*)out, (const float*)q,
                            (const float*)k_pool, (const float*)v_pool, block_table, bt_stride, token_seq, token_pos,
-                           slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk);
+                           slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink);
     else if (dtype == PTA_BF16)
         hipLaunchKernelGGL(attn_generic_kernel<bf16_t>, grid, dim3(PTA_WAVE), 0, s, (bf16_t*)out, (const bf16_t*)q,
                            (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_table, bt_stride, token_seq,
-                           token_pos, slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk);
+                           token_pos, slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink);
     else
         return pta_fail("attn_generic: unknown dtype %d", dtype);
     return pta_check_launch("attn_generic");

@@ -64,8 +64,8 @@ extern "C" int pta_latent_prep(float* q_full, void* k_pool, const void* q_rows, 
                                const int* block_table, int bt_stride, int M, int H, int dn, int dr, int R,
                                int write_cache, int dtype, void* stream) {
     PTA_REQUIRE(M > 0 && H > 0 && dn > 0 && dr >= 0 && R > 0, "latent_prep: sizes must be positive");
-    PTA_REQUIRE(q_full && k_pool && q_rows && proj && w_norm && token_pos && token_seq && block_table, "latent_prep: null pointer");
-    PTA_REQUIRE(q_ld >= (long)H * (dn + dr) && ld >= (long)R + dr, "latent_prep: rows lie closer together than they are long");
+    PTA_REQUIRE(q_full && q_rows && token_pos && token_seq && (!write_cache || (k_pool && proj && w_norm && block_table)), "latent_prep: null pointer");
+    PTA_REQUIRE(q_ld >= (long)H * (dn + dr) && (!write_cache || ld >= (long)R + dr), "latent_prep: rows lie closer together than they are long");
     const float* inv_freq = rot ? rot->inv_freq : nullptr;
     int rot_n = 0, pairing = PTA_PAIR_HALF, freq_ld = 0;
     float cs = 1.f;

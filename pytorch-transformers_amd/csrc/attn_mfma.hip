@@ -8,7 +8,8 @@ PTA_ATTN_HEAD(8) PTA_ATTN_HEAD(16)
 #undef PTA_ATTN_HEAD
 
 // out[row, :] = sum_s w_s po[row, s, :] / sum_s w_s pl[row, s], w_s = 2^(pm[row, s] - max_s pm).  A split whose
-// maximum is -inf (a range past the row's keys) has weight zero and is not read.
+// maximum is -inf (a range past the row's keys) has weight zero and is not read.  With `sink` (a number per head; row =
+// token * nh + head) e^sink joins the sum of the weights; the maxima are in units of log 2.
 //
 // A row's splits are many short vectors, and a chain of loads one behind the other is what this kernel's time
 // would be: so LPS lanes (the next power of two from D/4) take one split's vector as float4 each, the 64/LPS
@@ -18,7 +19,7 @@ PTA_ATTN_HEAD(8) PTA_ATTN_HEAD(16)
 template <int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void attn_combine_kernel(bf16_t* __restrict__ out, const float* __restrict__ po,
                                                                   const float* __restrict__ pm, const float* __restrict__ pl,
-                                                                  int D, int n_splits, int lps) {
+                                                                  int D, int n_splits, int lps, const float* __restrict__ sink, int nh) {
     __shared__ float part[WAVES][256 + 4];
     const long row = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -77,6 +78,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_combine_kernel(bf16_t* __rest
         }
     }
     if (g == 0 && active) {
+        if (sink) L += __builtin_amdgcn_exp2f(sink[row % nh] * PTA_LOG2E - mx);
         const float inv = 1.0f / L;
         bf16_t r[4] = {f32_to_bf16_bits(acc.x * inv), f32_to_bf16_bits(acc.y * inv), f32_to_bf16_bits(acc.z * inv),
                        f32_to_bf16_bits(acc.w * inv)};
@@ -85,7 +87,8 @@ __global__ __launch_bounds__(64 * WAVES) void attn_combine_kernel(bf16_t* __rest
 }
 
 extern "C" int pta_attn_combine(void* out, const float* po, const float* pm, const float* pl, long n_rows, int d,
-                                int n_splits, void* stream) {
+                                int n_splits, const float* sink, int nh, void* stream) {
+    PTA_REQUIRE(!sink || nh > 0, "attn_combine: numbers per head need the number of heads");
     PTA_REQUIRE(n_rows > 0 && n_rows <= 0x7fffffffL && d > 0 && d <= 256 && d % 4 == 0 && n_splits >= 1,
                 "attn_combine: %ld rows of %d elements in %d ranges", n_rows, d, n_splits);
     hipStream_t s = (hipStream_t)stream;
@@ -93,9 +96,9 @@ extern "C" int pta_attn_combine(void* out, const float* po, const float* pm, con
     while (lps * 4 < d) lps *= 2;
     const dim3 rows((unsigned)n_rows);
     if (n_splits > 4 * (64 / lps))  // more splits than one wave has in flight at once
-        hipLaunchKernelGGL(attn_combine_kernel<4>, rows, dim3(256), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps);
+        hipLaunchKernelGGL(attn_combine_kernel<4>, rows, dim3(256), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh);
     else
-        hipLaunchKernelGGL(attn_combine_kernel<1>, rows, dim3(64), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps);
+        hipLaunchKernelGGL(attn_combine_kernel<1>, rows, dim3(64), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh);
     return pta_check_launch("attn_combine");
 }
 
@@ -115,7 +118,7 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
                              int bt_stride, const int* cu_tokens, const int* seq_start, const PtaScoreBias* score_bias,
                              int n_seqs, int max_new, int M, int nh, int nkv, int d, float scale, int split_size, int n_splits,
                              float* po, float* pm, float* pl, int window, int chunk, int decode_tiles, int decode_waves,
-                             int prompt_wide, void* stream) {
+                             int prompt_wide, const float* sink, void* stream) {
     PTA_REQUIRE(n_seqs > 0 && max_new > 0 && M > 0 && nh > 0 && nkv > 0, "attn_mfma: sizes must be positive");
     int bias_mode = 0;
     if (pta_score_bias_mode("attn_mfma", score_bias, &bias_mode)) return 1;
@@ -177,7 +180,7 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
                 "attn_mfma: %d waves on the keys of a workgroup with %d column tiles are not built for head size %d "
                 "(one wave, or four or eight with up to two tiles)", decode_waves, dct, d);
     const AttnLaunch a{(bf16_t*)out, po, pm, pl, (const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool,
-                       block_table, bt_stride, cu_tokens, seq_start, slopes, bias_mode, bias_scale, n_seqs, max_new, nh, nkv, scale,
+                       block_table, bt_stride, cu_tokens, seq_start, slopes, bias_mode, bias_scale, sink, n_seqs, max_new, nh, nkv, scale,
                        split_size, n_splits, window, chunk, paired, narrow ? decode_waves : 1, s};
 #define PTA_ATTN_CASE(DT_)                                                                        \
     case DT_: {                                                                                   \
@@ -203,6 +206,6 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
 #undef PTA_ATTN_CASE
     int rc = pta_check_launch("attn_mfma");
     if (rc) return rc;
-    if (n_splits > 1) rc = pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, stream);
+    if (n_splits > 1) rc = pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, sink, nh, stream);
     return rc;
 }

@@ -23,6 +23,9 @@
 // through LDS in the order of the waves; with the whole context in one workgroup there is no second
 // launch, but all of a sequence's keys then pass through one compute unit.  Prefill does not split.
 //
+// `sink` (null: none): a learned number per head whose exponential joins the sum of the weights, once per row, when
+// the row's result is normalised (here without ranges of keys, in the merge with them); it has no key and no value.
+//
 // score = q . k / sqrt(d) + alibi, alibi = bf16(bf16(slope) * bf16(key position)) / sqrt(d)
 // (src/transformers/models/falcon/modeling_falcon.py:371-386, :407-422, :196-198, :1078-1085).
 #pragma once
@@ -116,7 +119,7 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
     const int* __restrict__ block_table, int bt_stride, const int* __restrict__ cu_tokens,
     const int* __restrict__ seq_start, const float* __restrict__ slopes, int bias_mode, int nh, int nkv, float scale,
     float alibi_mul,
-    int split_size, int n_splits, int window_arg, int chunk_arg, int paired) {
+    int split_size, int n_splits, int window_arg, int chunk_arg, int paired, const float* __restrict__ sink) {
     constexpr int D = DT * 16;
     const int window = WIN ? window_arg : 0;
     const int chunk = WIN ? chunk_arg : 0;  // blocks of positions that a token does not see out of (0: none)
@@ -507,6 +510,7 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
                 }
                 const long row = (long)tok[ct] * nh + head[ct];
                 if (n_splits == 1) {
+                    if (sink) l += __builtin_amdgcn_exp2f(sink[head[ct]] * PTA_LOG2E - mx);
                     const float inv = 1.0f / l;
                     uint2 w2;
                     w2.x = pack_bf16(acc.x * inv, acc.y * inv);
@@ -524,10 +528,11 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
     } else {
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
-        const float l = lacc[ct][0];
+        float l = lacc[ct][0];
         if (qpos[ct] < 0) continue;
         const long row = (long)tok[ct] * nh + head[ct];
         if (n_splits == 1) {
+            if (sink) l += __builtin_amdgcn_exp2f(sink[head[ct]] * PTA_LOG2E - m_run[ct]);
             const float inv = 1.0f / l;
             bf16_t* o = out + row * D;
 #pragma unroll
@@ -562,7 +567,7 @@ struct AttnLaunch {
     bf16_t* out; float *po, *pm, *pl;
     const bf16_t *q, *k_pool, *v_pool;
     const int* block_table; int bt_stride;
-    const int *cu_tokens, *seq_start; const float* slopes; int bias_mode; float bias_scale;
+    const int *cu_tokens, *seq_start; const float* slopes; int bias_mode; float bias_scale; const float* sink;
     int n_seqs, max_new, nh, nkv; float scale;
     int split_size, n_splits, window;
     int chunk;   // 0, or the size of the blocks of positions that a token does not see out of
@@ -597,7 +602,7 @@ static void launch_attn(const AttnLaunch& a) {
     }
     hipLaunchKernelGGL(kern, grid, dim3(64 * W * KS), lds, a.s, a.out, a.po, a.pm, a.pl, a.q, a.k_pool, a.v_pool,
                        a.block_table, a.bt_stride, a.cu_tokens, a.seq_start, a.slopes, a.bias_mode, a.nh, a.nkv,
-                       a.scale * PTA_LOG2E, PTA_LOG2E * a.bias_scale, a.split_size, a.n_splits, a.window, a.chunk, paired);
+                       a.scale * PTA_LOG2E, PTA_LOG2E * a.bias_scale, a.split_size, a.n_splits, a.window, a.chunk, paired, a.sink);
 }
 
 // column tiles (of sixteen query heads of one KV head) that one wave of a decode launch holds at most:

@@ -8,7 +8,10 @@
 //                   an = 1/2 + softplus(act[1]), act two learned numbers held in 32-bit.
 // pta_glu:          out[m, f] = act(gate[m, f], up[m, f]) for a feed-forward with a gate:
 //                   PTA_GLU_SILU        silu(gate) * up
+//                   PTA_GLU_GELU_TANH   gelu_tanh(gate) * up
 //                   PTA_GLU_CLAMPED     g = min(gate, limit), u = clamp(up, -limit, limit): g * sigmoid(alpha g) * (u + 1)
+// pta_head_norm_gate: out[m, h * dv + e] = x / sqrt(mean over the head's dv elements (x^2) + eps) * w[e] * sigmoid(g),
+//                   every head by its own root mean square, one weight [dv] for all heads.
 // Arithmetic in 32-bit, results in the compute type.
 #include "common.h"
 #include "pta_kernels.h"
@@ -74,21 +77,47 @@ __global__ void glu_kernel(T* __restrict__ out, const T* __restrict__ gate, cons
         g = fminf(g, limit);
         u = fminf(fmaxf(u, -limit), limit);
         y = g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+    } else if (kind == PTA_GLU_GELU_TANH) {
+        y = apply_act(g, PTA_ACT_GELU_TANH) * u;
     } else {
         y = g / (1.0f + expf(-g)) * u;
     }
     Io<T>::st(out + i, y);
 }
 
+// bfloat16 rows of a multiple of eight elements at sixteen-byte addresses: eight elements a thread
+__global__ void glu_gelu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
+                                       long in_ld, int F8, long n8) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n8) return;
+    const long m = i / F8, f = (i - m * F8) * 8;
+    float g[8], u[8];
+    unpack8(*reinterpret_cast<const uint4*>(gate + m * in_ld + f), g);
+    unpack8(*reinterpret_cast<const uint4*>(up + m * in_ld + f), u);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+        // tanh(z) = 1 - 2 / (1 + e^(2z)): both ends saturate without a branch (e^(2z) to infinity or to zero)
+        const float z = 0.79788456080286535588f * (g[j] + 0.044715f * g[j] * g[j] * g[j]);
+        g[j] = g[j] * (1.0f - 1.0f / (1.0f + __expf(2.0f * z))) * u[j];
+    }
+    *reinterpret_cast<uint4*>(out + i * 8) = pack8(g);
+}
+
 // gate, up: [M, F] with rows in_ld apart (the two halves of one product's rows); out [M, F] dense
 extern "C" int pta_glu(void* out, const void* gate, const void* up, long in_ld, int M, int F, int kind, float alpha,
                        float limit, int dtype, void* stream) {
     PTA_REQUIRE(M > 0 && F > 0 && out && gate && up && in_ld >= F, "glu: sizes must be positive and pointers given");
-    PTA_REQUIRE(kind == PTA_GLU_SILU || kind == PTA_GLU_CLAMPED, "glu: kind %d is not built", kind);
+    PTA_REQUIRE(kind == PTA_GLU_SILU || kind == PTA_GLU_CLAMPED || kind == PTA_GLU_GELU_TANH, "glu: kind %d is not built", kind);
     PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "glu: unknown dtype %d", dtype);
     hipStream_t s = (hipStream_t)stream;
     const long n = (long)M * F;
     const dim3 grid((unsigned)((n + 255) / 256));
+    if (dtype == PTA_BF16 && kind == PTA_GLU_GELU_TANH && F % 8 == 0 && in_ld % 8 == 0 && ((uintptr_t)gate % 16) == 0 &&
+        ((uintptr_t)up % 16) == 0 && ((uintptr_t)out % 16) == 0) {
+        hipLaunchKernelGGL(glu_gelu_bf16x8_kernel, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0, s, (bf16_t*)out,
+                           (const bf16_t*)gate, (const bf16_t*)up, in_ld, F / 8, n / 8);
+        return pta_check_launch("glu");
+    }
     if (dtype == PTA_F32)
         hipLaunchKernelGGL(glu_kernel<float>, grid, dim3(256), 0, s, (float*)out, (const float*)gate, (const float*)up, in_ld, F, n, kind, alpha, limit);
     else
@@ -229,4 +258,39 @@ extern "C" int pta_polynorm(void* out, const void* z, long z_ld, const float* co
     else
         return pta_fail("polynorm: unknown dtype %d", dtype);
     return pta_check_launch("polynorm");
+}
+
+// one wave per (token, head)
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ x, const T* __restrict__ g,
+                                                             long g_ld, const float* __restrict__ w, float eps, long units,
+                                                             int heads, int dv) {
+    const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (unit >= units) return;
+    const int lane = threadIdx.x & 63;
+    const long m = unit / heads, h = unit - m * heads;
+    const float* xr = x + unit * dv;
+    const T* gr = g + m * g_ld + h * dv;
+    float ss = 0.f;
+    for (int e = lane; e < dv; e += PTA_WAVE) ss += xr[e] * xr[e];
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
+    for (int e = lane; e < dv; e += PTA_WAVE)
+        Io<T>::st(out + unit * dv + e, xr[e] * inv * w[e] / (1.0f + expf(-Io<T>::ld(gr + e))));
+}
+
+// x [M, heads * dv] 32-bit, dense; g [M, heads * dv] rows g_ld apart, out dense, both in the compute type; w [dv]
+extern "C" int pta_head_norm_gate(void* out, const float* x, const void* g, long g_ld, const float* w, float eps, int M,
+                                  int heads, int dv, int dtype, void* stream) {
+    PTA_REQUIRE(M > 0 && heads > 0 && dv > 0, "head_norm_gate: sizes must be positive");
+    PTA_REQUIRE(out && x && g && w, "head_norm_gate: null pointer");
+    PTA_REQUIRE(g_ld >= (long)heads * dv, "head_norm_gate: rows of the gate lie closer together than they are long");
+    PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "head_norm_gate: unknown dtype %d", dtype);
+    hipStream_t s = (hipStream_t)stream;
+    const long units = (long)M * heads;
+    const dim3 grid((unsigned)((units + 3) / 4));
+    if (dtype == PTA_F32)
+        hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, s, (float*)out, x, (const float*)g, g_ld, w, eps, units, heads, dv);
+    else
+        hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, s, (bf16_t*)out, x, (const bf16_t*)g, g_ld, w, eps, units, heads, dv);
+    return pta_check_launch("head_norm_gate");
 }

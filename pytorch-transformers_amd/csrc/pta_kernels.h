@@ -14,7 +14,7 @@
 
 #include <stdint.h>
 
-#define PTA_ABI_VERSION 14
+#define PTA_ABI_VERSION 15
 
 #ifdef __cplusplus
 extern "C" {
@@ -88,10 +88,11 @@ int pta_attention_sizes_ok(int nh, int nkv, int d, int rotated);
 // chunk: 0, or the size of the blocks of positions, counted from the sequence's start, that a token does not see out
 // of: position i sees j <= i only if floor(i / chunk) == floor(j / chunk)
 // score_bias (null: none): see PtaScoreBias above; with bf16 = 1 the slopes given are expected rounded to bfloat16 too
+// sink (null: none): a 32-bit number per head; its exponential joins the sum that the head's weights are divided by
 int pta_attn_generic(void* out, const void* q, const void* k_pool, const void* v_pool, const int* block_table,
                      int bt_stride, const int* token_seq, const int* token_pos, const PtaScoreBias* score_bias,
                      int M, int nh,
-                     int nkv, int d, float scale, int window, int chunk, int dtype, void* stream);
+                     int nkv, int d, float scale, int window, int chunk, const float* sink, int dtype, void* stream);
 
 // the same attention for bfloat16 on the matrix cores; cu_tokens [n_seqs + 1] and seq_start [n_seqs] say
 // which tokens are whose and how long each sequence was before the step; max_new bounds a sequence's new
@@ -115,7 +116,7 @@ int pta_attn_mfma(void* out, const void* q, const void* k_pool, const void* v_po
                   int bt_stride, const int* cu_tokens, const int* seq_start, const PtaScoreBias* score_bias,
                   int n_seqs, int max_new, int M, int nh, int nkv, int d, float scale, int split_size, int n_splits, float* po,
                   float* pm, float* pl, int window, int chunk, int decode_tiles, int decode_waves, int prompt_wide,
-                  void* stream);
+                  const float* sink, void* stream);
 
 // C = act(A . W^T + bias) + add1 + add2, all 32-bit, fixed summation order
 int pta_gemm_f32(float* C, const float* A, const float* W, const float* bias, const float* add1, const float* add2,
@@ -297,7 +298,7 @@ int pta_head_norm_rope_cache(void* q_out, const void* q_in, const void* k_in, co
                              int dtype, void* stream);
 
 // ---- gates between two products (gated.hip) ---------------------------------------------------------------------------
-enum PtaGlu { PTA_GLU_SILU = 0, PTA_GLU_CLAMPED = 1 };
+enum PtaGlu { PTA_GLU_SILU = 0, PTA_GLU_CLAMPED = 1, PTA_GLU_GELU_TANH = 2 };
 // How an expert's gate and up products meet: kind PTA_GLU_SILU is act(g) * u with the launch's activation; kind
 // PTA_GLU_CLAMPED is, with g' = min(g, limit) and u' = clamp(u, -limit, limit), g' * sigmoid(alpha g') * (u' + 1).
 typedef struct PtaGate {
@@ -314,6 +315,34 @@ int pta_gated_heads(void* out, const void* x, int x_f32, long x_ld, int x_head, 
 int pta_xielu(void* out, const void* z, long z_ld, int M, int F, const float* act, int dtype, void* stream);
 int pta_glu(void* out, const void* gate, const void* up, long in_ld, int M, int F, int kind, float alpha, float limit,
             int dtype, void* stream);
+
+// every head of x [M, heads * dv] (32-bit) over its own root mean square, times w [dv], times sigmoid(g)
+int pta_head_norm_gate(void* out, const float* x, const void* g, long g_ld, const float* w, float eps, int M, int heads, int dv,
+                       int dtype, void* stream);
+
+// ---- several residual streams (hyper_stream.hip) -----------------------------------------------------------------------
+// New streams from the old ones and a sublayer's result y, their sum weighted by `in` (null: the plain sum), its RMS norm,
+// and a causal convolution on that; every output may be null.  x: row m, stream s at x + m * x_row + s * x_stream
+// (x_stream 0: all streams are that one vector).  conv [taps, H] with the sequences' tails (rows tail_ld apart, found
+// through seq_slot[token_seq[m]]) is for steps in which every sequence brings one token.
+int pta_hyper_norm(void* h, float* n_out, float* u_out, float* x_out, const float* x, long x_row, long x_stream, const void* y,
+                   long y_ld, const float* mix, const float* out, const float* in, const float* w, float offset, float eps,
+                   const int* rows, const float* conv, int taps, float* tail, long tail_ld, const int* token_seq,
+                   const int* seq_slot, int M, int H, int streams, int dtype, void* stream);
+// out = in + a causal convolution of in (32-bit, [M, C]) per channel, w [K, C]; the tails are moved on (recurrent.hip)
+int pta_conv_add(void* out, const float* in, const float* w, float* tail, long tail_ld, const int* cu_tokens,
+                 const int* token_seq, const int* seq_slot, int n_seqs, int M, int C, int K, int dtype, void* stream);
+int pta_conv_tail(const void* in, long ld, float* tail, long tail_ld, const int* cu_tokens, const int* seq_slot, int n_seqs,
+                  int C, int K, int dtype, void* stream);
+
+// ---- the gated delta rule with a decay per key channel (delta.hip) ---------------------------------------------------------
+int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, const void* k, const void* v, long ld, const float* conv,
+                   const void* a, long a_ld, const void* b, long b_ld, const float* A_log, const float* dt_bias, float* tail,
+                   long tail_ld, const int* cu_tokens, const int* token_seq, const int* seq_slot, int several, int n_seqs, int M,
+                   int heads, int kv_heads, int N, int P, int taps, float q_scale, float norm_eps, int dtype, void* stream);
+int pta_delta_scan(float* y, const float* qkv, const float* g, const float* beta, float* state, long state_ld, float* chunk_state,
+                   const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int heads, int kv_heads, int P, int N,
+                   int chunk, int max_chunks, void* stream);
 
 // ---- linear attention with a decay per head (linear_attn.hip) ---------------------------------------------------------
 int pta_decay_scan(float* y, const void* q, const void* k, const void* v, long ld, const float* decay, float* state,
@@ -366,7 +395,7 @@ int pta_attn_talk_mfma(void* out, const void* q, const void* k_pool, const void*
 // Merge of the partial results of ranges of keys (attn_mfma.hip): out[row] = sum_s w_s po[row, s] / sum_s w_s pl[row, s],
 // w_s = 2^(pm[row, s] - max_s pm); a range whose pm is -inf is not read.
 int pta_attn_combine(void* out, const float* po, const float* pm, const float* pl, long rows, int d, int n_splits,
-                     void* stream);
+                     const float* sink, int nh, void* stream);
 
 #ifdef __cplusplus
 }

@@ -195,6 +195,75 @@ extern "C" int pta_conv_silu(float* out, const void* in, long ld, const float* w
     return pta_check_launch("conv_silu");
 }
 
+// A sequence's tail moved on by the step's inputs on its own, for launches that form the convolution themselves.
+extern "C" int pta_conv_tail(const void* in, long ld, float* tail, long tail_ld, const int* cu_tokens, const int* seq_slot,
+                             int n_seqs, int C, int K, int dtype, void* stream) {
+    PTA_REQUIRE(n_seqs > 0 && n_seqs <= 65535 && C > 0, "conv_tail: sequences=%d channels=%d", n_seqs, C);
+    PTA_REQUIRE(K >= 2 && K <= PTA_CONV_MAX_TAPS, "conv_tail: %d taps are outside 2..%d", K, PTA_CONV_MAX_TAPS);
+    PTA_REQUIRE(in && tail && cu_tokens && seq_slot, "conv_tail: null pointer");
+    PTA_REQUIRE(ld >= C && tail_ld >= (long)(K - 1) * C, "conv_tail: rows lie closer together than they are long");
+    PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "conv_tail: unknown dtype %d", dtype);
+    const dim3 block(C >= 256 ? 256 : 64), grid((C + block.x - 1) / block.x, n_seqs);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == PTA_F32)
+        hipLaunchKernelGGL(conv_tail_kernel<float>, grid, block, 0, s, (const float*)in, ld, tail, tail_ld, cu_tokens, seq_slot, C, K);
+    else
+        hipLaunchKernelGGL(conv_tail_kernel<bf16_t>, grid, block, 0, s, (const bf16_t*)in, ld, tail, tail_ld, cu_tokens, seq_slot, C, K);
+    return pta_check_launch("conv_tail");
+}
+
+// out[t, c] = in[t, c] + sum_k w[k, c] * in[t - (K - 1 - k), c], in and the tail in 32-bit, out in the compute type: an input
+// convolution that adds to what it reads.  Neighbouring threads take neighbouring channels, each CONV_ADD_TOKENS tokens.
+#define CONV_ADD_TOKENS 4
+
+template <typename T>
+__global__ void conv_add_kernel(T* __restrict__ out, const float* __restrict__ in, const float* __restrict__ w,
+                                const float* __restrict__ tail, long tail_ld, const int* __restrict__ cu_tokens,
+                                const int* __restrict__ token_seq, const int* __restrict__ seq_slot, int M, int C, int K) {
+    const int c = blockIdx.y * blockDim.x + threadIdx.x;
+    if (c >= C) return;
+    float wk[PTA_CONV_MAX_TAPS];
+#pragma unroll
+    for (int k = 0; k < PTA_CONV_MAX_TAPS; ++k) wk[k] = k < K ? w[(long)k * C + c] : 0.f;
+    for (int t = 0; t < CONV_ADD_TOKENS; ++t) {
+        const int m = blockIdx.x * CONV_ADD_TOKENS + t;
+        if (m >= M) return;
+        const int s = token_seq[m], first = cu_tokens[s], j = m - first;
+        const float* tl = tail + (K > 1 ? (long)seq_slot[s] * tail_ld : 0L);
+        const float now = in[(long)m * C + c];
+        float acc = 0.f;
+#pragma unroll
+        for (int k = 0; k < PTA_CONV_MAX_TAPS; ++k) {
+            if (k + 1 < K) {
+                const int jj = j - (K - 1 - k);
+                acc += wk[k] * (jj >= 0 ? in[(long)(first + jj) * C + c] : tl[(long)(K - 1 + jj) * C + c]);
+            }
+            if (k + 1 == K) acc += wk[k] * now;
+        }
+        Io<T>::st(out + (long)m * C + c, now + acc);
+    }
+}
+
+extern "C" int pta_conv_add(void* out, const float* in, const float* w, float* tail, long tail_ld, const int* cu_tokens,
+                            const int* token_seq, const int* seq_slot, int n_seqs, int M, int C, int K, int dtype, void* stream) {
+    PTA_REQUIRE(M > 0 && n_seqs > 0 && C > 0, "conv_add: tokens=%d sequences=%d channels=%d must be positive", M, n_seqs, C);
+    PTA_REQUIRE(K >= 1 && K <= PTA_CONV_MAX_TAPS, "conv_add: %d taps are outside 1..%d", K, PTA_CONV_MAX_TAPS);
+    PTA_REQUIRE(out && in && w && (tail || K == 1) && cu_tokens && token_seq && seq_slot, "conv_add: null pointer");
+    PTA_REQUIRE(K == 1 || tail_ld >= (long)(K - 1) * C, "conv_add: rows of the tail lie closer together than they are long");
+    PTA_REQUIRE(n_seqs <= 65535 && C <= 65535 * 64, "conv_add: too many sequences or channels for one launch");
+    PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "conv_add: unknown dtype %d", dtype);
+    hipStream_t s = (hipStream_t)stream;
+    const dim3 block(C >= 256 ? 256 : 64), grid((M + CONV_ADD_TOKENS - 1) / CONV_ADD_TOKENS, (C + block.x - 1) / block.x);
+    if (dtype == PTA_F32)
+        hipLaunchKernelGGL(conv_add_kernel<float>, grid, block, 0, s, (float*)out, in, w, tail, tail_ld, cu_tokens, token_seq,
+                           seq_slot, M, C, K);
+    else
+        hipLaunchKernelGGL(conv_add_kernel<bf16_t>, grid, block, 0, s, (bf16_t*)out, in, w, tail, tail_ld, cu_tokens, token_seq,
+                           seq_slot, M, C, K);
+    if (K > 1) return pta_conv_tail(in, C, tail, tail_ld, cu_tokens, seq_slot, n_seqs, C, K, PTA_F32, stream);
+    return pta_check_launch("conv_add");
+}
+
 // ---- a state-space recurrence with a scalar decay per head --------------------------------------------------
 // Per head h (of group g = h / (heads / groups)), with state S [N, P]:
 //   dt = softplus(dt_raw + dt_bias[h]);  S = exp(-exp(A_log[h]) dt) S + dt B_t x_t^T;  y_t = S^T C_t + D[h] x_t

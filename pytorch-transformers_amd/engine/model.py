@@ -24,7 +24,7 @@ from .. import host, ops, tuning
 from ..cache.paged import PagedCache
 from ..config.registry import AutoConfig, lookup
 from ..parts.base import ResidualSum, StepContext, WideResidual, as_tensor
-from ..weights.loader import load_weights
+from ..weights.loader import load_weights, tensor_shapes
 from ..weights.random_init import random_tensors
 from .spec import ModelSpec
 from .step import StepError, StepPlan, Want, plan_step
@@ -265,6 +265,7 @@ class CausalLM:
 
         device = _require_gpu(device)
         config = AutoConfig.from_pretrained(folder)
+        config.sizes_from_weights(tensor_shapes(folder))
         dtype = auto_dtype(config, folder) if dtype == "auto" else resolve_dtype(dtype)
         _, builder = lookup(config.model_type)
         spec = builder(config)

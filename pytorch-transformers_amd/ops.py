@@ -24,7 +24,7 @@ QKV_LAYOUT_CODES = {"grouped": 0, "tail": 1, "interleaved": 2}
 ACT_CODES = {None: 0, "none": 0, "linear": 0, "gelu": 1, "gelu_python": 1, "gelu_new": 2, "gelu_pytorch_tanh": 2,
              "gelu_fast": 2, "gelu_accurate": 2, "quick_gelu": 3, "relu": 4, "relu2": 5, "relu6": 6, "silu": 7, "swish": 7,
              "sigmoid": 8, "tanh": 9, "leaky_relu": 10, "mish": 11, "gelu_10": 12, "laplace": 13}
-ABI_VERSION = 14
+ABI_VERSION = 15
 PAIRING_CODES = {"half": 0, "interleaved": 1}  # PtaPairing: elements (i, i + rotary_dim / 2) or (2i, 2i + 1)
 BIAS_OF_CODES = {"key": 0, "distance": 1}  # PtaBiasOf: the slope times the key's position, or times key - query position
 
@@ -215,6 +215,22 @@ def _entry_cost(name: str, a) -> tuple:
         return (M * N * ((4.0 if a[2] else e) + 2 * e), 0.0)
     if name == "pta_xielu":
         return (float(a[3]) * a[4] * 2 * el(a[6]), 0.0)
+    if name == "pta_head_norm_gate":
+        return (float(a[6]) * a[7] * a[8] * (4.0 + 2 * el(a[9])), 0.0)
+    if name == "pta_hyper_norm":  # the streams in and out (32-bit), a sublayer's result in, the norm out (and 32-bit copies)
+        M, H, S, e = float(a[22]), float(a[23]), float(a[24]), el(a[25])
+        taps = (a[17] - 1) * 8.0 + 4.0 if given(16) else 0.0
+        read = 4.0 * (S if getattr(a[6], "value", a[6]) else 1.0)
+        return (M * H * (read + given(3) * S * 4.0 + (given(7) + given(0)) * e + (given(1) + given(2)) * 4.0 + taps), 0.0)
+    if name == "pta_conv_add":
+        return (float(a[9]) * a[10] * (4.0 + el(a[12])), 0.0)
+    if name == "pta_delta_prep":  # q, k, v, decays in (compute type) and out (32-bit)
+        M, heads, G, N, P = float(a[21]), a[22], a[23], a[24], a[25]
+        return (M * (2 * G * N + heads * (P + N)) * (el(a[29]) + 4.0), 0.0)
+    if name == "pta_delta_scan":  # q, k, v, g in, o out, all 32-bit; seven operations per state element and token
+        M, heads, G, P, N = float(timing_hint.get("rows", 0)), a[11], a[12], a[13], a[14]
+        state = 8.0 * a[9] * heads * N * P
+        return (M * (2 * G * N + heads * (2 * P + N)) * 4.0 + state, 7.0 * M * heads * N * P)
     if name == "pta_glu":
         return (float(a[4]) * a[5] * 3 * el(a[9]), 0.0)
     if name == "pta_decay_scan":  # q, k, v in, o out in 32-bit; two multiply-adds per state element and token
@@ -534,13 +550,16 @@ def attention_sizes_problem(nh: int, nkv: int, d: int, rotated: bool) -> Optiona
 
 def attn_generic(q: torch.Tensor, k_pool, v_pool, block_table, token_seq, token_pos, slopes, scale: float,
                  window: int = 0, alibi_exact: bool = False, bias_of: str = "key", bias_scale: Optional[float] = None,
-                 chunk: int = 0):
+                 chunk: int = 0, sink: Optional[torch.Tensor] = None):
     """Causal attention of every token over its sequence's cache (the last ``window`` positions of it, itself
     included, if ``window`` > 0; the positions of its own block of ``chunk``, counted from the sequence's start, if
     ``chunk`` > 0); out [M, nh*d].  ``slopes`` (None: no bias), ``bias_of``, ``alibi_exact`` (no
     rounding to bfloat16) and ``bias_scale`` (None: 1 / sqrt(head size), as the reference folds its bias into the
-    mask) describe a bias on the scores (``_score_bias_arg``)."""
+    mask) describe a bias on the scores (``_score_bias_arg``).  ``sink`` (``[nh]`` 32-bit): ``exp(sink[h])`` joins the
+    sum that head h's weights are divided by."""
     _need(q, "q")
+    if sink is not None:
+        _need(sink, "sink", torch.float32, (q.shape[1],))
     M, nh, d = q.shape
     nkv = k_pool.shape[1]
     _need_pools(k_pool, v_pool, q.dtype, nkv, d)
@@ -551,7 +570,7 @@ def attn_generic(q: torch.Tensor, k_pool, v_pool, block_table, token_seq, token_
     out = torch.empty((M, nh * d), dtype=q.dtype, device=q.device)
     _call("pta_attn_generic", _ptr(out), _ptr(q), _ptr(k_pool), _ptr(v_pool), _ptr(block_table),
           block_table.shape[1], _ptr(token_seq), _ptr(token_pos), bias, M, nh, nkv, d,
-          ctypes.c_float(scale), int(window), int(chunk), dtype_code(q.dtype), _stream())
+          ctypes.c_float(scale), int(window), int(chunk), _ptr(sink), dtype_code(q.dtype), _stream())
     return out
 
 
@@ -643,7 +662,7 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
               max_new: int, n_splits: int = 1, split_size: int = ATTN_SPLIT_KEYS, window: int = 0,
               decode_tiles: int = 0, decode_waves: int = 1, alibi_exact: bool = False,
               prompt_wide: Optional[bool] = None, bias_of: str = "key", bias_scale: Optional[float] = None,
-              chunk: int = 0) -> torch.Tensor:
+              chunk: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of a step's tokens over the cache on the matrix cores; out [M, nh*d].
 
     ``max_new`` bounds the new tokens of any sequence of the step; with ``n_splits > 1`` the keys
@@ -653,9 +672,11 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
     them, or ``SHARED_KEYS``: the heads of a KV head on the waves of one workgroup, which share its keys through
     LDS (``attn_decode_shared_ok``).  ``prompt_wide``: workgroups of eight waves (True) or four (False) for prompts
     with heads up to 64 (None: eight where the launch has workgroups enough).  ``slopes``, ``alibi_exact``,
-    ``bias_of`` and ``bias_scale``: the bias on the scores, as in ``attn_generic``."""
+    ``bias_of`` and ``bias_scale``: the bias on the scores, and ``sink``, as in ``attn_generic``."""
     _need(q, "q", torch.bfloat16)
     M, nh, d = q.shape
+    if sink is not None:
+        _need(sink, "sink", torch.float32, (nh,))
     nkv = k_pool.shape[1]
     _need_pools(k_pool, v_pool, q.dtype, nkv, d)
     _need(block_table, "block_table", torch.int32)
@@ -673,14 +694,14 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
           _ptr(cu_tokens), _ptr(seq_start), bias, n_seqs, int(max_new), M, nh, nkv, d,
           ctypes.c_float(scale),
           int(split_size), int(n_splits), _ptr(po), _ptr(pm), _ptr(pl), int(window), int(chunk), int(decode_tiles), int(decode_waves),
-          ATTN_FORCE_WIDE if prompt_wide is None else int(bool(prompt_wide)), _stream())
+          ATTN_FORCE_WIDE if prompt_wide is None else int(bool(prompt_wide)), _ptr(sink), _stream())
     return out
 
 
 
 def attention(q: torch.Tensor, k_pool, v_pool, block_table, ctx, slopes, scale: float, window: int = 0,
               alibi_exact: bool = False, bias_of: str = "key", bias_scale: Optional[float] = None,
-              chunk: int = 0) -> torch.Tensor:
+              chunk: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of a step's tokens over the cache: picks the kernel for the step's shape and type.
     ``chunk`` > 0: a token sees the keys of its own block of so many positions only (``attn_generic``).
 
@@ -698,9 +719,9 @@ def attention(q: torch.Tensor, k_pool, v_pool, block_table, ctx, slopes, scale: 
         return attn_mfma(q, k_pool, v_pool, block_table, ctx.cu_tokens, ctx.seq_start, slopes, scale,
                          max_new=max(ctx.new_tokens), n_splits=n_splits, split_size=size, window=window,
                          decode_tiles=tiles, decode_waves=waves, alibi_exact=alibi_exact, bias_of=bias_of,
-                         bias_scale=bias_scale, chunk=chunk)
+                         bias_scale=bias_scale, chunk=chunk, sink=sink)
     return attn_generic(q, k_pool, v_pool, block_table, ctx.token_seq, ctx.token_pos, slopes, scale, window, alibi_exact,
-                        bias_of, bias_scale, chunk)
+                        bias_of, bias_scale, chunk, sink)
 
 
 def attn_talk_mfma_ok(q: torch.Tensor, nkv: int, mixed: bool = True) -> bool:
@@ -1510,38 +1531,45 @@ def latent_sizes_problem(heads: int, dim: int, rot_dim: int, rank: int) -> Optio
     return lib.pta_last_error().decode("utf-8", "replace")
 
 
-def latent_prep(proj: torch.Tensor, w_norm: torch.Tensor, eps: float, inv_freq, cs_scale: float, rotary_dim, pairing: str,
+def latent_prep(proj: Optional[torch.Tensor], w_norm: Optional[torch.Tensor], eps: float, inv_freq, cs_scale: float, rotary_dim, pairing: str,
                 token_pos, token_seq, block_table, k_pool, heads: int, dim: int, rot_dim: int, rank: int,
                 write_cache: bool = True, q: Optional[torch.Tensor] = None) -> torch.Tensor:
     """From ``proj`` ``[tokens, heads * (dim + rot_dim) + rank + rot_dim]`` (the queries, then the down-projection), or
     with the queries ``q`` ``[tokens, heads * (dim + rot_dim)]`` given apart from ``proj`` ``[tokens, rank + rot_dim]``
     (each may be a block of columns): the normed latent and the rotated shared key part go into the token's cache row
     ``[rank + rot_dim]``; returns the queries' frame ``[tokens, heads, rank + rot_dim]`` in 32-bit with the rotated
-    parts filled in (the first ``rank`` of each head are for ``head_project``)."""
-    M = proj.shape[0]
+    parts filled in (the first ``rank`` of each head are for ``head_project``).  ``write_cache`` False with ``q`` given:
+    the queries alone (``proj`` and ``w_norm`` None), for a layer that reads rows another layer has written."""
+    M = (q if proj is None else proj).shape[0]
     q_cols = heads * (dim + rot_dim)
     if q is None:
         ld = _rows_of(proj, "proj", q_cols + rank + rot_dim)
         q_ptr, q_ld, down_ptr = proj.data_ptr(), ld, proj.data_ptr() + q_cols * proj.element_size()
+    elif proj is None:
+        if write_cache:
+            raise KernelError("a cache row is made from a down-projection")
+        ld, down_ptr, q_ld, q_ptr = 0, 0, _rows_of(q, "q", q_cols), q.data_ptr()
     else:
         ld = _rows_of(proj, "proj", rank + rot_dim)
         q_ld = _rows_of(q, "q", q_cols, proj.dtype)
         q_ptr, down_ptr = q.data_ptr(), proj.data_ptr()
-    _need(w_norm, "w_norm", torch.float32, (rank,))
+    ref = q if proj is None else proj
+    if write_cache:
+        _need(w_norm, "w_norm", torch.float32, (rank,))
     _need(token_pos, "token_pos", torch.int32, (M,))
     _need(token_seq, "token_seq", torch.int32, (M,))
     _need(block_table, "block_table", torch.int32)
     D = rank + rot_dim
-    _need(k_pool, "k_pool", proj.dtype)
+    _need(k_pool, "k_pool", ref.dtype)
     if k_pool.dim() != 4 or tuple(k_pool.shape[1:]) != (1, 64, D):
         raise KernelError(f"k_pool must be [pages, 1, 64, {D}], got {tuple(k_pool.shape)}")
     rot = _rotation_arg(inv_freq, cs_scale, rot_dim, block_table.shape[0], rotary_dim, pairing) if rot_dim else None
-    q_full = torch.empty((M, heads, D), dtype=torch.float32, device=proj.device)
+    q_full = torch.empty((M, heads, D), dtype=torch.float32, device=ref.device)
     if M:
         _call("pta_latent_prep", _ptr(q_full), _ptr(k_pool), ctypes.c_void_p(q_ptr), ctypes.c_long(q_ld),
               ctypes.c_void_p(down_ptr), ctypes.c_long(ld), _ptr(w_norm),
               ctypes.c_float(eps), rot, _ptr(token_pos), _ptr(token_seq), _ptr(block_table), block_table.shape[1], M,
-              heads, dim, rot_dim, rank, int(write_cache), dtype_code(proj.dtype), _stream())
+              heads, dim, rot_dim, rank, int(write_cache), dtype_code(ref.dtype), _stream())
     return q_full
 
 
@@ -1716,7 +1744,7 @@ def head_norm_rope_cache(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Ten
 
 
 # ---- gates between two products -------------------------------------------------------------------------------------
-GLU_CODES = {"silu": 0, "clamped": 1}
+GLU_CODES = {"silu": 0, "clamped": 1, "gelu_tanh": 2}
 
 
 def gated_heads(x: torch.Tensor, x_head: int, g: torch.Tensor, heads: int, dv: int, dtype: torch.dtype,
@@ -1752,7 +1780,7 @@ def xielu(z: torch.Tensor, act: torch.Tensor) -> torch.Tensor:
 
 
 def glu(gate: torch.Tensor, up: torch.Tensor, kind: str = "silu", alpha: float = 1.0, limit: float = 0.0) -> torch.Tensor:
-    """``silu(gate) * up`` (``"silu"``), or with ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``:
+    """``silu(gate) * up`` (``"silu"``), ``gelu_tanh(gate) * up`` (``"gelu_tanh"``), or with ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``:
     ``g * sigmoid(alpha * g) * (u + 1)`` (``"clamped"``); gate and up are blocks of columns of one product."""
     M, F = gate.shape
     ld = _rows_of(gate, "gate", F)
@@ -1763,6 +1791,174 @@ def glu(gate: torch.Tensor, up: torch.Tensor, kind: str = "silu", alpha: float =
         _call("pta_glu", _ptr(out), _ptr(gate), _ptr(up), ctypes.c_long(ld), M, F, GLU_CODES[kind], ctypes.c_float(alpha),
               ctypes.c_float(limit), dtype_code(gate.dtype), _stream())
     return out
+
+
+def head_norm_gate(x: torch.Tensor, g: torch.Tensor, w: torch.Tensor, eps: float, heads: int, dv: int,
+                   dtype: torch.dtype) -> torch.Tensor:
+    """``x / sqrt(mean over a head's elements (x^2) + eps) * w * sigmoid(g)`` ``[M, heads * dv]`` in ``dtype``: ``x``
+    ``[M, heads * dv]`` 32-bit, every head by its own root mean square, ``w`` ``[dv]`` for all of them; ``g`` ``[M, heads
+    * dv]`` (``dtype``) may be a block of columns."""
+    M = x.shape[0]
+    _need(x, "x", torch.float32, (M, heads * dv))
+    _need(w, "w", torch.float32, (dv,))
+    g_ld = _rows_of(g, "g", heads * dv, dtype)
+    if g.shape[0] != M:
+        raise KernelError("gate and x differ in their number of rows")
+    out = torch.empty((M, heads * dv), dtype=dtype, device=x.device)
+    if M:
+        _call("pta_head_norm_gate", _ptr(out), _ptr(x), _ptr(g), ctypes.c_long(g_ld), _ptr(w), ctypes.c_float(eps), M, heads, dv,
+              dtype_code(dtype), _stream())
+    return out
+
+
+# ---- several residual streams ---------------------------------------------------------------------------------------
+HYPER_MAX_STREAMS = 8
+
+
+def hyper_norm(x: torch.Tensor, streams: int, dtype: torch.dtype, *, y: Optional[torch.Tensor] = None, mix=None, out=None,
+               weights=None, norm=None, rows=None, want_x: bool = False, want_u: bool = False, want_n: bool = False,
+               want_h: bool = False, conv=None, ctx=None):
+    """One pass over ``streams`` residual streams in 32-bit: ``x`` ``[M, streams, H]``, or ``[M, H]`` where all of them are
+    that one.  With ``y`` (a sublayer's result in ``dtype``, rows may lie apart) the new streams are ``x_t <- sum_s mix[s, t]
+    x_s + out[t] y``; ``u = sum_t weights[t] x_t`` (None: the plain sum); ``n`` is u's RMS norm with ``norm = (weight,
+    offset, eps)``; ``h`` is n in ``dtype``, with ``conv = (w [taps, H], tail [slots, (taps - 1) * H])`` plus the causal
+    convolution of n (only where every sequence of ``ctx`` brings one token; the tail is moved on).  ``rows`` takes those
+    tokens alone.  Returns ``(h, n, u, x)``, each None unless wanted."""
+    H = x.shape[-1]
+    S = int(streams)
+    _need(x, "x", torch.float32)
+    if not (1 <= S <= HYPER_MAX_STREAMS) or x.dim() not in (2, 3) or (x.dim() == 3 and x.shape[1] != S):
+        raise KernelError(f"x must be [tokens, {S}, features] or [tokens, features], got {tuple(x.shape)} (at most "
+                          f"{HYPER_MAX_STREAMS} streams)")
+    M_in = x.shape[0]
+    y_ld = 0
+    if y is not None:
+        y_ld = _rows_of(y, "y", H, dtype)
+        if y.shape[0] != M_in:
+            raise KernelError("a sublayer's result and the streams differ in their number of rows")
+        _need(mix, "mix", torch.float32, (S, S))
+        _need(out, "out", torch.float32, (S,))
+    elif want_x:
+        raise KernelError("without a sublayer's result the streams stay what they are")
+    if weights is not None:
+        _need(weights, "weights", torch.float32, (S,))
+    w, offset, eps = norm if norm is not None else (None, 0.0, 0.0)
+    if w is not None:
+        _need(w, "weight", torch.float32, (H,))
+    elif want_n or want_h:
+        raise KernelError("a norm needs its weight")
+    if rows is not None:
+        _need(rows, "rows", torch.int32)
+    M = M_in if rows is None else rows.numel()
+    new = lambda shape, dt: torch.empty(shape, dtype=dt, device=x.device)
+    x_out = new((M, S, H), torch.float32) if want_x else None
+    u = new((M, H), torch.float32) if want_u else None
+    n = new((M, H), torch.float32) if want_n else None
+    h = new((M, H), dtype) if want_h else None
+    conv_w = tail = token_seq = seq_slot = None
+    taps = tail_ld = 0
+    if conv is not None:
+        conv_w, tail = conv
+        taps = conv_w.shape[0]
+        _need(conv_w, "conv", torch.float32, (taps, H))
+        if taps > 1:
+            tail_ld = _need_state(tail, (taps - 1) * H, "tail")
+        token_seq, seq_slot = ctx.token_seq, ctx.seq_slot
+        _need(token_seq, "token_seq", torch.int32, (M,))
+        _need(seq_slot, "seq_slot", torch.int32, (M,))  # one token a sequence: as many sequences as tokens
+    if M:
+        _call("pta_hyper_norm", _ptr(h), _ptr(n), _ptr(u), _ptr(x_out), _ptr(x), ctypes.c_long(H if x.dim() == 2 else S * H),
+              ctypes.c_long(0 if x.dim() == 2 else H), _ptr(y), ctypes.c_long(y_ld), _ptr(mix), _ptr(out), _ptr(weights), _ptr(w),
+              ctypes.c_float(offset), ctypes.c_float(eps), _ptr(rows), _ptr(conv_w), int(taps), _ptr(tail), ctypes.c_long(tail_ld),
+              _ptr(token_seq), _ptr(seq_slot), M, H, S, dtype_code(dtype), _stream())
+    return h, n, u, x_out
+
+
+def conv_add(x: torch.Tensor, w: torch.Tensor, tail: Optional[torch.Tensor], ctx, dtype: torch.dtype) -> torch.Tensor:
+    """``x`` plus a causal convolution of it per channel over each sequence's tokens, in ``dtype``: ``x`` ``[tokens,
+    channels]`` and ``w`` ``[taps, channels]`` (the last tap is the token's own) in 32-bit; ``tail`` ``[slots, (taps - 1) *
+    channels]`` holds every sequence's last inputs from before the step and is moved on."""
+    K, C = w.shape
+    M = x.shape[0]
+    _need(x, "x", torch.float32, (M, C))
+    _need(w, "w", torch.float32)
+    n = ctx.seq_slot.numel()
+    _need(ctx.cu_tokens, "cu_tokens", torch.int32, (n + 1,))
+    _need(ctx.token_seq, "token_seq", torch.int32, (M,))
+    tail_ld = _need_state(tail, (K - 1) * C, "tail") if K > 1 else 0
+    out = torch.empty((M, C), dtype=dtype, device=x.device)
+    if M:
+        _call("pta_conv_add", _ptr(out), _ptr(x), _ptr(w), _ptr(tail), ctypes.c_long(tail_ld), _ptr(ctx.cu_tokens), _ptr(ctx.token_seq),
+              _ptr(ctx.seq_slot), n, M, C, K, dtype_code(dtype), _stream())
+    return out
+
+
+# ---- the gated delta rule with a decay per key channel --------------------------------------------------------------
+DELTA_CHUNK_TOKENS = 128  # a sequence that brings more than twice as many tokens is cut into chunks that run side by side
+
+
+def delta_prep(qkv: torch.Tensor, conv: torch.Tensor, a: torch.Tensor, b: torch.Tensor, a_log, dt_bias, tail, ctx, heads: int,
+               kv_heads: int, key_dim: int, value_dim: int, norm_eps: float):
+    """What the delta rule's recurrence reads, in 32-bit: from ``qkv`` ``[tokens, channels]`` (q and k of ``kv_heads`` heads,
+    v of ``heads`` heads; may be a block of columns) through a causal convolution (``conv`` ``[taps, channels]``, the
+    sequences' last inputs in ``tail``, which is moved on) and silu, q and k to unit length per head (``norm_eps`` in the
+    root), q times key_dim^(-1/2); the decays ``exp(-exp(a_log) softplus(a + dt_bias))`` per head and key channel; the step
+    sizes ``sigmoid(b)``.  Returns ``(qkv, decays, step sizes)``."""
+    K, C = conv.shape
+    if C != 2 * kv_heads * key_dim + heads * value_dim:
+        raise KernelError(f"conv has {C} channels, q, k and v have {2 * kv_heads * key_dim + heads * value_dim}")
+    M = qkv.shape[0]
+    ld = _rows_of(qkv, "qkv", C)
+    _need(conv, "conv", torch.float32)
+    a_ld, b_ld = _rows_of(a, "a", heads * key_dim, qkv.dtype), _rows_of(b, "b", heads, qkv.dtype)
+    if a.shape[0] != M or b.shape[0] != M:
+        raise KernelError("qkv, a and b differ in their number of rows")
+    _need(a_log, "A_log", torch.float32, (heads,))
+    _need(dt_bias, "dt_bias", torch.float32, (heads * key_dim,))
+    n = ctx.seq_slot.numel()
+    _need(ctx.cu_tokens, "cu_tokens", torch.int32, (n + 1,))
+    _need(ctx.token_seq, "token_seq", torch.int32, (M,))
+    tail_ld = _need_state(tail, (K - 1) * C, "tail") if K > 1 else 0
+    new = lambda cols: torch.empty((M, cols), dtype=torch.float32, device=qkv.device)
+    out, g, beta = new(C), new(heads * key_dim), new(heads)
+    size = qkv.element_size()
+    at = lambda cols: ctypes.c_void_p(qkv.data_ptr() + cols * size)
+    if M:
+        _call("pta_delta_prep", _ptr(out), _ptr(g), _ptr(beta), at(0), at(kv_heads * key_dim), at(2 * kv_heads * key_dim),
+              ctypes.c_long(ld), _ptr(conv), _ptr(a), ctypes.c_long(a_ld), _ptr(b), ctypes.c_long(b_ld), _ptr(a_log), _ptr(dt_bias),
+              _ptr(tail), ctypes.c_long(tail_ld), _ptr(ctx.cu_tokens), _ptr(ctx.token_seq), _ptr(ctx.seq_slot),
+              int(max(ctx.new_tokens) > 1), n, M, heads, kv_heads, key_dim, value_dim, K, ctypes.c_float(key_dim ** -0.5),
+              ctypes.c_float(norm_eps), dtype_code(qkv.dtype), _stream())
+    return out, g, beta
+
+
+def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: torch.Tensor, ctx, heads: int, kv_heads: int,
+               key_dim: int, value_dim: int) -> torch.Tensor:
+    """Per head ``S <- diag(g) S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q`` over every sequence's tokens,
+    from and into its row of ``state`` ``[slots, heads * key_dim * value_dim]``; inputs as ``delta_prep`` returns them.
+    Returns o ``[tokens, heads * value_dim]``; all 32-bit."""
+    C = 2 * kv_heads * key_dim + heads * value_dim
+    M = qkv.shape[0]
+    _need(qkv, "qkv", torch.float32, (M, C))
+    _need(g, "g", torch.float32, (M, heads * key_dim))
+    _need(beta, "beta", torch.float32, (M, heads))
+    n = ctx.seq_slot.numel()
+    _need(ctx.seq_slot, "seq_slot", torch.int32, (n,))
+    _need(ctx.cu_tokens, "cu_tokens", torch.int32, (n + 1,))
+    state_ld = _need_state(state, heads * key_dim * value_dim)
+    y = torch.empty((M, heads * value_dim), dtype=torch.float32, device=qkv.device)
+    timing_hint["rows"] = M
+    longest = int(max(ctx.new_tokens))
+    chunk, chunks = DELTA_CHUNK_TOKENS, 1
+    if longest > 2 * chunk:
+        chunks = (longest + chunk - 1) // chunk
+    chunk_state = None
+    if chunks > 1:
+        chunk_state = torch.empty((n * chunks, heads, key_dim, value_dim + key_dim), dtype=torch.float32, device=qkv.device)
+    if M:
+        _call("pta_delta_scan", _ptr(y), _ptr(qkv), _ptr(g), _ptr(beta), _ptr(state), ctypes.c_long(state_ld), _ptr(chunk_state),
+              _ptr(ctx.cu_tokens), _ptr(ctx.seq_slot), n, longest, heads, kv_heads, value_dim, key_dim, chunk, chunks, _stream())
+    return y
 
 
 # ---- linear attention with a decay per head -------------------------------------------------------------------------

@@ -5,9 +5,10 @@ from .norms import LayerNorm, RMSNorm
 from .positions import AlibiPositions, NoPositions, Rotation, RotaryPositions, ScoreBias, alibi_slopes
 from .attention import AttentionMixer
 from .feedforward import DenseFeedForward, GatedFeedForward, PolyNormFeedForward, RoutedFeedForward, XieluFeedForward
-from .blocks import ParallelBlock, PostNormBlock, SandwichBlock, SequentialBlock, ShiftedParallelBlock
+from .blocks import HyperBlock, ParallelBlock, PostNormBlock, SandwichBlock, SequentialBlock, ShiftedParallelBlock
 from .gated_attention import GatedAttentionMixer
 from .linear_attention import DecayLinearAttentionMixer
+from .delta_rule import ChannelDeltaMixer
 from .depth import DepthMix, LoopEntry
 from .latent_attention import LatentAttentionMixer
 from .recurrent import GatedScanMixer, StateSpaceMixer
@@ -17,4 +18,4 @@ __all__ = ["Part", "StepContext", "make_part", "register_part", "registered_part
            "AttentionMixer", "DenseFeedForward", "ParallelBlock", "SequentialBlock", "PostNormBlock", "RMSNorm", "DepthMix",
            "LatentAttentionMixer", "GatedScanMixer", "StateSpaceMixer", "GatedFeedForward", "RoutedFeedForward",
            "ShiftedParallelBlock", "GatedAttentionMixer", "DecayLinearAttentionMixer", "SandwichBlock", "LoopEntry",
-           "PolyNormFeedForward", "XieluFeedForward"]
+           "PolyNormFeedForward", "XieluFeedForward", "HyperBlock", "ChannelDeltaMixer"]

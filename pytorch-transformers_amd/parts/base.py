@@ -206,6 +206,35 @@ class PendingNormSum(WideResidual):
         return self.wide if self.dtype == torch.float32 else self.wide.to(self.dtype)
 
 
+class HyperStreams(WideResidual):
+    """``count`` residual streams per token in 32-bit: ``x`` ``[tokens, count, features]``, or ``[tokens, features]`` where
+    all of them are still that one.  A sublayer's result ``y`` (compute type) may be not yet taken in: the streams are then
+    ``sum_s mix[s, t] x_s + out[t] y``, formed by the launch that reads them next (``parts.blocks.HyperBlock``; the final
+    norm, for the wanted rows alone).  As one stream (``wide``) they are their sum."""
+
+    def __init__(self, x: torch.Tensor, count: int, dtype: torch.dtype, y: Optional[torch.Tensor] = None, mix=None, out=None):
+        self.x, self.count, self.dtype = x, int(count), dtype
+        self.y, self.mix, self.out = y, mix, out
+        self.history = None
+        self._wide = None
+
+    def launch(self, **how):
+        """``ops.hyper_norm`` on these streams."""
+        from .. import ops
+
+        return ops.hyper_norm(self.x, self.count, self.dtype, y=self.y, mix=self.mix, out=self.out, **how)
+
+    @property
+    def wide(self) -> torch.Tensor:
+        if self._wide is None:
+            self._wide = self.launch(want_u=True)[2]
+        return self._wide
+
+    @property
+    def narrow(self) -> torch.Tensor:
+        return self.wide if self.dtype == torch.float32 else self.wide.to(self.dtype)
+
+
 def as_tensor(x):
     """A tensor from what a part may hand on: a tensor, a ``PartialProduct``, a ``ResidualSum`` or a
     ``WideResidual`` (its 32-bit side)."""

@@ -17,8 +17,8 @@ from typing import Optional, Sequence
 
 import torch
 
-from ..engine.spec import INIT_ZERO_NOISE, VECTOR, TensorSpec
-from .base import Part, PendingNormSum, ResidualSum, StepContext, WideResidual, WideSum, as_tensor, register_part
+from ..engine.spec import INIT_EYE_NOISE, INIT_NORMAL, INIT_ONE_NOISE, INIT_ZERO_NOISE, VECTOR, TensorSpec
+from .base import HyperStreams, Part, PendingNormSum, ResidualSum, StepContext, WideResidual, WideSum, as_tensor, register_part
 from .linear import Linear, PendingProjection
 
 
@@ -323,6 +323,112 @@ class SandwichBlock(Part):
         return PendingNormSum(wide, out, self.norm_ffn_out.affine(), m, eps, dtype)
 
 
+class HyperBlock(Part):
+    """Several residual streams (hyper-connections) with a norm in front of each sublayer.  For sublayer q (1: the mixer, 2:
+    the feed-forward), over the streams x_1 .. x_S held in 32-bit:
+
+        u = sum_s in_q[s] x_s;   y = sublayer(norm_q(u));   x_t <- sum_s mix_q[s, t] x_s + out_q[t] y  (all at once)
+
+    Between norm and mixer stands a causal convolution per channel that adds to what it reads, ``h + conv(h)`` (``taps``
+    inputs, the last column of ``conv_name`` ``[width, taps]`` being the token's own; 0: none), whose last ``taps - 1``
+    inputs are part of a sequence's state: a row of the state table that the run order's entry names as ``also("conv")``.
+    ``feed_forward`` may be None (a layer of the mixer alone).  The file holds ``name.hc<q>.in``, ``.out`` ``[S]`` and
+    ``.mix`` ``[S, S]`` (from, to).
+
+    Everything between two sublayers is one launch (``ops.hyper_norm``), across the block's end too: the block hands its
+    last sublayer's result on not yet taken in (``HyperStreams``).  In steps of one token per sequence the convolution
+    rides in that launch as well."""
+
+    accepts_sum = False
+    accepts_wide = True
+
+    def __init__(self, name: str, mixer: Part, feed_forward: Optional[Part], norm_mixer: Part, norm_ffn: Optional[Part],
+                 streams: int, hidden_size: int, taps: int = 0, conv_name: Optional[str] = None):
+        if (feed_forward is None) != (norm_ffn is None):
+            raise ValueError("a feed-forward and its norm come together or not at all")
+        if any(n is not None and (not hasattr(n, "launch_terms") or n.groups != 1) for n in (norm_mixer, norm_ffn)):
+            raise ValueError("the block's launches take RMS norms over whole rows")
+        if taps and conv_name is None:
+            raise ValueError("a convolution needs its tensor's name")
+        self.name, self.streams, self.hidden_size, self.taps, self.conv_name = name, int(streams), int(hidden_size), int(taps), conv_name
+        self.mixer, self.feed_forward, self.norm_mixer, self.norm_ffn = mixer, feed_forward, norm_mixer, norm_ffn
+        self.links = {}  # sublayer -> (in, mix, out)
+        self.conv_w: Optional[torch.Tensor] = None
+
+    @property
+    def conv_state(self) -> int:
+        """Elements of a sequence's state that the convolution keeps."""
+        return max(self.taps - 1, 0) * self.hidden_size
+
+    def children(self) -> Sequence[Part]:
+        return tuple(p for p in (self.norm_mixer, self.norm_ffn, self.mixer, self.feed_forward) if p is not None)
+
+    def _sublayers(self):
+        return (1,) if self.feed_forward is None else (1, 2)
+
+    def tensor_specs(self):
+        S, specs = self.streams, []
+        for q in self._sublayers():
+            specs += [TensorSpec(f"{self.name}.hc{q}.in", (S,), VECTOR, INIT_ONE_NOISE),
+                      TensorSpec(f"{self.name}.hc{q}.out", (S,), VECTOR, INIT_ONE_NOISE),
+                      TensorSpec(f"{self.name}.hc{q}.mix", (S, S), VECTOR, INIT_EYE_NOISE)]
+        if self.taps:
+            specs.append(TensorSpec(self.conv_name, (self.hidden_size, self.taps), VECTOR, INIT_NORMAL))
+        return specs
+
+    def load(self, tensors) -> None:
+        for q in self._sublayers():
+            self.links[q] = tuple(tensors[f"{self.name}.hc{q}.{t}"] for t in ("in", "mix", "out"))
+        if self.taps:
+            self.conv_w = tensors[self.conv_name].t().contiguous()  # tap by tap, so that neighbouring channels lie side by side
+
+    def after_load(self) -> None:
+        for part in (self.mixer, self.feed_forward):
+            if part is not None and hasattr(part, "after_load"):
+                part.after_load()
+
+    def check_sizes(self) -> None:
+        from .. import ops
+
+        if not (1 <= self.streams <= ops.HYPER_MAX_STREAMS):
+            raise ValueError(f"{self.name}: {self.streams} streams are outside the 1..{ops.HYPER_MAX_STREAMS} that the kernel takes")
+        if self.taps > 16:
+            raise ValueError(f"{self.name}: a convolution of {self.taps} taps is more than the kernel's 16")
+        if self.hidden_size > 16384:
+            raise ValueError(f"{self.name}: rows of {self.hidden_size} features are more than the kernel's 16384")
+
+    def _head(self, x: HyperStreams, q: int, norm: Part, ctx: StepContext, conv=None):
+        """``(h, the streams with nothing left to take in)``: what sublayer q reads."""
+        from .. import ops
+
+        one_each = conv is None or ctx.n_tokens == ctx.n_seqs  # (the convolution rides along: its inputs are in the tails)
+        h, n, _, new = x.launch(weights=self.links[q][0], norm=norm.launch_terms(), want_x=x.y is not None, want_h=one_each,
+                                want_n=not one_each, conv=conv if one_each else None, ctx=ctx)
+        if not one_each:
+            h = ops.conv_add(n, conv[0], conv[1], ctx, ctx.dtype)
+        return h, (x.x if new is None else new)
+
+    def forward(self, x, ctx: StepContext, call):
+        from .. import ops
+
+        if not isinstance(x, HyperStreams):
+            x = as_tensor(x)
+            x = HyperStreams(x if x.dtype == torch.float32 else ops.widen(x), self.streams, ctx.dtype)
+        conv = None
+        if self.taps:
+            tail = ctx.cache.state_layer(*call.also("conv")) if self.taps > 1 else None
+            conv = (self.conv_w, tail)
+        h, streams = self._head(x, 1, self.norm_mixer, ctx, conv)
+        _, mix, out = self.links[1]
+        x = HyperStreams(streams, self.streams, ctx.dtype, self.mixer.forward(h, ctx, call), mix, out)
+        if self.feed_forward is None:
+            return x
+        h, streams = self._head(x, 2, self.norm_ffn, ctx)
+        _, mix, out = self.links[2]
+        return HyperStreams(streams, self.streams, ctx.dtype, self.feed_forward.forward(h, ctx), mix, out)
+
+
+register_part("block", "hyper", HyperBlock)
 register_part("block", "sandwich", SandwichBlock)
 register_part("block", "shifted_parallel", ShiftedParallelBlock)
 register_part("block", "post_norm", PostNormBlock)

@@ -99,7 +99,7 @@ class XieluFeedForward(Part):
 
 class GatedFeedForward(Part):
     """A feed-forward with a gate: ``down(glu(gate(x), up(x)))``, no biases.  ``kind`` ``"silu"``: ``silu(gate) * up``;
-    ``"clamped"``: with ``g = min(gate, limit)`` and ``u = clamp(up, -limit, limit)``, ``g * sigmoid(alpha * g) * (u +
+    ``"gelu_tanh"``: ``gelu_tanh(gate) * up``; ``"clamped"``: with ``g = min(gate, limit)`` and ``u = clamp(up, -limit, limit)``, ``g * sigmoid(alpha * g) * (u +
     1)``.  The two input products run as one; the gate's arithmetic is 32-bit.  The file holds the matrices as
     ``name.gate``, ``name.up`` and ``name.down``."""
 
@@ -130,6 +130,9 @@ class GatedFeedForward(Part):
         F = self.ffn_size
         y = ops.glu(both[:, :F], both[:, F:], self.kind, self.alpha, self.limit)
         return self.down(y, add1=as_tensor(add1), add2=as_tensor(add2))
+
+
+EXPERT_GATES = ("silu", "clamped")  # the kinds of gate that the experts' launches form
 
 
 def _stack_experts(experts: int, rows_each: Sequence[int]):
@@ -175,8 +178,8 @@ class RoutedFeedForward(Part):
     def __init__(self, name: str, hidden_size: int, ffn_size: int, experts: int, top: int, scale: float = 1.0,
                  score: str = "sigmoid", normalise: bool = True, act: str = "silu", router_bias: bool = False, gate=None,
                  gated: bool = True, groups=None, shared_ff: int = 0, shared_gate: bool = False):
-        if gate is not None and gate[0] not in ops.GLU_CODES:
-            raise ValueError(f"{name}: a gate of kind {gate[0]!r} is not built; built: {sorted(ops.GLU_CODES)}")
+        if gate is not None and gate[0] not in EXPERT_GATES:
+            raise ValueError(f"{name}: a gate of kind {gate[0]!r} is not built; built: {sorted(EXPERT_GATES)}")
         if not (0 < top <= experts):
             raise ValueError(f"{name}: {top} of {experts} experts per token")
         if score not in ops.ROUTE_SCORE_CODES:

@@ -15,7 +15,10 @@ With h the mixer's input, H query heads on G key/value heads, queries and keys o
         and / or the last ``window``
     out = W_o (heads side by side * sigmoid(W_g h))
 
-Options beside these: ``bias`` (q, k, v and the output projection have biases, ``name.q.b`` and so on); ``head_scale`` (a
+Options beside these: ``bias`` (q, k, v and the output projection have biases, ``name.q.b`` and so on; or a string that
+says which of them have one, ``"qk"``); ``v_from_k`` (no W_v: a head's value is its key as projected, before norm and
+rotation; ``value_dim`` equals ``key_dim``); ``sink`` (a learned number per head ``name.sink`` whose exponential joins the
+sum that the head's weights are divided by: a key without a value); ``head_scale`` (a
 learned number per head, ``name.temp``, multiplies the head's scores before the cap); ``weights="sigmoid"`` (no softmax:
 a seen key's weight is ``sigmoid(score + pb[h])`` with a learned number per head ``name.pb``, not normalised over the
 keys); ``gate_per_head`` (the gate is one number a head, ``W_g`` has a row per head).
@@ -47,8 +50,9 @@ def attention_frame(key_dim: int, value_dim: int) -> int:
 class GatedAttentionMixer(Part):
     def __init__(self, name: str, hidden_size: int, num_heads: int, kv_heads: int, key_dim: int, value_dim: int,
                  scale: float, eps: float, positions: Part, chunk: int = 0, window: int = 0, qk_norm: bool = True,
-                 v_norm: bool = True, gate: bool = True, softcap: float = 0.0, talk: bool = False, bias: bool = False,
-                 head_scale: bool = False, weights: str = "softmax", gate_per_head: bool = False):
+                 v_norm: bool = True, gate: bool = True, softcap: float = 0.0, talk: bool = False, bias=False,
+                 head_scale: bool = False, weights: str = "softmax", gate_per_head: bool = False, v_from_k: bool = False,
+                 sink: bool = False):
         if num_heads % kv_heads:
             raise ValueError(f"{name}: heads ({num_heads}) must be a multiple of kv heads ({kv_heads})")
         self.name, self.hidden_size = name, int(hidden_size)
@@ -59,17 +63,23 @@ class GatedAttentionMixer(Part):
         self.softcap, self.talk = float(softcap), bool(talk)
         if weights not in ops.WEIGHTS_CODES:
             raise ValueError(f"{name}: attention weights of kind {weights!r} are not built; built: {sorted(ops.WEIGHTS_CODES)}")
-        self.bias, self.head_scale, self.weights, self.gate_per_head = bool(bias), bool(head_scale), weights, bool(gate_per_head)
+        biased = bias if isinstance(bias, str) else ("qkvo" if bias else "")
+        if set(biased) - set("qkvo"):
+            raise ValueError(f"{name}: biases are for the projections q, k, v and o, not {bias!r}")
+        self.bias, self.head_scale, self.weights, self.gate_per_head = biased, bool(head_scale), weights, bool(gate_per_head)
+        self.v_from_k, self.sink = bool(v_from_k), bool(sink)
+        if self.v_from_k and self.key_dim != self.value_dim:
+            raise ValueError(f"{name}: values that are the keys have the keys' size {key_dim}, not {value_dim}")
         self.talk_w: Optional[torch.Tensor] = None
-        self.temp = self.head_bias = None
+        self.temp = self.head_bias = self.sink_w = None
         self.frame = attention_frame(key_dim, value_dim)
         bare = lambda short, i, o, b=False: Linear(f"{name}.{short}", i, o, b, weight_name=f"{name}.{short}",
                                                    bias_name=f"{name}.{short}.b")
-        self.q = bare("q", hidden_size, self.num_heads * self.key_dim, self.bias)
-        self.k = bare("k", hidden_size, self.kv_heads * self.key_dim, self.bias)
-        self.v = bare("v", hidden_size, self.kv_heads * self.value_dim, self.bias)
+        self.q = bare("q", hidden_size, self.num_heads * self.key_dim, "q" in biased)
+        self.k = bare("k", hidden_size, self.kv_heads * self.key_dim, "k" in biased)
+        self.v = None if self.v_from_k else bare("v", hidden_size, self.kv_heads * self.value_dim, "v" in biased)
         self.g = bare("g", hidden_size, self.num_heads * (1 if self.gate_per_head else self.value_dim)) if self.gate else None
-        self.out = bare("o", self.num_heads * self.value_dim, hidden_size, self.bias)
+        self.out = bare("o", self.num_heads * self.value_dim, hidden_size, "o" in biased)
         self.q_w = self.k_w = None
         self.inp: Optional[Linear] = None
 
@@ -85,6 +95,8 @@ class GatedAttentionMixer(Part):
             specs.append(TensorSpec(f"{self.name}.talk", (self.num_heads, self.num_heads), VECTOR, INIT_EYE_NOISE))
         if self.head_scale:
             specs.append(TensorSpec(f"{self.name}.temp", (self.num_heads,), VECTOR, INIT_ONE_NOISE))
+        if self.sink:
+            specs.append(TensorSpec(f"{self.name}.sink", (self.num_heads,), VECTOR, INIT_ZERO_NOISE))
         if self.weights == "sigmoid":
             specs.append(TensorSpec(f"{self.name}.pb", (self.num_heads,), VECTOR, INIT_ZERO_NOISE))
         return specs
@@ -96,12 +108,14 @@ class GatedAttentionMixer(Part):
             self.talk_w = tensors[f"{self.name}.talk"]
         if self.head_scale:
             self.temp = tensors[f"{self.name}.temp"]
+        if self.sink:
+            self.sink_w = tensors[f"{self.name}.sink"]
         if self.weights == "sigmoid":
             self.head_bias = tensors[f"{self.name}.pb"]
 
     def after_load(self) -> None:
         self.inp = Linear.stacked(f"{self.name}.qkvg", [p for p in (self.q, self.k, self.v, self.g) if p is not None],
-                                  pad_to=8, with_bias=self.bias)
+                                  pad_to=8, with_bias=bool(self.bias))
 
     def check_sizes(self) -> None:
         rot = as_rotation(self.positions.rotation())
@@ -112,6 +126,8 @@ class GatedAttentionMixer(Part):
             problem = ops.rotation_problem(self.key_dim, rot.rotary_dim, rot.pairing)
         if problem is None and (self.chunk < 0 or self.window < 0 or self.softcap < 0):
             problem = "chunk, window and softcap are 0 (none) or positive"
+        if problem is None and self.sink and self._talk_kernels():
+            problem = "a number that joins the weights' sum goes with plain softmax attention"
         if problem is None and self._talk_kernels():
             problem = ops.attn_talk_sizes_problem(self.num_heads, self.kv_heads, self.frame)
         if problem is not None:
@@ -132,8 +148,9 @@ class GatedAttentionMixer(Part):
         table = ctx.block_tables[call.cache_group]
         H, G, dk, dv = self.num_heads, self.kv_heads, self.key_dim, self.value_dim
         proj = projected if projected is not None else self.inp(x)
-        at = [0, H * dk, (H + G) * dk, (H + G) * dk + G * dv]
-        q = ops.head_norm_rope_cache(proj[:, at[0]:at[1]], proj[:, at[1]:at[2]], proj[:, at[2]:at[3]], self.q_w, self.k_w,
+        at = [0, H * dk, (H + G) * dk, (H + G) * dk + (0 if self.v_from_k else G * dv)]
+        keys = proj[:, at[1]:at[2]]
+        q = ops.head_norm_rope_cache(proj[:, at[0]:at[1]], keys, keys if self.v_from_k else proj[:, at[2]:at[3]], self.q_w, self.k_w,
                                      self.eps, self.v_norm, as_rotation(self.positions.rotation()), ctx, table, k_pool,
                                      v_pool, H, G, dk, dv, write_cache=call.write_cache)
         if self._talk_kernels():
@@ -141,7 +158,7 @@ class GatedAttentionMixer(Part):
                                    window=self.window, chunk=self.chunk, head_scale=self.temp, head_bias=self.head_bias,
                                    weights=self.weights)
         else:
-            o = ops.attention(q, k_pool, v_pool, table, ctx, None, self.scale, self.window, chunk=self.chunk)
+            o = ops.attention(q, k_pool, v_pool, table, ctx, None, self.scale, self.window, chunk=self.chunk, sink=self.sink_w)
         if self.gate:
             g_cols = H if self.gate_per_head else H * dv
             o = ops.gated_heads(o, self.frame, proj[:, at[3]:at[3] + g_cols], H, dv, x.dtype, per_head=self.gate_per_head)

@@ -10,7 +10,9 @@ and nothing but c and the rotated part is ever stored.
 
 Options: the queries may themselves come through a latent (``q_rank``: ``q = W_uq (rmsnorm(W_dq h) * w)``, the file's
 ``dq``, ``dq.norm`` and ``uq`` in place of ``q``), and the heads' values side by side may be multiplied by ``sigmoid(W_g
-h)`` element by element before the output projection (``gate``).
+h)`` element by element before the output projection (``gate``).  A layer with ``reads_other`` has no down-projection of
+its own: it attends over the cache rows that another layer has written for the same tokens (the run order names that
+layer's storage, with ``write_cache=False``), with queries and expansions of its own.
 """
 from __future__ import annotations
 
@@ -27,7 +29,7 @@ from .positions import as_rotation
 
 class LatentAttentionMixer(Part):
     def __init__(self, name: str, hidden_size: int, heads: int, dim: int, rot_dim: int, value_dim: int, rank: int,
-                 scale: float, eps: float, positions: Part, q_rank: int = 0, gate: bool = False):
+                 scale: float, eps: float, positions: Part, q_rank: int = 0, gate: bool = False, reads_other: bool = False):
         """``dim`` / ``rot_dim``: plain and rotated elements of a head's query and key; ``positions`` says how the
         rotated part turns (a ``Rotation`` over ``rot_dim`` elements); ``q_rank`` > 0: the size of the queries' latent;
         ``gate``: an output gate ``name.g``."""
@@ -36,13 +38,13 @@ class LatentAttentionMixer(Part):
         self.scale, self.eps = float(scale), float(eps)
         self.positions = positions
         bare = lambda short, i, o: Linear(f"{name}.{short}", i, o, False, weight_name=f"{name}.{short}")
-        self.q_rank, self.gate = int(q_rank), bool(gate)
+        self.q_rank, self.gate, self.reads_other = int(q_rank), bool(gate), bool(reads_other)
         q_cols = self.heads * (self.dim + self.rot_dim)
         if self.q_rank:
             self.q_latent, self.q = bare("dq", hidden_size, self.q_rank), bare("uq", self.q_rank, q_cols)
         else:
             self.q_latent, self.q = None, bare("q", hidden_size, q_cols)
-        self.down = bare("dkv", hidden_size, self.rank + self.rot_dim)
+        self.down = None if self.reads_other else bare("dkv", hidden_size, self.rank + self.rot_dim)
         self.g = bare("g", hidden_size, self.heads * self.value_dim) if self.gate else None
         self.out = bare("o", self.heads * self.value_dim, hidden_size)
         self.q_down: Optional[Linear] = None
@@ -59,13 +61,15 @@ class LatentAttentionMixer(Part):
     def tensor_specs(self) -> List[TensorSpec]:
         n = self.name
         q_norm = [TensorSpec(f"{n}.dq.norm", (self.q_rank,), VECTOR, INIT_ONE_NOISE)] if self.q_rank else []
-        return q_norm + [TensorSpec(f"{n}.dkv.norm", (self.rank,), VECTOR, INIT_ONE_NOISE),
+        kv_norm = [] if self.reads_other else [TensorSpec(f"{n}.dkv.norm", (self.rank,), VECTOR, INIT_ONE_NOISE)]
+        return q_norm + kv_norm + [
                 TensorSpec(f"{n}.uk", (self.heads * self.dim, self.rank), MATRIX, INIT_NORMAL),
                 TensorSpec(f"{n}.uv", (self.heads * self.value_dim, self.rank), MATRIX, INIT_NORMAL)]
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         n = self.name
-        self.norm_w, self.up_k, self.up_v = tensors[f"{n}.dkv.norm"], tensors[f"{n}.uk"], tensors[f"{n}.uv"]
+        self.up_k, self.up_v = tensors[f"{n}.uk"], tensors[f"{n}.uv"]
+        self.norm_w = None if self.reads_other else tensors[f"{n}.dkv.norm"]
         self.q_norm_w = tensors[f"{n}.dq.norm"] if self.q_rank else None
 
     def after_load(self) -> None:
@@ -93,17 +97,18 @@ class LatentAttentionMixer(Part):
         rot = as_rotation(self.positions.rotation())
         proj = self.q_down(x)
         M, D, H = x.shape[0], self.cache_row, self.heads
+        made = 0 if self.reads_other else D  # columns of the product that become the token's cache row
         q_cols = H * (self.dim + self.rot_dim)
         if self.q_rank:  # the queries through their own latent: norm in 32-bit, then the second product
             lat_q = ops.rmsnorm(proj[:, :self.q_rank], self.q_norm_w, self.eps, x.dtype)[0]
             queries, at = self.q(lat_q), self.q_rank
         else:
             queries, at = proj[:, :q_cols], q_cols
-        q_full = ops.latent_prep(proj[:, at:at + D], self.norm_w, self.eps, None if rot is None else rot.inv_freq,
+        q_full = ops.latent_prep(proj[:, at:at + D] if made else None, self.norm_w, self.eps, None if rot is None else rot.inv_freq,
                                  1.0 if rot is None else rot.scale, None if rot is None else rot.rotary_dim,
                                  "half" if rot is None else rot.pairing, ctx.token_pos, ctx.token_seq, table, k_pool,
-                                 self.heads, self.dim, self.rot_dim, self.rank, write_cache=call.write_cache, q=queries)
-        gate = proj[:, at + D:at + D + H * self.value_dim] if self.gate else None
+                                 self.heads, self.dim, self.rot_dim, self.rank, write_cache=call.write_cache and not self.reads_other, q=queries)
+        gate = proj[:, at + made:at + made + H * self.value_dim] if self.gate else None
         library = x.dtype == torch.bfloat16 and M > ops.HEAD_PROJECT_LIBRARY_ROWS
         # each head's plain query through the transpose of its key expansion: the first `rank` of its frame
         if library:

@@ -257,10 +257,14 @@ class Embedding(Part):
 
     With ``scale`` and / or ``position_name`` (a learned table ``[max_positions, hidden]`` under that name in the file):
     ``h[t] = E[id_t] * scale + P[position of t]``, formed and handed on in 32-bit as the start of a stream that is held
-    so; the model then calls ``forward(ids, ctx)`` (``wants_context``)."""
+    so; the model then calls ``forward(ids, ctx)`` (``wants_context``).  With ``norm`` (an ``RMSNorm``): ``h[t] =
+    norm(E[id_t])``, likewise in 32-bit, in one launch over the table's rows."""
 
     def __init__(self, name: str, vocab_size: int, hidden_size: int, weight_name: Optional[str] = None, scale: float = 1.0,
-                 position_name: Optional[str] = None, max_positions: int = 0):
+                 position_name: Optional[str] = None, max_positions: int = 0, norm: Optional[Part] = None):
+        if norm is not None and (position_name is not None or scale != 1.0):
+            raise ValueError(f"{name}: a norm on the embedding goes with neither a scale nor a position table")
+        self.norm = norm
         self.name = name
         self.weight_name = weight_name or name + ".weight"
         self.vocab_size = vocab_size
@@ -278,12 +282,17 @@ class Embedding(Part):
             specs.append(TensorSpec(self.position_name, (self.max_positions, self.hidden_size), MATRIX, INIT_NORMAL))
         return specs
 
+    def children(self) -> Sequence[Part]:
+        return () if self.norm is None else (self.norm,)
+
     def load(self, tensors) -> None:
         self.weight = tensors[self.weight_name]
         if self.position_name is not None:
             self.positions = tensors[self.position_name]
 
     def forward(self, ids: torch.Tensor, ctx=None) -> torch.Tensor:
+        if self.norm is not None:
+            return self.norm.apply(self.weight, self.weight.dtype, rows=ids, want_wide=True, want_narrow=False)[1]
         if not self.wants_context:
             return ops.embed(self.weight, ids)
         if self.positions is not None and ctx.starts and ctx.new_tokens:

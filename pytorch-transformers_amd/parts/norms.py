@@ -8,7 +8,7 @@ import torch
 
 from .. import ops
 from ..engine.spec import INIT_ONE_NOISE, INIT_ZERO_NOISE, VECTOR, TensorSpec
-from .base import Part, ResidualSum, register_part
+from .base import HyperStreams, Part, ResidualSum, register_part
 
 
 class LayerNorm(Part):
@@ -115,6 +115,10 @@ class RMSNorm(Part):
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         self.weight = tensors[self.name]
 
+    def launch_terms(self):
+        """(weight, offset, eps), for a launch that applies this norm beside other work (``ops.hyper_norm``)."""
+        return self.weight, self.offset, self.eps
+
     def apply(self, x: torch.Tensor, dtype: torch.dtype, **how):
         """``ops.rmsnorm`` with this norm's weight and constants: ``(narrow, wide)``."""
         return ops.rmsnorm(x, self.weight, self.eps, dtype, offset=self.offset, groups=self.groups, **how)
@@ -123,7 +127,10 @@ class RMSNorm(Part):
         return self.apply(x, x.dtype, rows=rows)[0]
 
     def forward_wide(self, x, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """The norm of a ``WideResidual``'s 32-bit side, in its compute type."""
+        """The norm of a ``WideResidual``'s 32-bit side, in its compute type.  Several streams are summed in the same
+        launch, for the wanted rows alone."""
+        if isinstance(x, HyperStreams) and self.groups == 1:
+            return x.launch(norm=self.launch_terms(), rows=rows, want_h=True)[0]
         dtype = getattr(x, "dtype", None) or x.narrow.dtype  # (a sum that is not formed says its compute type itself)
         return self.apply(x.wide, dtype, rows=rows)[0]
 

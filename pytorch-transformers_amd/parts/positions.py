@@ -208,11 +208,15 @@ def yarn_ramp_frequencies(rotary_dim: int, base: float, factor: float, original:
 
 
 def llama3_frequencies(head_dim: int, theta: float, factor: float, low_freq_factor: float, high_freq_factor: float,
-                       original_max_position_embeddings: int) -> torch.Tensor:
+                       original_max_position_embeddings: int, precise: bool = False) -> torch.Tensor:
     """Llama 3.1's scheme (src/transformers/modeling_rope_utils.py:310-341): wavelengths beyond
     ``original / low_freq_factor`` are stretched by ``factor``, those under ``original / high_freq_factor`` stay,
-    and in between the two are blended by where the wavelength lies."""
-    inv = default_frequencies(head_dim, theta)
+    and in between the two are blended by where the wavelength lies.  ``precise``: evaluated in 64-bit and rounded once,
+    not step by step in 32-bit as the reference evaluates it."""
+    if precise:
+        inv = float(theta) ** (-torch.arange(0, head_dim, 2, dtype=torch.float64) / head_dim)
+    else:
+        inv = default_frequencies(head_dim, theta)
     wavelen = 2 * math.pi / inv
     long_from = original_max_position_embeddings / low_freq_factor
     short_to = original_max_position_embeddings / high_freq_factor
@@ -220,7 +224,7 @@ def llama3_frequencies(head_dim: int, theta: float, factor: float, low_freq_fact
     smooth = (original_max_position_embeddings / wavelen - low_freq_factor) / (high_freq_factor - low_freq_factor)
     blended = (1 - smooth) * out / factor + smooth * out
     middle = ~(wavelen < short_to) & ~(wavelen > long_from)
-    return torch.where(middle, blended, out)
+    return torch.where(middle, blended, out).float()
 
 
 def longrope_frequencies(head_dim: int, theta: float, short_factor, factor: Optional[float],

@@ -109,6 +109,20 @@ def first_float_dtype(folder: str) -> Optional[torch.dtype]:
     return None
 
 
+def tensor_shapes(folder: str) -> Dict[str, tuple]:
+    """Tensor name -> shape of everything the weight files hold, read from their headers."""
+    from safetensors import safe_open
+
+    files = resolve_files(folder)
+    out = {}
+    for path in sorted(set(files.values())):
+        with safe_open(path, framework="pt") as f:
+            for k in f.keys():
+                if files.get(k) == path:
+                    out[k] = tuple(f.get_slice(k).get_shape())
+    return out
+
+
 def device_dtype_for(spec: TensorSpec, compute_dtype: torch.dtype) -> torch.dtype:
     if spec.kind == MATRIX:
         return compute_dtype
