@@ -504,6 +504,45 @@ def nopuzen_config(size, layers, vocab=32768):
                          initializer_range=0.02)
 
 
+# ---- the Verelorn design beside the Nopuzen, Bimepel and Pavodra models (--design verelorn) -----------------------------------
+VERELORN_SIZES = {
+    # width; the dense feed-forward (three matrices: two thirds of a two-matrix one for as many weights); latent attention
+    # heads as Nopuzen's; attention heads of 128 on 8 KV heads; delta-rule heads of 128 x 128 on half as many q / k heads
+    "2k": dict(width=2048, ff=5504, heads=16, delta_heads=16),
+    "4k": dict(width=4096, ff=10880, heads=32, delta_heads=32),
+}
+VERELORN_STREAMS = 4
+VERELORN_KERNEL_LABELS = {
+    "pta_hyper_norm": "new streams, their weighted sum, RMS norm (+ the input convolution in decode steps)",
+    "pta_conv_add": "input convolution added to what the mixer reads (prompts)",
+    "pta_delta_prep": "delta rule: convolutions, unit lengths, decays, step sizes",
+    "pta_delta_scan": "delta rule's recurrence",
+    "pta_head_norm_gate": "delta rule: norm per head and output gate",
+    "pta_glu": "the dense feed-forward's gate",
+}
+
+
+def verelorn_config(size, layers, vocab=32768):
+    """Latent attention, delta rule, attention, and latent attention over the first layer's latents, in turn; the delta
+    rule's layers have a feed-forward too, so that the models compare layer by layer."""
+    from pytorch_transformers_amd.config import VerelornConfig
+
+    z = VERELORN_SIZES[size]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    lat = {"heads": z["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "scale": 192 ** -0.5,
+           "rot": {"base": 10000.0, "dims": 64}}
+    delta = {"heads": z["delta_heads"], "kv_heads": z["delta_heads"] // 2, "dim": 128, "vdim": 128, "conv": 4, "a_rank": 128, "g_rank": 128}
+    attn = {"heads": z["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+            "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    kinds = [{"type": "latent_attention", "mixer": lat, "mlp": dense}, {"type": "channel_delta", "mixer": delta, "mlp": dense},
+             {"type": "attention", "mixer": attn, "mlp": dense}]
+    out = [dict(kinds[i % 3]) for i in range(layers)]
+    for i in range(3, layers, 6):  # every second latent layer reads the layer three before it
+        out[i] = {"type": "latent_attention", "mixer": dict(lat, kv_from=i - 3), "mlp": dense}
+    return VerelornConfig(vocab=vocab, width=z["width"], streams=VERELORN_STREAMS, layers=out, norm={"eps": 1e-6}, canon={"taps": 4},
+                          initializer_range=0.02)
+
+
 def falcon_like(size, layers, vocab=32768):
     """The closest model the library had: Falcon's new architecture at the same width, feed-forward, depth and
     vocabulary, heads of 128 in 8 groups."""
@@ -529,12 +568,14 @@ def design_record(args):
     KERNEL_LABELS.update(BIMEPEL_KERNEL_LABELS)
     KERNEL_LABELS.update(KEKAPEL_KERNEL_LABELS)
     KERNEL_LABELS.update(NOPUZEN_KERNEL_LABELS)
+    if args.design == "verelorn":
+        KERNEL_LABELS.update(VERELORN_KERNEL_LABELS)
     design = args.design
     configs = {"pavodra": pavodra_config, "bimepel": bimepel_config, "kekapel": kekapel_config, "nopuzen": nopuzen_config,
-               "falcon": falcon_like}
+               "verelorn": verelorn_config, "falcon": falcon_like}
     design_config = configs[design]
     # the models a design stands beside: Falcon's, or for a design whose mechanisms came with other designs, those
-    beside = {"nopuzen": ("kekapel", "pavodra")}.get(design, ("falcon",))
+    beside = {"nopuzen": ("kekapel", "pavodra"), "verelorn": ("nopuzen", "bimepel", "pavodra")}.get(design, ("falcon",))
     gen_cfg = GenerationConfig(do_sample=False, eos_token_id=None)
     layers, T, ctx_len = args.layers or 6, args.prefill_tokens, args.prompt_len
     beside_text = "falcon (new architecture, 8 KV groups of head size 128)" if beside == ("falcon",) else ", ".join(beside)
@@ -572,6 +613,14 @@ def design_record(args):
                                 "attn_flops:pta_attn_talk_mfma": 0.0}
                     by_prompt = {"attn_bytes:pta_attn_talk_mfma": 0.0,
                                  "attn_flops:pta_attn_talk_mfma": 2.0 * (a["dim"] + a["vdim"]) * a["heads"] * T * (T + 1) / 2}
+                elif name == "verelorn":  # latent rows for one kind of layer, keys and values for another
+                    row, heads, rank = 576, VERELORN_SIZES[size]["heads"], 512
+                    kv, fl = b * (ctx_len + 1) * row * 2, 2.0 * heads * (row + rank) * T * (T + 1) / 2
+                    a = cfg.layers[2]["mixer"]
+                    by_entry = {"attn_bytes:pta_attn_mfma": b * (ctx_len + 1) * a["kv_heads"] * (a["dim"] + a["vdim"]) * 2,
+                                "attn_flops:pta_attn_mfma": 0.0}
+                    by_prompt = {"attn_bytes:pta_attn_mfma": 0.0,
+                                 "attn_flops:pta_attn_mfma": 2.0 * (a["dim"] + a["vdim"]) * a["heads"] * T * (T + 1) / 2}
                 elif name == "bimepel":  # keys and values of a token's own block of positions only
                     a = cfg.layers[0]["mixer"]
                     block = a["mask"]["size"]
@@ -615,7 +664,7 @@ def design_record(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["pavodra", "bimepel", "kekapel", "nopuzen"],
+    ap.add_argument("--design", default=None, choices=["pavodra", "bimepel", "kekapel", "nopuzen", "verelorn"],
                     help="measure that design beside the closest Falcon model at equal layer sizes and print that record "
                          "instead of the default run's (--layers, --prefill-tokens, --prompt-len and --dtype apply)")
     ap.add_argument("--design-sizes", default="2k,4k", help="with --design: which of the layer sizes 2k, 4k")

@@ -17,7 +17,6 @@ which otherwise follow from the weight file's tensors (``vdim`` where there is n
 """
 from __future__ import annotations
 
-import copy
 import dataclasses
 from typing import Any, ClassVar, Dict, List
 
@@ -80,7 +79,7 @@ class VerelornConfig(ModelConfig):
         return int(m.get(key) or m["vdim"])
 
     def sizes_from_weights(self, shapes) -> None:
-        layers = copy.deepcopy(self.layers)  # (entries of the list may be one object)
+        layers = [dict(l, mixer=dict(l["mixer"])) for l in self.layers]  # (entries of the list may be one object)
         for i, layer in enumerate(layers):
             if layer["type"] != "channel_delta":
                 continue
