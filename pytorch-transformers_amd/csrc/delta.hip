@@ -8,17 +8,30 @@
 // pta_delta_prep makes what the recurrence reads: q, k and v through a short causal convolution per channel and silu, q and
 // k to unit length per head (q times a constant), g = exp(-exp(A_log) softplus(a + dt_bias)), beta = sigmoid(b).
 //
-// pta_delta_scan runs the recurrence.  A workgroup of four waves owns (sequence, head, 64 * CPL columns p of the state) and
-// a run of tokens; a wave owns 16 * CPL columns, and its four groups of sixteen lanes hold NPT consecutive rows n each in
-// registers; sums over rows end with two exchanges between the groups.  A piece of the run's g, k, q, v and beta is staged
-// in LDS by the whole workgroup, then walked in order.  Columns never meet, so a workgroup may take any of them.
+// pta_delta_scan runs the recurrence, in one of two ways.
 //
-// Short steps are one launch from each sequence's state to its state (DELTA_WHOLE).  A long prompt is cut into chunks that
-// run side by side.  The recurrence is affine in the state: over chunk c, S_out = A_c S_in + B_c, with B_c the result from a
-// zero state and A_c (N x N) that of the unit matrix with values of zero, so:
+// Few tokens a sequence (decoding, short portions): delta_step_kernel walks each sequence's tokens from its state to its
+// state.  A workgroup of four waves owns (sequence, head, 64 columns p of the state); a wave owns sixteen columns, and its
+// four groups of sixteen lanes hold NPT consecutive rows n each in registers; sums over rows end with two exchanges between
+// the groups.  A piece of the tokens' g, k, q, v and beta is staged in LDS by the whole workgroup, then walked in order.
+//
+// Prompts: blocks of sixteen tokens as 32-bit matrix products.  With b_t = g_1 * ... * g_t inside a block (element by
+// element) and S the block's first state, the recurrence says
+//   R   = V - K^ S                        K^_t = b_t * k_t
+//   U   = (I + diag(beta) L)^-1 diag(beta) R      L_ts = sum_n k_t k_s (g_(s+1) ... g_t), s < t
+//   O   = Q^ S + A U                      Q^_t = b_t * q_t,  A_ts = sum_n q_t k_s (g_(s+1) ... g_t), s <= t
+//   S  <- diag(b_16) S + Kd^T U           Kd_s = k_s * (g_(s+1) ... g_16)
+// Every product of decays runs forward from a token to a later one, so nothing is divided by a decay and nothing can
+// overflow.  delta_block_kernel makes K^, Q^, Kd, A and the triangular inverse for all blocks at once; delta_scan_kernel walks the
+// blocks: a wave owns sixteen columns of the state as the accumulators of its row tiles, which are the second operand of the
+// products with K^ and Q^ as they lie (a lane's four rows are the four products' rows of the state).
+//
+// A long prompt of few sequences and heads is also cut into chunks that run side by side.  The recurrence is affine in the
+// state: over chunk c, S_out = A_c S_in + B_c, with B_c the result from a zero state and A_c (N x N) that of the unit matrix
+// with values of zero, so:
 //   DELTA_LOCAL   every chunk from [0 | I]: columns 0 .. P - 1 leave B_c, columns P .. P + N - 1 leave A_c;
-//   delta_carry   chunk after chunk, S_in(c + 1) = A_c S_in(c) + B_c, from the sequence's state to its state (32-bit matrix
-//                 products; A_c is a product of contractions, so nothing grows);
+//   delta_carry   chunk after chunk, S_in(c + 1) = A_c S_in(c) + B_c, from the sequence's state to its state (A_c is a
+//                 product of contractions, so nothing grows);
 //   DELTA_OUTPUT  every chunk again from its S_in, with the outputs.
 #include "common.h"
 #include "pta_kernels.h"
@@ -127,49 +140,32 @@ extern "C" int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, 
     return pta_check_launch("delta_prep");
 }
 
-template <int NPT, int CPL, int MODE>
-__global__ __launch_bounds__(256) void delta_scan_kernel(
+// y, state as pta_delta_scan has them: every sequence's tokens in order, from its state to its state
+template <int NPT>
+__global__ __launch_bounds__(256) void delta_step_kernel(
     float* __restrict__ y, const float* __restrict__ qkv, const float* __restrict__ g, const float* __restrict__ beta,
-    float* __restrict__ state, long state_ld, float* __restrict__ chunk_state, const int* __restrict__ cu_tokens,
-    const int* __restrict__ seq_slot, int heads, int G, int P, int N, int chunk, int max_chunks) {
+    float* __restrict__ state, long state_ld, const int* __restrict__ cu_tokens, const int* __restrict__ seq_slot, int heads,
+    int G, int P, int N) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     constexpr int GS = NPT + 4;      // a lane group's rows of a token in LDS, padded so that the four groups' banks differ
     constexpr int NP = 4 * GS;
-    constexpr int COLS = 64 * CPL;   // columns of a workgroup
-    const int h = blockIdx.y, kh = h / (heads / G);
-    const int s = MODE == DELTA_WHOLE ? blockIdx.z : blockIdx.z / max_chunks;
-    const int c = MODE == DELTA_WHOLE ? 0 : blockIdx.z - s * max_chunks;
+    const int h = blockIdx.y, kh = h / (heads / G), s = blockIdx.z;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int pl = lane & 15, g4 = lane >> 4;
-    const int p0 = blockIdx.x * COLS;
-    const int pw = (wave * 16 + pl) * CPL;  // the lane's first column within the workgroup's
-    const int W = MODE == DELTA_WHOLE ? P : P + N;  // columns of the stored state
-    const int used = MODE == DELTA_LOCAL ? P + N : P;
-    int t0 = cu_tokens[s];
-    int t1 = cu_tokens[s + 1];
-    if (MODE != DELTA_WHOLE) {
-        t0 += c * chunk;
-        if (t0 >= t1) return;  // the sequence has fewer chunks
-        t1 = min(t1, t0 + chunk);
-    }
-    float* sb = MODE == DELTA_WHOLE ? state + (long)seq_slot[s] * state_ld + (long)h * N * P
-                                    : chunk_state + ((long)blockIdx.z * heads + h) * N * W;
+    const int p0 = blockIdx.x * 64, pw = wave * 16 + pl, p = p0 + pw;
+    const int t0 = cu_tokens[s], t1 = cu_tokens[s + 1];
+    float* sb = state + (long)seq_slot[s] * state_ld + (long)h * N * P;
     float* g_s = lds;                          // [DELTA_PIECE][NP]
     float* k_s = g_s + DELTA_PIECE * NP;       // [DELTA_PIECE][NP]
     float* q_s = k_s + DELTA_PIECE * NP;       // [DELTA_PIECE][NP]
-    float* v_s = q_s + DELTA_PIECE * NP;       // [DELTA_PIECE][COLS]
-    float* b_s = v_s + DELTA_PIECE * COLS;     // [DELTA_PIECE]
+    float* v_s = q_s + DELTA_PIECE * NP;       // [DELTA_PIECE][64]
+    float* b_s = v_s + DELTA_PIECE * 64;       // [DELTA_PIECE]
     const int C = 2 * G * N + heads * P;
-    float S[CPL][NPT];
+    float S[NPT];
 #pragma unroll
-    for (int j = 0; j < CPL; ++j) {
-        const int p = p0 + pw + j;
-#pragma unroll
-        for (int i = 0; i < NPT; ++i) {
-            const int n = g4 * NPT + i;
-            if (MODE == DELTA_LOCAL) S[j][i] = (p >= P && n == p - P) ? 1.f : 0.f;
-            else S[j][i] = (n < N && p < P) ? sb[(long)n * W + p] : 0.f;
-        }
+    for (int i = 0; i < NPT; ++i) {
+        const int n = g4 * NPT + i;
+        S[i] = (n < N && p < P) ? sb[(long)n * P + p] : 0.f;
     }
     for (int c0 = t0; c0 < t1; c0 += DELTA_PIECE) {
         const int cnt = min(DELTA_PIECE, t1 - c0);
@@ -180,10 +176,10 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
             const float* row = qkv + (long)(c0 + tt) * C + kh * N + n;
             g_s[at] = n < N ? g[((long)(c0 + tt) * heads + h) * N + n] : 0.f;
             k_s[at] = n < N ? row[(long)G * N] : 0.f;
-            if (MODE != DELTA_LOCAL) q_s[at] = n < N ? row[0] : 0.f;
+            q_s[at] = n < N ? row[0] : 0.f;
         }
-        for (int i = threadIdx.x; i < cnt * COLS; i += 256) {
-            const int tt = i / COLS, pp = i % COLS;
+        for (int i = threadIdx.x; i < cnt * 64; i += 256) {
+            const int tt = i >> 6, pp = i & 63;
             v_s[i] = p0 + pp < P ? qkv[(long)(c0 + tt) * C + 2 * G * N + h * P + p0 + pp] : 0.f;
         }
         if (threadIdx.x < cnt) b_s[threadIdx.x] = beta[(long)(c0 + threadIdx.x) * heads + h];
@@ -192,207 +188,477 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
             const float4* gv = reinterpret_cast<const float4*>(g_s + tt * NP + g4 * GS);
             const float4* kv = reinterpret_cast<const float4*>(k_s + tt * NP + g4 * GS);
             const float4* qv = reinterpret_cast<const float4*>(q_s + tt * NP + g4 * GS);
-            const float b = b_s[tt];
-            float kk[NPT], u[CPL], o[CPL];
-#pragma unroll
-            for (int j = 0; j < CPL; ++j) u[j] = 0.f, o[j] = 0.f;
+            float u = 0.f, o = 0.f;
 #pragma unroll
             for (int i = 0; i < NPT; i += 4) {
-                const float4 gg = gv[i >> 2], k4 = kv[i >> 2];
-                kk[i] = k4.x; kk[i + 1] = k4.y; kk[i + 2] = k4.z; kk[i + 3] = k4.w;
-#pragma unroll
-                for (int j = 0; j < CPL; ++j) {
-                    S[j][i] *= gg.x; S[j][i + 1] *= gg.y; S[j][i + 2] *= gg.z; S[j][i + 3] *= gg.w;
-                    u[j] += S[j][i] * k4.x;
-                    u[j] += S[j][i + 1] * k4.y;
-                    u[j] += S[j][i + 2] * k4.z;
-                    u[j] += S[j][i + 3] * k4.w;
-                }
+                const float4 gg = gv[i >> 2], kk = kv[i >> 2];
+                S[i] *= gg.x; S[i + 1] *= gg.y; S[i + 2] *= gg.z; S[i + 3] *= gg.w;
+                u += S[i] * kk.x; u += S[i + 1] * kk.y; u += S[i + 2] * kk.z; u += S[i + 3] * kk.w;
             }
-#pragma unroll
-            for (int j = 0; j < CPL; ++j) {
-                u[j] += __shfl_xor(u[j], 16, 64);
-                u[j] += __shfl_xor(u[j], 32, 64);
-                u[j] = b * (v_s[tt * COLS + pw + j] - u[j]);
-            }
+            u += __shfl_xor(u, 16, 64);
+            u += __shfl_xor(u, 32, 64);
+            u = b_s[tt] * (v_s[tt * 64 + pw] - u);
 #pragma unroll
             for (int i = 0; i < NPT; i += 4) {
-                float4 q4 = make_float4(0.f, 0.f, 0.f, 0.f);
-                if (MODE != DELTA_LOCAL) q4 = qv[i >> 2];
-#pragma unroll
-                for (int j = 0; j < CPL; ++j) {
-                    S[j][i] += kk[i] * u[j]; S[j][i + 1] += kk[i + 1] * u[j];
-                    S[j][i + 2] += kk[i + 2] * u[j]; S[j][i + 3] += kk[i + 3] * u[j];
-                    if (MODE != DELTA_LOCAL) {
-                        o[j] += S[j][i] * q4.x;
-                        o[j] += S[j][i + 1] * q4.y;
-                        o[j] += S[j][i + 2] * q4.z;
-                        o[j] += S[j][i + 3] * q4.w;
-                    }
-                }
+                const float4 kk = kv[i >> 2], qq = qv[i >> 2];
+                S[i] += kk.x * u; S[i + 1] += kk.y * u; S[i + 2] += kk.z * u; S[i + 3] += kk.w * u;
+                o += S[i] * qq.x; o += S[i + 1] * qq.y; o += S[i + 2] * qq.z; o += S[i + 3] * qq.w;
             }
-            if (MODE != DELTA_LOCAL) {
+            o += __shfl_xor(o, 16, 64);
+            o += __shfl_xor(o, 32, 64);
+            if (g4 == 0 && p < P) y[((long)(c0 + tt) * heads + h) * P + p] = o;
+        }
+    }
 #pragma unroll
-                for (int j = 0; j < CPL; ++j) {
-                    o[j] += __shfl_xor(o[j], 16, 64);
-                    o[j] += __shfl_xor(o[j], 32, 64);
-                    const int p = p0 + pw + j;
-                    if (g4 == 0 && p < P) y[((long)(c0 + tt) * heads + h) * P + p] = o[j];
-                }
+    for (int i = 0; i < NPT; ++i) {
+        const int n = g4 * NPT + i;
+        if (n < N && p < P) sb[(long)n * P + p] = S[i];
+    }
+}
+
+// ---- blocks of sixteen tokens ------------------------------------------------------------------------------------------
+typedef float delta_f4 __attribute__((ext_vector_type(4)));
+#define DELTA_BLOCK 16
+
+template <int V>
+__device__ __forceinline__ void delta_load(const float* p, float (&v)[V]) {
+    if constexpr (V == 4) {
+        const float4 q = *reinterpret_cast<const float4*>(p);
+        v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+    } else {
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] = p[i];
+    }
+}
+
+// One workgroup per (block, head, sequence).  hat [M, heads, 3, N]: K^, Q^ and Kd of every token; ta [M, heads, 2, 16]: its row of
+// the inverse times diag(beta), and of A; the decays over the whole block take the place of its first token's row of g.
+// Thread (token s, group of RT channels): k_s carried forward over the later tokens, channel by channel, gives a column of L
+// and of A, summed over the channels by exchanges and through LDS in wave order.
+template <int RT>
+__global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ hat, float* __restrict__ ta, float* __restrict__ g,
+                                                          const float* __restrict__ qkv, const float* __restrict__ beta,
+                                                          const int* __restrict__ cu_tokens, int heads, int G, int P, int N) {
+    constexpr int NP = 16 * RT, ROW = NP + 4;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    float* g_s = lds;                    // [16][ROW]
+    float* k_s = g_s + 16 * ROW;         // [16][ROW]
+    float* q_s = k_s + 16 * ROW;         // [16][ROW]
+    float* red = q_s + 16 * ROW;         // [4 waves][2][16 t][16 s]
+    __shared__ float L_s[16][17];
+    __shared__ float b_s[16];
+    const int h = blockIdx.y, kh = h / (heads / G), s = blockIdx.z;
+    const int m0 = cu_tokens[s] + blockIdx.x * DELTA_BLOCK, t1 = cu_tokens[s + 1];
+    if (m0 >= t1) return;
+    const int cnt = min(DELTA_BLOCK, t1 - m0);
+    const int C = 2 * G * N + heads * P;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    for (int i = tid; i < 16 * NP; i += 256) {
+        const int t = i / NP, n = i - t * NP;
+        const bool in = t < cnt && n < N;
+        const float* row = qkv + (long)(m0 + t) * C + kh * N + n;
+        g_s[t * ROW + n] = in ? g[((long)(m0 + t) * heads + h) * N + n] : 1.f;  // (a token past the end changes nothing)
+        k_s[t * ROW + n] = in ? row[(long)G * N] : 0.f;
+        q_s[t * ROW + n] = in ? row[0] : 0.f;
+    }
+    if (tid < 16) b_s[tid] = tid < cnt ? beta[(long)(m0 + tid) * heads + h] : 0.f;
+    __syncthreads();
+    const int st = lane & 15, ch = (wave * 4 + (lane >> 4)) * RT;
+    float lk[16], aq[16];
+#pragma unroll
+    for (int t = 0; t < 16; ++t) lk[t] = 0.f, aq[t] = 0.f;
+    constexpr int VN = RT < 4 ? RT : 4;  // channels at a time
+#pragma unroll 1
+    for (int c0 = 0; c0 < RT; c0 += VN) {
+        const float* gp = g_s + ch + c0;
+        const float* kp = k_s + ch + c0;
+        const float* qp = q_s + ch + c0;
+        float r[VN];
+#pragma unroll
+        for (int i = 0; i < VN; ++i) r[i] = 0.f;
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float gt[VN], kt[VN], qt[VN];
+            delta_load<VN>(gp + t * ROW, gt);
+            delta_load<VN>(kp + t * ROW, kt);
+            delta_load<VN>(qp + t * ROW, qt);
+#pragma unroll
+            for (int i = 0; i < VN; ++i) {
+                r[i] = t == st ? kt[i] : r[i] * gt[i];
+                lk[t] += kt[i] * r[i];
+                aq[t] += qt[i] * r[i];
+            }
+            if ((t & 3) == 3) asm volatile("" ::: "memory");  // (not all sixteen tokens' loads at once)
+        }
+        if (st < cnt) {
+            float* to = hat + (((long)(m0 + st) * heads + h) * 3 + 2) * N + ch + c0;
+#pragma unroll
+            for (int i = 0; i < VN; ++i)
+                if (ch + c0 + i < N) to[i] = r[i];
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+        lk[t] += __shfl_xor(lk[t], 16, 64);
+        lk[t] += __shfl_xor(lk[t], 32, 64);
+        aq[t] += __shfl_xor(aq[t], 16, 64);
+        aq[t] += __shfl_xor(aq[t], 32, 64);
+        if (lane < 16) {
+            red[((wave * 2 + 0) * 16 + t) * 16 + st] = lk[t];
+            red[((wave * 2 + 1) * 16 + t) * 16 + st] = aq[t];
+        }
+    }
+    if (tid < N) {  // forward products from the block's start
+        float b = 1.f;
+        for (int t = 0; t < cnt; ++t) {
+            b *= g_s[t * ROW + tid];
+            float* to = hat + ((long)(m0 + t) * heads + h) * 3 * N + tid;
+            to[0] = b * k_s[t * ROW + tid];
+            to[N] = b * q_s[t * ROW + tid];
+        }
+        g[((long)m0 * heads + h) * N + tid] = b;
+    }
+    __syncthreads();
+    {
+        const int t = tid >> 4, sc = tid & 15;
+        float l = 0.f, a = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            l += red[((w * 2 + 0) * 16 + t) * 16 + sc];
+            a += red[((w * 2 + 1) * 16 + t) * 16 + sc];
+        }
+        L_s[t][sc] = sc < t ? l * b_s[t] : 0.f;
+        if (t < cnt) ta[((long)(m0 + t) * heads + h) * 32 + 16 + sc] = sc <= t ? a : 0.f;
+    }
+    __syncthreads();
+    if (tid < 16) {  // column tid of (I + diag(beta) L)^-1, times beta of its token
+        float x[16];
+#pragma unroll
+        for (int t = 0; t < 16; ++t) {
+            float acc = t == tid ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < t; ++j) acc -= L_s[t][j] * x[j];
+            x[t] = acc;
+            if (t < cnt) ta[((long)(m0 + t) * heads + h) * 32 + tid] = acc * b_s[tid];
+        }
+    }
+}
+
+template <int RT, int MODE>
+__global__ __launch_bounds__(256) void delta_scan_kernel(
+    float* __restrict__ y, const float* __restrict__ qkv, const float* __restrict__ hat, const float* __restrict__ ta,
+    const float* __restrict__ g, float* __restrict__ state, long state_ld, float* __restrict__ chunk_state,
+    const int* __restrict__ cu_tokens, const int* __restrict__ seq_slot, int heads, int G, int P, int N, int chunk,
+    int max_chunks) {
+    constexpr int NP = 16 * RT, ROW = NP + 4, TROW = 36;
+    constexpr int PIECES = 16 * 3 * NP / 4;                 // four elements of K^, Q^ or Kd each
+    constexpr int PER = (PIECES + 255) / 256;
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    float* hat_s = lds;                      // [3][16][ROW]
+    float* ta_s = hat_s + 3 * 16 * ROW;      // [16][TROW]
+    float* b_s = ta_s + 16 * TROW;           // [NP]
+    const int h = blockIdx.y;
+    const int s = MODE == DELTA_WHOLE ? blockIdx.z : blockIdx.z / max_chunks;
+    const int c = MODE == DELTA_WHOLE ? 0 : blockIdx.z - s * max_chunks;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, lk = lane >> 4;
+    const int p = blockIdx.x * 64 + wave * 16 + lr;
+    const int W = MODE == DELTA_WHOLE ? P : P + N;  // columns of the stored state
+    int t0 = cu_tokens[s], t1 = cu_tokens[s + 1];
+    if (MODE != DELTA_WHOLE) {
+        t0 += c * chunk;
+        if (t0 >= t1) return;  // the sequence has fewer chunks
+        t1 = min(t1, t0 + chunk);
+    }
+    float* sb = MODE == DELTA_WHOLE ? state + (long)seq_slot[s] * state_ld + (long)h * N * P
+                                    : chunk_state + ((long)blockIdx.z * heads + h) * N * W;
+    const int C = 2 * G * N + heads * P;
+    const bool vec = (N & 3) == 0;
+    delta_f4 S[RT];
+#pragma unroll
+    for (int r = 0; r < RT; ++r)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int n = r * 16 + lk * 4 + e;
+            if (MODE == DELTA_LOCAL) S[r][e] = (p >= P && n == p - P) ? 1.f : 0.f;
+            else S[r][e] = (n < N && p < P) ? sb[(long)n * W + p] : 0.f;
+        }
+    // what a block needs, asked for one block ahead
+    float4 ph[PER];
+    float pt[2], pb, pv[4];
+    auto fetch = [&](int m0) {
+        const int cnt = t1 - m0;  // (tokens from sixteen on belong to the next block; none at or below zero)
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            const int i = tid + j * 256;
+            const int t = i / (3 * NP / 4), rest = i - t * (3 * NP / 4), which = rest / (NP / 4), n = (rest - which * (NP / 4)) * 4;
+            ph[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (i >= PIECES || t >= cnt || (MODE == DELTA_LOCAL && which == 1)) continue;
+            const float* from = hat + (((long)(m0 + t) * heads + h) * 3 + which) * N + n;
+            if (vec) {
+                if (n < N) ph[j] = *reinterpret_cast<const float4*>(from);
+            } else {
+                if (n < N) ph[j].x = from[0];
+                if (n + 1 < N) ph[j].y = from[1];
+                if (n + 2 < N) ph[j].z = from[2];
+                if (n + 3 < N) ph[j].w = from[3];
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+            const int i = tid + j * 256, t = i >> 5;
+            pt[j] = t < cnt ? ta[((long)(m0 + t) * heads + h) * 32 + (i & 31)] : 0.f;
+        }
+        pb = (tid < N && cnt > 0) ? g[((long)m0 * heads + h) * N + tid] : 0.f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+            pv[e] = (lk * 4 + e < cnt && p < P) ? qkv[(long)(m0 + lk * 4 + e) * C + 2 * G * N + h * P + p] : 0.f;
+    };
+    fetch(t0);
+    for (int m0 = t0; m0 < t1; m0 += DELTA_BLOCK) {
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            const int i = tid + j * 256;
+            const int t = i / (3 * NP / 4), rest = i - t * (3 * NP / 4), which = rest / (NP / 4), n = (rest - which * (NP / 4)) * 4;
+            if (i < PIECES) *reinterpret_cast<float4*>(hat_s + (which * 16 + t) * ROW + n) = ph[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 2; ++j) ta_s[((tid + j * 256) >> 5) * TROW + ((tid + j * 256) & 31)] = pt[j];
+        if (tid < NP) b_s[tid] = pb;
+        delta_f4 R0, R1 = {0.f, 0.f, 0.f, 0.f}, O0 = {0.f, 0.f, 0.f, 0.f}, O1 = {0.f, 0.f, 0.f, 0.f}, U = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) R0[e] = pv[e];
+        __syncthreads();
+        fetch(m0 + DELTA_BLOCK);
+        const float* kh_row = hat_s + lr * ROW + lk * 4;
+        const float* qh_row = kh_row + 16 * ROW;
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+            const float4 a4 = *reinterpret_cast<const float4*>(kh_row + r * 16);
+            const float a[4] = {-a4.x, -a4.y, -a4.z, -a4.w};
+            delta_f4& R = (r & 1) ? R1 : R0;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) R = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], S[r][e], R, 0, 0, 0);
+        }
+        if (MODE != DELTA_LOCAL) {
+#pragma unroll
+            for (int r = 0; r < RT; ++r) {
+                const float4 a4 = *reinterpret_cast<const float4*>(qh_row + r * 16);
+                const float a[4] = {a4.x, a4.y, a4.z, a4.w};
+                delta_f4& O = (r & 1) ? O1 : O0;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) O = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], S[r][e], O, 0, 0, 0);
+            }
+        }
+        {
+            const float4 a4 = *reinterpret_cast<const float4*>(ta_s + lr * TROW + lk * 4);
+            const float a[4] = {a4.x, a4.y, a4.z, a4.w};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) U = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], R0[e] + R1[e], U, 0, 0, 0);
+        }
+        const float* kd = hat_s + 32 * ROW + lk * 4 * ROW + lr;
+#pragma unroll
+        for (int r = 0; r < RT; ++r) {
+            const float4 b4 = *reinterpret_cast<const float4*>(b_s + r * 16 + lk * 4);
+            S[r][0] *= b4.x; S[r][1] *= b4.y; S[r][2] *= b4.z; S[r][3] *= b4.w;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) S[r] = __builtin_amdgcn_mfma_f32_16x16x4f32(kd[e * ROW + r * 16], U[e], S[r], 0, 0, 0);
+        }
+        if (MODE != DELTA_LOCAL) {
+            const float4 a4 = *reinterpret_cast<const float4*>(ta_s + lr * TROW + 16 + lk * 4);
+            const float a[4] = {a4.x, a4.y, a4.z, a4.w};
+#pragma unroll
+            for (int e = 0; e < 4; ++e) O0 = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], U[e], O0, 0, 0, 0);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int m = m0 + lk * 4 + e;
+                if (m < t1 && p < P) y[((long)m * heads + h) * P + p] = O0[e] + O1[e];
             }
         }
     }
     if (MODE != DELTA_OUTPUT) {
+        const int used = MODE == DELTA_LOCAL ? P + N : P;
 #pragma unroll
-        for (int j = 0; j < CPL; ++j) {
-            const int p = p0 + pw + j;
+        for (int r = 0; r < RT; ++r)
 #pragma unroll
-            for (int i = 0; i < NPT; ++i) {
-                const int n = g4 * NPT + i;
-                if (n < N && p < used) sb[(long)n * W + p] = S[j][i];
+            for (int e = 0; e < 4; ++e) {
+                const int n = r * 16 + lk * 4 + e;
+                if (n < N && p < used) sb[(long)n * W + p] = S[r][e];
             }
-        }
     }
 }
 
-// chunk after chunk: what a chunk starts from takes the place of B_c, the sequence's state moves to its end.  A workgroup
-// owns (sequence, head, sixteen columns); the state stands in LDS between two chunks.  N a multiple of 16: products on the
-// matrix cores in 32-bit, a wave a tile of sixteen rows in turn; a lane's four consecutive elements of a row of A_c are
-// four products' operands (the order of a sum over rows of the state is that of the products).
-typedef float delta_f4 __attribute__((ext_vector_type(4)));
-
-template <bool MFMA>
-__global__ __launch_bounds__(256) void delta_carry_kernel(float* __restrict__ state, long state_ld, float* __restrict__ chunk_state,
+// chunk after chunk: what a chunk starts from takes the place of B_c, the sequence's state moves to its end.  A workgroup of
+// eight waves owns (sequence, head, sixteen columns); a wave forms RTW tiles of sixteen rows; the state stands in LDS between
+// two chunks, and the next chunk's A_c and B_c are asked for while this one's products run.  VEC: A_c's rows can be loaded
+// four elements at a time.
+template <int RTW, bool VEC>
+__global__ __launch_bounds__(512) void delta_carry_kernel(float* __restrict__ state, long state_ld, float* __restrict__ chunk_state,
                                                           const int* __restrict__ cu_tokens, const int* __restrict__ seq_slot,
                                                           int heads, int P, int N, int chunk, int max_chunks) {
-    __shared__ float S_s[256 * 17];  // [N][16 + 1]
+    constexpr int RT = 8 * RTW;      // row tiles, and pieces of sixteen elements of a row of A_c
+    __shared__ float S_s[RT * 16 * 17];
     const int h = blockIdx.y, s = blockIdx.z, p0 = blockIdx.x * 16;
     const int n_chunks = (cu_tokens[s + 1] - cu_tokens[s] + chunk - 1) / chunk;
-    const int W = P + N;
-    const int col = threadIdx.x & 15, rg = threadIdx.x >> 4;  // sixteen groups of rows
-    const bool in = p0 + col < P;
-    float* sp = state + (long)seq_slot[s] * state_ld + (long)h * N * P + p0 + col;
-    for (int n = rg; n < N; n += 16) S_s[n * 17 + col] = in ? sp[(long)n * P] : 0.f;
-    __syncthreads();
+    if (n_chunks <= 0) return;
+    const long W = P + N;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lk = lane >> 4;
-    for (int c = 0; c < n_chunks; ++c) {
-        float* cs = chunk_state + (((long)s * max_chunks + c) * heads + h) * (long)N * W;
-        float next[16];  // rows this thread forms: (wave-tile rows) or rg, rg + 16, ...
-        if constexpr (MFMA) {
+    const bool in = p0 + lr < P;
+    float* sp = state + (long)seq_slot[s] * state_ld + (long)h * N * P + p0 + lr;
+    float4 a[RTW][RT];
+    delta_f4 S[RTW], B[RTW];
+    auto base = [&](int c) { return chunk_state + (((long)s * max_chunks + c) * heads + h) * (long)N * W; };
+    auto fetch = [&](int c) {
+        const float* cs = base(c);
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int r0 = (wave + 4 * j) * 16;
-                if (r0 >= N) continue;
-                delta_f4 acc;
+        for (int j = 0; j < RTW; ++j) {
+            const int r0 = (wave + 8 * j) * 16;
+            const float* row = cs + (long)(r0 + lr) * W + P;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) acc[e] = p0 + lr < P ? cs[(long)(r0 + lk * 4 + e) * W + p0 + lr] : 0.f;
-                const float* arow = cs + (long)(r0 + lr) * W + P + lk * 4;
-                for (int m0 = 0; m0 < N; m0 += 16) {
-                    float a[4];
-#pragma unroll
-                    for (int e = 0; e < 4; ++e) a[e] = arow[m0 + e];
-#pragma unroll
-                    for (int e = 0; e < 4; ++e)
-                        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], S_s[(m0 + lk * 4 + e) * 17 + lr], acc, 0, 0, 0);
+            for (int m = 0; m < RT; ++m) {
+                const int k = m * 16 + lk * 4;
+                a[j][m] = make_float4(0.f, 0.f, 0.f, 0.f);
+                if (r0 + lr >= N) continue;
+                if (VEC) {
+                    if (k < N) a[j][m] = *reinterpret_cast<const float4*>(row + k);
+                } else {
+                    if (k < N) a[j][m].x = row[k];
+                    if (k + 1 < N) a[j][m].y = row[k + 1];
+                    if (k + 2 < N) a[j][m].z = row[k + 2];
+                    if (k + 3 < N) a[j][m].w = row[k + 3];
                 }
-#pragma unroll
-                for (int e = 0; e < 4; ++e) next[j * 4 + e] = acc[e];
             }
-        } else {
 #pragma unroll
-            for (int j = 0; j < 16; ++j) {
-                const int n = rg + 16 * j;
-                if (n >= N) continue;
-                const float* arow = cs + (long)n * W + P;
-                float acc = in ? cs[(long)n * W + p0 + col] : 0.f;
-                for (int m = 0; m < N; ++m) acc += arow[m] * S_s[m * 17 + col];
-                next[j] = acc;
+            for (int e = 0; e < 4; ++e) {
+                const int n = r0 + lk * 4 + e;
+                B[j][e] = (in && n < N) ? cs[(long)n * W + p0 + lr] : 0.f;
             }
         }
-        __syncthreads();  // every sum has been formed: B_c and the state may be replaced
-        for (int n = rg; n < N; n += 16)
-            if (in) cs[(long)n * W + p0 + col] = S_s[n * 17 + col];
-        __syncthreads();
-        if constexpr (MFMA) {
+    };
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int r0 = (wave + 4 * j) * 16;
-                if (r0 >= N) continue;
+    for (int j = 0; j < RTW; ++j)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) S_s[(r0 + lk * 4 + e) * 17 + lr] = next[j * 4 + e];
-            }
-        } else {
-#pragma unroll
-            for (int j = 0; j < 16; ++j)
-                if (rg + 16 * j < N) S_s[(rg + 16 * j) * 17 + col] = next[j];
+        for (int e = 0; e < 4; ++e) {
+            const int n = (wave + 8 * j) * 16 + lk * 4 + e;
+            S[j][e] = (in && n < N) ? sp[(long)n * P] : 0.f;
         }
+    fetch(0);
+    for (int c = 0; c < n_chunks; ++c) {
+        float* cs = base(c);
+#pragma unroll
+        for (int j = 0; j < RTW; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                const int n = (wave + 8 * j) * 16 + lk * 4 + e;
+                S_s[n * 17 + lr] = S[j][e];
+                if (in && n < N) cs[(long)n * W + p0 + lr] = S[j][e];  // (B_c of these elements is this lane's own, already here)
+            }
         __syncthreads();
+        delta_f4 acc[RTW][2];
+#pragma unroll
+        for (int j = 0; j < RTW; ++j) acc[j][0] = B[j], acc[j][1] = delta_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int m = 0; m < RT; ++m) {
+            float b[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) b[e] = S_s[(m * 16 + lk * 4 + e) * 17 + lr];
+#pragma unroll
+            for (int j = 0; j < RTW; ++j) {
+                const float av[4] = {a[j][m].x, a[j][m].y, a[j][m].z, a[j][m].w};
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    acc[j][m & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(av[e], b[e], acc[j][m & 1], 0, 0, 0);
+            }
+        }
+        if (c + 1 < n_chunks) fetch(c + 1);
+#pragma unroll
+        for (int j = 0; j < RTW; ++j) S[j] = acc[j][0] + acc[j][1];
+        __syncthreads();  // everyone has read the state that the next turn replaces
     }
-    if (n_chunks > 0)
-        for (int n = rg; n < N; n += 16)
-            if (in) sp[(long)n * P] = S_s[n * 17 + col];
+#pragma unroll
+    for (int j = 0; j < RTW; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int n = (wave + 8 * j) * 16 + lk * 4 + e;
+            if (in && n < N) sp[(long)n * P] = S[j][e];
+        }
 }
 
-template <int NPT, int CPL, int MODE>
-static void launch_delta_mode(const dim3& grid, float* y, const float* qkv, const float* g, const float* beta, float* state,
-                              long state_ld, float* chunk_state, const int* cu_tokens, const int* seq_slot, int heads, int G, int P,
-                              int N, int chunk, int max_chunks, hipStream_t s) {
-    constexpr size_t lds = (size_t)DELTA_PIECE * (3 * 4 * (NPT + 4) + 64 * CPL + 1) * sizeof(float);
-    static_assert(lds <= 64 * 1024, "the piece's rows fit the LDS a launch may ask for without saying so");
-    hipLaunchKernelGGL((delta_scan_kernel<NPT, CPL, MODE>), grid, dim3(256), lds, s, y, qkv, g, beta, state, state_ld, chunk_state,
-                       cu_tokens, seq_slot, heads, G, P, N, chunk, max_chunks);
-}
+struct DeltaLaunch {
+    float* y; const float* qkv; float* g; const float* beta; float* state; long state_ld;
+    float *hat, *ta, *chunk_state;
+    const int *cu_tokens, *seq_slot;
+    int n_seqs, max_new, heads, G, P, N, chunk, max_chunks;
+    hipStream_t s;
+};
 
 template <int NPT>
-static int launch_delta(float* y, const float* qkv, const float* g, const float* beta, float* state, long state_ld,
-                        float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int heads, int G,
-                        int P, int N, int chunk, int max_chunks, hipStream_t s) {
-#define DELTA_ARGS y, qkv, g, beta, state, state_ld, chunk_state, cu_tokens, seq_slot, heads, G, P, N, chunk, max_chunks, s
-    constexpr int WIDE = NPT <= 32 ? 2 : 1;  // columns a lane where a launch is bound by its reads of LDS, not by its length
-    auto tiles = [](int cols, int per) { return (unsigned)((cols + per - 1) / per); };
-    if (max_chunks <= 1) {
-        launch_delta_mode<NPT, 1, DELTA_WHOLE>(dim3(tiles(P, 64), heads, n_seqs), DELTA_ARGS);
+static int launch_delta_steps(const DeltaLaunch& d) {
+    constexpr size_t lds = (size_t)DELTA_PIECE * (3 * 4 * (NPT + 4) + 64 + 1) * sizeof(float);
+    static_assert(lds <= 64 * 1024, "a piece's rows fit the LDS a launch may ask for without saying so");
+    hipLaunchKernelGGL(delta_step_kernel<NPT>, dim3((d.P + 63) / 64, d.heads, d.n_seqs), dim3(256), lds, d.s, d.y, d.qkv, d.g, d.beta,
+                       d.state, d.state_ld, d.cu_tokens, d.seq_slot, d.heads, d.G, d.P, d.N);
+    return pta_check_launch("delta_scan");
+}
+
+template <int RT>
+static int launch_delta_blocks(const DeltaLaunch& d) {
+    constexpr size_t block_lds = (size_t)(3 * 16 * (16 * RT + 4) + 4 * 2 * 256) * sizeof(float);
+    constexpr size_t scan_lds = (size_t)(3 * 16 * (16 * RT + 4) + 16 * 36 + 16 * RT) * sizeof(float);
+    static_assert(block_lds <= 62 * 1024 && scan_lds <= 64 * 1024, "a block's rows fit the LDS a launch may ask for without saying so");
+    hipLaunchKernelGGL(delta_block_kernel<RT>, dim3((d.max_new + DELTA_BLOCK - 1) / DELTA_BLOCK, d.heads, d.n_seqs), dim3(256), block_lds,
+                       d.s, d.hat, d.ta, d.g, d.qkv, d.beta, d.cu_tokens, d.heads, d.G, d.P, d.N);
+#define DELTA_SCAN(MODE_, COLS_, RUNS_)                                                                                          \
+    hipLaunchKernelGGL((delta_scan_kernel<RT, MODE_>), dim3(((COLS_) + 63) / 64, d.heads, (RUNS_)), dim3(256), scan_lds, d.s, d.y,   \
+                       d.qkv, d.hat, d.ta, d.g, d.state, d.state_ld, d.chunk_state, d.cu_tokens, d.seq_slot, d.heads, d.G, d.P, d.N, \
+                       d.chunk, d.max_chunks)
+    if (d.max_chunks <= 1) {
+        DELTA_SCAN(DELTA_WHOLE, d.P, d.n_seqs);
         return pta_check_launch("delta_scan");
     }
-    const unsigned runs = (unsigned)(n_seqs * max_chunks);
-    if (P + N > 64) launch_delta_mode<NPT, WIDE, DELTA_LOCAL>(dim3(tiles(P + N, 64 * WIDE), heads, runs), DELTA_ARGS);
-    else launch_delta_mode<NPT, 1, DELTA_LOCAL>(dim3(tiles(P + N, 64), heads, runs), DELTA_ARGS);
-    const dim3 carry((P + 15) / 16, heads, n_seqs);
-    if (N % 16 == 0)
-        hipLaunchKernelGGL(delta_carry_kernel<true>, carry, dim3(256), 0, s, state, state_ld, chunk_state, cu_tokens, seq_slot, heads,
-                           P, N, chunk, max_chunks);
-    else
-        hipLaunchKernelGGL(delta_carry_kernel<false>, carry, dim3(256), 0, s, state, state_ld, chunk_state, cu_tokens, seq_slot, heads,
-                           P, N, chunk, max_chunks);
-    if (P > 64) launch_delta_mode<NPT, WIDE, DELTA_OUTPUT>(dim3(tiles(P, 64 * WIDE), heads, runs), DELTA_ARGS);
-    else launch_delta_mode<NPT, 1, DELTA_OUTPUT>(dim3(tiles(P, 64), heads, runs), DELTA_ARGS);
-#undef DELTA_ARGS
+    DELTA_SCAN(DELTA_LOCAL, d.P + d.N, d.n_seqs * d.max_chunks);
+    const dim3 carry((d.P + 15) / 16, d.heads, d.n_seqs);
+    const bool vec = d.N % 4 == 0 && d.P % 4 == 0;
+    auto kern = d.N <= 128 ? (vec ? delta_carry_kernel<1, true> : delta_carry_kernel<1, false>)
+                           : (vec ? delta_carry_kernel<2, true> : delta_carry_kernel<2, false>);
+    hipLaunchKernelGGL(kern, carry, dim3(512), 0, d.s, d.state, d.state_ld, d.chunk_state, d.cu_tokens, d.seq_slot, d.heads, d.P, d.N,
+                       d.chunk, d.max_chunks);
+    DELTA_SCAN(DELTA_OUTPUT, d.P, d.n_seqs * d.max_chunks);
+#undef DELTA_SCAN
     return pta_check_launch("delta_scan");
 }
 
 // y [M, heads * P], qkv [M, 2 * kv_heads * N + heads * P], g [M, heads * N], beta [M, heads], all 32-bit and dense; state
-// [slots, >= heads * N * P] rows state_ld apart.  chunk_state [n_seqs * max_chunks, heads, N, P + N] is scratch for steps whose
-// longest sequence is cut into max_chunks > 1 chunks of `chunk` tokens; else unused.
-extern "C" int pta_delta_scan(float* y, const float* qkv, const float* g, const float* beta, float* state, long state_ld,
-                              float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int heads,
-                              int kv_heads, int P, int N, int chunk, int max_chunks, void* stream) {
+// [slots, >= heads * N * P] rows state_ld apart.  hat [M, heads, 3, N] and ta [M, heads, 2, 16] given (scratch): blocks of sixteen
+// tokens; g is then written over.  Without them the tokens are walked one by one.  chunk_state [n_seqs * max_chunks, heads, N,
+// P + N] is scratch for steps whose longest sequence is cut into max_chunks > 1 chunks of `chunk` tokens (a multiple of 16).
+extern "C" int pta_delta_scan(float* y, const float* qkv, float* g, const float* beta, float* state, long state_ld, float* hat,
+                              float* ta, float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new,
+                              int heads, int kv_heads, int P, int N, int chunk, int max_chunks, void* stream) {
     PTA_REQUIRE(n_seqs > 0 && max_new > 0 && heads > 0 && kv_heads > 0 && P > 0 && N > 0, "delta_scan: sizes must be positive");
     PTA_REQUIRE(heads % kv_heads == 0, "delta_scan: %d heads are no multiple of %d key heads", heads, kv_heads);
     PTA_REQUIRE(N <= 256, "delta_scan: keys of %d elements are more than the 256 rows of state the kernel holds", N);
     PTA_REQUIRE(heads <= 65535 && n_seqs <= 65535, "delta_scan: too many heads or sequences for one launch");
     PTA_REQUIRE(y && qkv && g && beta && state && cu_tokens && seq_slot, "delta_scan: null pointer");
     PTA_REQUIRE(state_ld >= (long)heads * N * P, "delta_scan: state rows lie closer together than they are long");
-    PTA_REQUIRE(max_chunks >= 1 && (max_chunks == 1 || (chunk > 0 && chunk_state && (long)max_chunks * chunk >= max_new)),
-                "delta_scan: chunks need their size, enough of them and scratch memory");
+    PTA_REQUIRE((hat == nullptr) == (ta == nullptr), "delta_scan: blocks need all of their scratch memory");
+    PTA_REQUIRE(max_chunks >= 1 && (max_chunks == 1 || (hat && chunk > 0 && chunk % DELTA_BLOCK == 0 && chunk_state &&
+                                                        (long)max_chunks * chunk >= max_new)),
+                "delta_scan: chunks need their size, a multiple of %d, enough of them and scratch memory", DELTA_BLOCK);
     PTA_REQUIRE((long)n_seqs * max_chunks <= 65535, "delta_scan: %ld chunks are more than one launch takes", (long)n_seqs * max_chunks);
-    hipStream_t s = (hipStream_t)stream;
-#define DELTA_LAUNCH(NPT_) return launch_delta<NPT_>(y, qkv, g, beta, state, state_ld, chunk_state, cu_tokens, seq_slot, n_seqs, \
-                                                     max_new, heads, kv_heads, P, N, chunk, max_chunks, s)
-    const int npt = (N + 3) / 4;
-    if (npt <= 4) DELTA_LAUNCH(4);
-    if (npt <= 8) DELTA_LAUNCH(8);
-    if (npt <= 16) DELTA_LAUNCH(16);
-    if (npt <= 32) DELTA_LAUNCH(32);
-    DELTA_LAUNCH(64);
-#undef DELTA_LAUNCH
+    PTA_REQUIRE(((uintptr_t)hat % 16) == 0 && ((uintptr_t)chunk_state % 16) == 0, "delta_scan: scratch memory must be 16-byte aligned");
+    const DeltaLaunch d{y, qkv, g, beta, state, state_ld, hat, ta, chunk_state, cu_tokens, seq_slot, n_seqs, max_new, heads, kv_heads,
+                        P, N, chunk, max_chunks, (hipStream_t)stream};
+    if (hat) {
+        if (N <= 16) return launch_delta_blocks<1>(d);
+        if (N <= 32) return launch_delta_blocks<2>(d);
+        if (N <= 64) return launch_delta_blocks<4>(d);
+        if (N <= 128) return launch_delta_blocks<8>(d);
+        return launch_delta_blocks<16>(d);
+    }
+    if (N <= 16) return launch_delta_steps<4>(d);
+    if (N <= 32) return launch_delta_steps<8>(d);
+    if (N <= 64) return launch_delta_steps<16>(d);
+    if (N <= 128) return launch_delta_steps<32>(d);
+    return launch_delta_steps<64>(d);
 }

@@ -340,9 +340,9 @@ int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, const void*
                    const void* a, long a_ld, const void* b, long b_ld, const float* A_log, const float* dt_bias, float* tail,
                    long tail_ld, const int* cu_tokens, const int* token_seq, const int* seq_slot, int several, int n_seqs, int M,
                    int heads, int kv_heads, int N, int P, int taps, float q_scale, float norm_eps, int dtype, void* stream);
-int pta_delta_scan(float* y, const float* qkv, const float* g, const float* beta, float* state, long state_ld, float* chunk_state,
-                   const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int heads, int kv_heads, int P, int N,
-                   int chunk, int max_chunks, void* stream);
+int pta_delta_scan(float* y, const float* qkv, float* g, const float* beta, float* state, long state_ld, float* hat, float* ta,
+                   float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int heads, int kv_heads,
+                   int P, int N, int chunk, int max_chunks, void* stream);
 
 // ---- linear attention with a decay per head (linear_attn.hip) ---------------------------------------------------------
 int pta_decay_scan(float* y, const void* q, const void* k, const void* v, long ld, const float* decay, float* state,

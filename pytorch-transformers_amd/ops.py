@@ -228,8 +228,8 @@ def _entry_cost(name: str, a) -> tuple:
         M, heads, G, N, P = float(a[21]), a[22], a[23], a[24], a[25]
         return (M * (2 * G * N + heads * (P + N)) * (el(a[29]) + 4.0), 0.0)
     if name == "pta_delta_scan":  # q, k, v, g in, o out, all 32-bit; seven operations per state element and token
-        M, heads, G, P, N = float(timing_hint.get("rows", 0)), a[11], a[12], a[13], a[14]
-        state = 8.0 * a[9] * heads * N * P
+        M, heads, G, P, N = float(timing_hint.get("rows", 0)), a[13], a[14], a[15], a[16]
+        state = 8.0 * a[11] * heads * N * P
         return (M * (2 * G * N + heads * (2 * P + N)) * 4.0 + state, 7.0 * M * heads * N * P)
     if name == "pta_glu":
         return (float(a[4]) * a[5] * 3 * el(a[9]), 0.0)
@@ -1894,7 +1894,9 @@ def conv_add(x: torch.Tensor, w: torch.Tensor, tail: Optional[torch.Tensor], ctx
 
 
 # ---- the gated delta rule with a decay per key channel --------------------------------------------------------------
-DELTA_CHUNK_TOKENS = 128  # a sequence that brings more than twice as many tokens is cut into chunks that run side by side
+DELTA_BLOCKS_FROM = 24  # a step in which some sequence brings so many tokens runs blocks of sixteen as matrix products
+DELTA_CHUNK_TOKENS = 256  # a sequence that brings more than twice as many is cut into chunks that run side by side ...
+DELTA_CHUNK_WAVES = 512  # ... where the launch would otherwise have fewer waves (sixteen columns of a head's state each)
 
 
 def delta_prep(qkv: torch.Tensor, conv: torch.Tensor, a: torch.Tensor, b: torch.Tensor, a_log, dt_bias, tail, ctx, heads: int,
@@ -1935,7 +1937,8 @@ def delta_prep(qkv: torch.Tensor, conv: torch.Tensor, a: torch.Tensor, b: torch.
 def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: torch.Tensor, ctx, heads: int, kv_heads: int,
                key_dim: int, value_dim: int) -> torch.Tensor:
     """Per head ``S <- diag(g) S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q`` over every sequence's tokens,
-    from and into its row of ``state`` ``[slots, heads * key_dim * value_dim]``; inputs as ``delta_prep`` returns them.
+    from and into its row of ``state`` ``[slots, heads * key_dim * value_dim]``; inputs as ``delta_prep`` returns them
+    (``g`` may be written over).
     Returns o ``[tokens, heads * value_dim]``; all 32-bit."""
     C = 2 * kv_heads * key_dim + heads * value_dim
     M = qkv.shape[0]
@@ -1950,14 +1953,17 @@ def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: to
     timing_hint["rows"] = M
     longest = int(max(ctx.new_tokens))
     chunk, chunks = DELTA_CHUNK_TOKENS, 1
-    if longest > 2 * chunk:
-        chunks = (longest + chunk - 1) // chunk
-    chunk_state = None
+    hat = ta = chunk_state = None
+    if longest >= DELTA_BLOCKS_FROM:
+        hat = torch.empty((M, heads, 3, key_dim), dtype=torch.float32, device=qkv.device)
+        ta = torch.empty((M, heads, 2, 16), dtype=torch.float32, device=qkv.device)
+        if longest > 2 * chunk and n * heads * ((value_dim + 15) // 16) < DELTA_CHUNK_WAVES:
+            chunks = (longest + chunk - 1) // chunk
     if chunks > 1:
         chunk_state = torch.empty((n * chunks, heads, key_dim, value_dim + key_dim), dtype=torch.float32, device=qkv.device)
     if M:
-        _call("pta_delta_scan", _ptr(y), _ptr(qkv), _ptr(g), _ptr(beta), _ptr(state), ctypes.c_long(state_ld), _ptr(chunk_state),
-              _ptr(ctx.cu_tokens), _ptr(ctx.seq_slot), n, longest, heads, kv_heads, value_dim, key_dim, chunk, chunks, _stream())
+        _call("pta_delta_scan", _ptr(y), _ptr(qkv), _ptr(g), _ptr(beta), _ptr(state), ctypes.c_long(state_ld), _ptr(hat), _ptr(ta),
+              _ptr(chunk_state), _ptr(ctx.cu_tokens), _ptr(ctx.seq_slot), n, longest, heads, kv_heads, value_dim, key_dim, chunk, chunks, _stream())
     return y
 
 
