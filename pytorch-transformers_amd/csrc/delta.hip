@@ -36,29 +36,38 @@
 #include "common.h"
 #include "pta_kernels.h"
 
+#include <algorithm>
+
 #define DELTA_PIECE 16
 #define DELTA_MAX_TAPS 16
 enum { DELTA_WHOLE = 0, DELTA_LOCAL = 1, DELTA_OUTPUT = 2 };
 
 __device__ __forceinline__ float softplus_32(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
-// One wave per (token, unit): units are the q heads, the k heads, the value heads and the heads' decays (with beta).
-template <typename T>
-__global__ __launch_bounds__(64) void delta_prep_kernel(
+// One wave per (PREP_TOKENS tokens, unit): units are the q heads, the k heads, the value heads and the heads' decays (with
+// beta); a unit's convolution weights stay in registers over its tokens.
+#define PREP_TOKENS 4
+
+template <typename T, int KMAX>
+__global__ __launch_bounds__(256) void delta_prep_kernel(
     float* __restrict__ qkv, float* __restrict__ g, float* __restrict__ beta, const T* __restrict__ q, const T* __restrict__ k,
     const T* __restrict__ v, long ld, const float* __restrict__ conv, const T* __restrict__ a, long a_ld,
     const T* __restrict__ b, long b_ld, const float* __restrict__ A_log, const float* __restrict__ dt_bias,
     float* __restrict__ tail, long tail_ld, const int* __restrict__ cu_tokens, const int* __restrict__ token_seq,
-    const int* __restrict__ seq_slot, int move_tail, int heads, int G, int N, int P, int K, float q_scale, float norm_eps) {
-    const int m = blockIdx.x, unit = blockIdx.y, lane = threadIdx.x;
+    const int* __restrict__ seq_slot, int move_tail, int M, int heads, int G, int N, int P, int K, float q_scale, float norm_eps) {
+    const int unit = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int m0 = blockIdx.x * PREP_TOKENS, m1 = min(M, m0 + PREP_TOKENS);
+    if (unit >= 2 * G + 2 * heads) return;
     if (unit >= 2 * G + heads) {  // a head's decays and step size
         const int h = unit - 2 * G - heads;
         const float rate = expf(A_log[h]);
         for (int e = lane; e < N; e += PTA_WAVE) {
             const int at = h * N + e;
-            g[(long)m * heads * N + at] = expf(-rate * softplus_32(Io<T>::ld(a + (long)m * a_ld + at) + dt_bias[at]));
+            const float bias = dt_bias[at];
+            for (int m = m0; m < m1; ++m)
+                g[(long)m * heads * N + at] = expf(-rate * softplus_32(Io<T>::ld(a + (long)m * a_ld + at) + bias));
         }
-        if (lane == 0) beta[(long)m * heads + h] = 1.0f / (1.0f + expf(-Io<T>::ld(b + (long)m * b_ld + h)));
+        if (lane < m1 - m0) beta[(long)(m0 + lane) * heads + h] = 1.0f / (1.0f + expf(-Io<T>::ld(b + (long)(m0 + lane) * b_ld + h)));
         return;
     }
     const bool is_v = unit >= 2 * G, is_q = unit < G;
@@ -66,36 +75,77 @@ __global__ __launch_bounds__(64) void delta_prep_kernel(
     const T* src = (is_v ? v : is_q ? q : k) + (long)local * len;
     const int c0 = is_v ? 2 * G * N + local * P : unit * N;  // first channel of the head in q | k | v
     const int C = 2 * G * N + heads * P;
-    const int s = token_seq[m], first = cu_tokens[s], j = m - first;
-    float* tl = tail + (K > 1 ? (long)seq_slot[s] * tail_ld : 0L);
-    float y[4], ss = 0.f;
+    // whether every input of these tokens is a row of this step: they are then asked for all at once
+    const bool inside = m1 - m0 == PREP_TOKENS && token_seq[m0] == token_seq[m1 - 1] && m0 - cu_tokens[token_seq[m0]] >= K - 1;
     for (int e0 = 0; e0 < len; e0 += 4 * PTA_WAVE) {  // (heads of q and k fit one round)
+        float w[4][KMAX];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int e = e0 + lane + r * PTA_WAVE, c = c0 + e;
-            y[r] = 0.f;
-            if (e >= len) continue;
-            const float now = Io<T>::ld(src + (long)m * ld + e);
-            float acc = 0.f;
-            for (int kk = 0; kk + 1 < K; ++kk) {
-                const int jj = j - (K - 1 - kk);
-                const float before = jj >= 0 ? Io<T>::ld(src + (long)(first + jj) * ld + e) : tl[(long)(K - 1 + jj) * C + c];
-                acc += conv[(long)kk * C + c] * before;
-                if (move_tail && kk > 0) tl[(long)(kk - 1) * C + c] = before;  // (the sequence's one token: before is tail[kk])
-            }
-            if (move_tail && K > 1) tl[(long)(K - 2) * C + c] = now;
-            acc += conv[(long)(K - 1) * C + c] * now;
-            y[r] = acc / (1.0f + expf(-acc));
-            ss += y[r] * y[r];
-            if (is_v) qkv[(long)m * C + c] = y[r];
-        }
-    }
-    if (is_v) return;
-    const float inv = (is_q ? q_scale : 1.0f) / sqrtf(wave_sum(ss) + norm_eps);
+            const int e = e0 + lane + r * PTA_WAVE;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const int e = lane + r * PTA_WAVE;
-        if (e < len) qkv[(long)m * C + c0 + e] = y[r] * inv;
+            for (int kk = 0; kk < KMAX; ++kk)  // (fewer taps: zeros in front)
+                w[r][kk] = (e < len && kk >= KMAX - K) ? conv[(long)(kk - (KMAX - K)) * C + c0 + e] : 0.f;
+        }
+        float x[4][PREP_TOKENS + KMAX - 1];  // row m0 - (KMAX - 1) + i
+        if (KMAX <= 4 && inside) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int e = e0 + lane + r * PTA_WAVE;
+                if (e0 + r * PTA_WAVE >= len) continue;
+#pragma unroll
+                for (int i = 0; i < PREP_TOKENS + KMAX - 1; ++i)
+                    x[r][i] = Io<T>::ld(src + (long)max(m0 - (KMAX - 1) + i, 0) * ld + min(e, len - 1));
+            }
+#pragma unroll
+            for (int t = 0; t < PREP_TOKENS; ++t) {
+                float y[4], ss = 0.f;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    y[r] = 0.f;
+                    if (e0 + lane + r * PTA_WAVE >= len) continue;
+                    float acc = 0.f;
+#pragma unroll
+                    for (int kk = 0; kk < KMAX; ++kk) acc += w[r][kk] * x[r][t + kk];
+                    y[r] = acc / (1.0f + expf(-acc));
+                    ss += y[r] * y[r];
+                }
+                const float by = is_v ? 1.0f : (is_q ? q_scale : 1.0f) / sqrtf(wave_sum(ss) + norm_eps);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int e = e0 + lane + r * PTA_WAVE;
+                    if (e < len) qkv[(long)(m0 + t) * C + c0 + e] = y[r] * by;
+                }
+            }
+            continue;
+        }
+        for (int m = m0; m < m1; ++m) {
+            const int s = token_seq[m], first = cu_tokens[s], j = m - first;
+            float* tl = tail + (K > 1 ? (long)seq_slot[s] * tail_ld : 0L);
+            float y[4], ss = 0.f;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int e = e0 + lane + r * PTA_WAVE, c = c0 + e;
+                y[r] = 0.f;
+                if (e >= len) continue;
+                float acc = 0.f;
+#pragma unroll
+                for (int kk = 0; kk < KMAX; ++kk) {
+                    if (kk < KMAX - K) continue;
+                    const int jj = j - (KMAX - 1 - kk);
+                    const float x = jj >= 0 ? Io<T>::ld(src + (long)(first + jj) * ld + e) : tl[(long)(K - 1 + jj) * C + c];
+                    acc += w[r][kk] * x;
+                    if (move_tail && kk > KMAX - K) tl[(long)(kk - 1 - (KMAX - K)) * C + c] = x;  // (the one token: x is the tail's next, or its own)
+                }
+                y[r] = acc / (1.0f + expf(-acc));
+                ss += y[r] * y[r];
+            }
+            const float by = is_v ? 1.0f : (is_q ? q_scale : 1.0f) / sqrtf(wave_sum(ss) + norm_eps);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int e = e0 + lane + r * PTA_WAVE;
+                if (e < len) qkv[(long)m * C + c0 + e] = y[r] * by;
+            }
+        }
     }
 }
 
@@ -123,16 +173,20 @@ extern "C" int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, 
     PTA_REQUIRE(!several || ((const char*)k - (const char*)q == kv_heads * N * size && (const char*)v - (const char*)k == kv_heads * N * size && ld >= C),
                 "delta_prep: q, k and v must lie side by side");
     hipStream_t s = (hipStream_t)stream;
-    const dim3 grid(M, 2 * kv_heads + 2 * heads);
+    const dim3 grid((M + PREP_TOKENS - 1) / PREP_TOKENS, (2 * kv_heads + 2 * heads + 3) / 4);
     const int move = several ? 0 : 1;
-    if (dtype == PTA_F32)
-        hipLaunchKernelGGL(delta_prep_kernel<float>, grid, dim3(64), 0, s, qkv, g, beta, (const float*)q, (const float*)k,
-                           (const float*)v, ld, conv, (const float*)a, a_ld, (const float*)b, b_ld, A_log, dt_bias, tail, tail_ld,
-                           cu_tokens, token_seq, seq_slot, move, heads, kv_heads, N, P, taps, q_scale, norm_eps);
-    else
-        hipLaunchKernelGGL(delta_prep_kernel<bf16_t>, grid, dim3(64), 0, s, qkv, g, beta, (const bf16_t*)q, (const bf16_t*)k,
-                           (const bf16_t*)v, ld, conv, (const bf16_t*)a, a_ld, (const bf16_t*)b, b_ld, A_log, dt_bias, tail, tail_ld,
-                           cu_tokens, token_seq, seq_slot, move, heads, kv_heads, N, P, taps, q_scale, norm_eps);
+#define DELTA_PREP(T_, KMAX_)                                                                                                    \
+    hipLaunchKernelGGL((delta_prep_kernel<T_, KMAX_>), grid, dim3(256), 0, s, qkv, g, beta, (const T_*)q, (const T_*)k, (const T_*)v, \
+                       ld, conv, (const T_*)a, a_ld, (const T_*)b, b_ld, A_log, dt_bias, tail, tail_ld, cu_tokens, token_seq,         \
+                       seq_slot, move, M, heads, kv_heads, N, P, taps, q_scale, norm_eps)
+    if (dtype == PTA_F32) {
+        if (taps <= 4) DELTA_PREP(float, 4);
+        else DELTA_PREP(float, DELTA_MAX_TAPS);
+    } else {
+        if (taps <= 4) DELTA_PREP(bf16_t, 4);
+        else DELTA_PREP(bf16_t, DELTA_MAX_TAPS);
+    }
+#undef DELTA_PREP
     if (several && taps > 1) {
         if (pta_check_launch("delta_prep")) return 1;
         return pta_conv_tail(q, ld, tail, tail_ld, cu_tokens, seq_slot, n_seqs, (int)C, taps, dtype, stream);
@@ -222,9 +276,9 @@ typedef float delta_f4 __attribute__((ext_vector_type(4)));
 
 template <int V>
 __device__ __forceinline__ void delta_load(const float* p, float (&v)[V]) {
-    if constexpr (V == 4) {
-        const float4 q = *reinterpret_cast<const float4*>(p);
-        v[0] = q.x; v[1] = q.y; v[2] = q.z; v[3] = q.w;
+    if constexpr (V == 2) {
+        const float2 q = *reinterpret_cast<const float2*>(p);
+        v[0] = q.x; v[1] = q.y;
     } else {
 #pragma unroll
         for (int i = 0; i < V; ++i) v[i] = p[i];
@@ -244,7 +298,8 @@ __global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ ha
     float* g_s = lds;                    // [16][ROW]
     float* k_s = g_s + 16 * ROW;         // [16][ROW]
     float* q_s = k_s + 16 * ROW;         // [16][ROW]
-    float* red = q_s + 16 * ROW;         // [4 waves][2][16 t][16 s]
+    float* kd_s = q_s + 16 * ROW;        // [16][ROW]; later the waves' sums [4][2][16 t][16 s]
+    float* red = kd_s;
     __shared__ float L_s[16][17];
     __shared__ float b_s[16];
     const int h = blockIdx.y, kh = h / (heads / G), s = blockIdx.z;
@@ -253,13 +308,25 @@ __global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ ha
     const int cnt = min(DELTA_BLOCK, t1 - m0);
     const int C = 2 * G * N + heads * P;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-    for (int i = tid; i < 16 * NP; i += 256) {
-        const int t = i / NP, n = i - t * NP;
-        const bool in = t < cnt && n < N;
-        const float* row = qkv + (long)(m0 + t) * C + kh * N + n;
-        g_s[t * ROW + n] = in ? g[((long)(m0 + t) * heads + h) * N + n] : 1.f;  // (a token past the end changes nothing)
-        k_s[t * ROW + n] = in ? row[(long)G * N] : 0.f;
-        q_s[t * ROW + n] = in ? row[0] : 0.f;
+    {
+        float gr[RT], kr[RT], qr[RT];  // all loads in flight at once; what lies past an end is read from inside and put down as nothing
+#pragma unroll
+        for (int j = 0; j < RT; ++j) {
+            const int t = (tid + j * 256) / NP, n = (tid + j * 256) % NP;
+            const long m = m0 + min(t, cnt - 1);
+            const float* row = qkv + m * C + kh * N + min(n, N - 1);
+            gr[j] = g[(m * heads + h) * N + min(n, N - 1)];
+            kr[j] = row[(long)G * N];
+            qr[j] = row[0];
+        }
+#pragma unroll
+        for (int j = 0; j < RT; ++j) {
+            const int t = (tid + j * 256) / NP, n = (tid + j * 256) % NP;
+            const bool in = t < cnt && n < N;
+            g_s[t * ROW + n] = in ? gr[j] : 1.f;  // (a token past the end changes nothing)
+            k_s[t * ROW + n] = in ? kr[j] : 0.f;
+            q_s[t * ROW + n] = in ? qr[j] : 0.f;
+        }
     }
     if (tid < 16) b_s[tid] = tid < cnt ? beta[(long)(m0 + tid) * heads + h] : 0.f;
     __syncthreads();
@@ -267,7 +334,7 @@ __global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ ha
     float lk[16], aq[16];
 #pragma unroll
     for (int t = 0; t < 16; ++t) lk[t] = 0.f, aq[t] = 0.f;
-    constexpr int VN = RT < 4 ? RT : 4;  // channels at a time
+    constexpr int VN = RT < 2 ? RT : 2;  // channels at a time (the compiler asks for all sixteen tokens' rows at once)
 #pragma unroll 1
     for (int c0 = 0; c0 < RT; c0 += VN) {
         const float* gp = g_s + ch + c0;
@@ -288,15 +355,16 @@ __global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ ha
                 lk[t] += kt[i] * r[i];
                 aq[t] += qt[i] * r[i];
             }
-            if ((t & 3) == 3) asm volatile("" ::: "memory");  // (not all sixteen tokens' loads at once)
         }
-        if (st < cnt) {
-            float* to = hat + (((long)(m0 + st) * heads + h) * 3 + 2) * N + ch + c0;
 #pragma unroll
-            for (int i = 0; i < VN; ++i)
-                if (ch + c0 + i < N) to[i] = r[i];
-        }
+        for (int i = 0; i < VN; ++i) kd_s[st * ROW + ch + c0 + i] = r[i];
     }
+    __syncthreads();
+    for (int i = tid; i < cnt * N; i += 256) {
+        const int t = i / N, n = i - t * N;
+        hat[(((long)(m0 + t) * heads + h) * 3 + 2) * N + n] = kd_s[t * ROW + n];
+    }
+    __syncthreads();
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
         lk[t] += __shfl_xor(lk[t], 16, 64);
@@ -344,7 +412,8 @@ __global__ __launch_bounds__(256) void delta_block_kernel(float* __restrict__ ha
     }
 }
 
-template <int RT, int MODE>
+// VEC: N is a multiple of four.  hat and ta are readable for a block past their last token (hat for 256 elements more).
+template <int RT, int MODE, bool VEC>
 __global__ __launch_bounds__(256) void delta_scan_kernel(
     float* __restrict__ y, const float* __restrict__ qkv, const float* __restrict__ hat, const float* __restrict__ ta,
     const float* __restrict__ g, float* __restrict__ state, long state_ld, float* __restrict__ chunk_state,
@@ -372,7 +441,6 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     float* sb = MODE == DELTA_WHOLE ? state + (long)seq_slot[s] * state_ld + (long)h * N * P
                                     : chunk_state + ((long)blockIdx.z * heads + h) * N * W;
     const int C = 2 * G * N + heads * P;
-    const bool vec = (N & 3) == 0;
     delta_f4 S[RT];
 #pragma unroll
     for (int r = 0; r < RT; ++r)
@@ -382,54 +450,58 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
             if (MODE == DELTA_LOCAL) S[r][e] = (p >= P && n == p - P) ? 1.f : 0.f;
             else S[r][e] = (n < N && p < P) ? sb[(long)n * W + p] : 0.f;
         }
-    // what a block needs, asked for one block ahead
+    // What a block needs is asked for one block ahead.  The loads branch on nothing: rows past the sequence's end are read
+    // (they lie within the buffers) and elements past a row's end are read from inside the row, and both are put down as zeros.
     float4 ph[PER];
     float pt[2], pb, pv[4];
+    int off[PER];
+    bool keep[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int i = min(tid + j * 256, PIECES - 1);
+        const int t = i / (3 * NP / 4), rest = i - t * (3 * NP / 4), which = rest / (NP / 4), n = (rest - which * (NP / 4)) * 4;
+        keep[j] = n < N;
+        off[j] = (t * heads * 3 + which) * N + (VEC ? min(n, N - 4) : n);
+    }
     auto fetch = [&](int m0) {
-        const int cnt = t1 - m0;  // (tokens from sixteen on belong to the next block; none at or below zero)
+        const long first = (long)m0 * heads + h;
+        const float* hb = hat + first * 3 * N;
+        const float* tb = ta + first * 32;
 #pragma unroll
         for (int j = 0; j < PER; ++j) {
-            const int i = tid + j * 256;
-            const int t = i / (3 * NP / 4), rest = i - t * (3 * NP / 4), which = rest / (NP / 4), n = (rest - which * (NP / 4)) * 4;
-            ph[j] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (i >= PIECES || t >= cnt || (MODE == DELTA_LOCAL && which == 1)) continue;
-            const float* from = hat + (((long)(m0 + t) * heads + h) * 3 + which) * N + n;
-            if (vec) {
-                if (n < N) ph[j] = *reinterpret_cast<const float4*>(from);
-            } else {
-                if (n < N) ph[j].x = from[0];
-                if (n + 1 < N) ph[j].y = from[1];
-                if (n + 2 < N) ph[j].z = from[2];
-                if (n + 3 < N) ph[j].w = from[3];
+            if constexpr (VEC) ph[j] = *reinterpret_cast<const float4*>(hb + off[j]);
+            else {  // (off[j] + 3 may lie in the next vector of the token, or in the next token's first)
+                ph[j] = make_float4(hb[off[j]], hb[off[j] + 1], hb[off[j] + 2], hb[off[j] + 3]);
             }
         }
 #pragma unroll
-        for (int j = 0; j < 2; ++j) {
-            const int i = tid + j * 256, t = i >> 5;
-            pt[j] = t < cnt ? ta[((long)(m0 + t) * heads + h) * 32 + (i & 31)] : 0.f;
-        }
-        pb = (tid < N && cnt > 0) ? g[((long)m0 * heads + h) * N + tid] : 0.f;
+        for (int j = 0; j < 2; ++j) pt[j] = tb[((tid >> 5) + 8 * j) * heads * 32 + (tid & 31)];
+        pb = g[first * N + min(tid, N - 1)];
+        const float* vb = qkv + (long)m0 * C + 2 * G * N + h * P + min(p, P - 1);
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-            pv[e] = (lk * 4 + e < cnt && p < P) ? qkv[(long)(m0 + lk * 4 + e) * C + 2 * G * N + h * P + p] : 0.f;
+        for (int e = 0; e < 4; ++e) pv[e] = vb[(long)min(lk * 4 + e, t1 - 1 - m0) * C];
     };
     fetch(t0);
     for (int m0 = t0; m0 < t1; m0 += DELTA_BLOCK) {
+        const int cnt = t1 - m0;  // (from sixteen on: a whole block)
         __syncthreads();
 #pragma unroll
         for (int j = 0; j < PER; ++j) {
             const int i = tid + j * 256;
             const int t = i / (3 * NP / 4), rest = i - t * (3 * NP / 4), which = rest / (NP / 4), n = (rest - which * (NP / 4)) * 4;
-            if (i < PIECES) *reinterpret_cast<float4*>(hat_s + (which * 16 + t) * ROW + n) = ph[j];
+            const bool in = keep[j] && t < cnt;
+            const float4 f = make_float4(in ? ph[j].x : 0.f, in && (VEC || n + 1 < N) ? ph[j].y : 0.f,
+                                         in && (VEC || n + 2 < N) ? ph[j].z : 0.f, in && (VEC || n + 3 < N) ? ph[j].w : 0.f);
+            if (PIECES % 256 == 0 || i < PIECES) *reinterpret_cast<float4*>(hat_s + (which * 16 + t) * ROW + n) = f;
         }
 #pragma unroll
-        for (int j = 0; j < 2; ++j) ta_s[((tid + j * 256) >> 5) * TROW + ((tid + j * 256) & 31)] = pt[j];
-        if (tid < NP) b_s[tid] = pb;
+        for (int j = 0; j < 2; ++j) ta_s[((tid >> 5) + 8 * j) * TROW + (tid & 31)] = (tid >> 5) + 8 * j < cnt ? pt[j] : 0.f;
+        if (tid < NP) b_s[tid] = tid < N ? pb : 0.f;
         delta_f4 R0, R1 = {0.f, 0.f, 0.f, 0.f}, O0 = {0.f, 0.f, 0.f, 0.f}, O1 = {0.f, 0.f, 0.f, 0.f}, U = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int e = 0; e < 4; ++e) R0[e] = pv[e];
+        for (int e = 0; e < 4; ++e) R0[e] = lk * 4 + e < cnt && p < P ? pv[e] : 0.f;
         __syncthreads();
-        fetch(m0 + DELTA_BLOCK);
+        if (cnt > DELTA_BLOCK) fetch(m0 + DELTA_BLOCK);
         const float* kh_row = hat_s + lr * ROW + lk * 4;
         const float* qh_row = kh_row + 16 * ROW;
 #pragma unroll
@@ -513,25 +585,17 @@ __global__ __launch_bounds__(512) void delta_carry_kernel(float* __restrict__ st
 #pragma unroll
         for (int j = 0; j < RTW; ++j) {
             const int r0 = (wave + 8 * j) * 16;
-            const float* row = cs + (long)(r0 + lr) * W + P;
+            const float* row = cs + (long)min(r0 + lr, N - 1) * W + P;
 #pragma unroll
             for (int m = 0; m < RT; ++m) {
                 const int k = m * 16 + lk * 4;
-                a[j][m] = make_float4(0.f, 0.f, 0.f, 0.f);
-                if (r0 + lr >= N) continue;
-                if (VEC) {
-                    if (k < N) a[j][m] = *reinterpret_cast<const float4*>(row + k);
-                } else {
-                    if (k < N) a[j][m].x = row[k];
-                    if (k + 1 < N) a[j][m].y = row[k + 1];
-                    if (k + 2 < N) a[j][m].z = row[k + 2];
-                    if (k + 3 < N) a[j][m].w = row[k + 3];
-                }
+                if (VEC) a[j][m] = *reinterpret_cast<const float4*>(row + min(k, N - 4));
+                else a[j][m] = make_float4(row[min(k, N - 1)], row[min(k + 1, N - 1)], row[min(k + 2, N - 1)], row[min(k + 3, N - 1)]);
             }
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int n = r0 + lk * 4 + e;
-                B[j][e] = (in && n < N) ? cs[(long)n * W + p0 + lr] : 0.f;
+                B[j][e] = cs[(long)min(n, N - 1) * W + min(p0 + lr, P - 1)];
             }
         }
     };
@@ -557,6 +621,7 @@ __global__ __launch_bounds__(512) void delta_carry_kernel(float* __restrict__ st
         delta_f4 acc[RTW][2];
 #pragma unroll
         for (int j = 0; j < RTW; ++j) acc[j][0] = B[j], acc[j][1] = delta_f4{0.f, 0.f, 0.f, 0.f};
+        // (what stands in LDS beyond row N - 1 is zero, so A_c's elements beyond column N - 1 count for nothing, whatever they are)
 #pragma unroll
         for (int m = 0; m < RT; ++m) {
             float b[4];
@@ -572,7 +637,10 @@ __global__ __launch_bounds__(512) void delta_carry_kernel(float* __restrict__ st
         }
         if (c + 1 < n_chunks) fetch(c + 1);
 #pragma unroll
-        for (int j = 0; j < RTW; ++j) S[j] = acc[j][0] + acc[j][1];
+        for (int j = 0; j < RTW; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                S[j][e] = (wave + 8 * j) * 16 + lk * 4 + e < N ? acc[j][0][e] + acc[j][1][e] : 0.f;
         __syncthreads();  // everyone has read the state that the next turn replaces
     }
 #pragma unroll
@@ -603,15 +671,17 @@ static int launch_delta_steps(const DeltaLaunch& d) {
 
 template <int RT>
 static int launch_delta_blocks(const DeltaLaunch& d) {
-    constexpr size_t block_lds = (size_t)(3 * 16 * (16 * RT + 4) + 4 * 2 * 256) * sizeof(float);
+    constexpr size_t block_lds = (size_t)(3 * 16 * (16 * RT + 4) + std::max(16 * (16 * RT + 4), 4 * 2 * 256)) * sizeof(float);
     constexpr size_t scan_lds = (size_t)(3 * 16 * (16 * RT + 4) + 16 * 36 + 16 * RT) * sizeof(float);
-    static_assert(block_lds <= 62 * 1024 && scan_lds <= 64 * 1024, "a block's rows fit the LDS a launch may ask for without saying so");
+    static_assert(block_lds <= 80 * 1024 && scan_lds <= 64 * 1024, "a block's rows fit the LDS");
+    if (block_lds > 62 * 1024)  // more than a launch may ask for unless the kernel has been told
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(delta_block_kernel<RT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)block_lds);
     hipLaunchKernelGGL(delta_block_kernel<RT>, dim3((d.max_new + DELTA_BLOCK - 1) / DELTA_BLOCK, d.heads, d.n_seqs), dim3(256), block_lds,
                        d.s, d.hat, d.ta, d.g, d.qkv, d.beta, d.cu_tokens, d.heads, d.G, d.P, d.N);
 #define DELTA_SCAN(MODE_, COLS_, RUNS_)                                                                                          \
-    hipLaunchKernelGGL((delta_scan_kernel<RT, MODE_>), dim3(((COLS_) + 63) / 64, d.heads, (RUNS_)), dim3(256), scan_lds, d.s, d.y,   \
-                       d.qkv, d.hat, d.ta, d.g, d.state, d.state_ld, d.chunk_state, d.cu_tokens, d.seq_slot, d.heads, d.G, d.P, d.N, \
-                       d.chunk, d.max_chunks)
+    hipLaunchKernelGGL((d.N % 4 ? delta_scan_kernel<RT, MODE_, false> : delta_scan_kernel<RT, MODE_, true>),                       \
+                       dim3(((COLS_) + 63) / 64, d.heads, (RUNS_)), dim3(256), scan_lds, d.s, d.y, d.qkv, d.hat, d.ta, d.g, d.state, \
+                        d.state_ld, d.chunk_state, d.cu_tokens, d.seq_slot, d.heads, d.G, d.P, d.N, d.chunk, d.max_chunks)
     if (d.max_chunks <= 1) {
         DELTA_SCAN(DELTA_WHOLE, d.P, d.n_seqs);
         return pta_check_launch("delta_scan");
@@ -629,8 +699,8 @@ static int launch_delta_blocks(const DeltaLaunch& d) {
 }
 
 // y [M, heads * P], qkv [M, 2 * kv_heads * N + heads * P], g [M, heads * N], beta [M, heads], all 32-bit and dense; state
-// [slots, >= heads * N * P] rows state_ld apart.  hat [M, heads, 3, N] and ta [M, heads, 2, 16] given (scratch): blocks of sixteen
-// tokens; g is then written over.  Without them the tokens are walked one by one.  chunk_state [n_seqs * max_chunks, heads, N,
+// [slots, >= heads * N * P] rows state_ld apart.  hat [M + 16, heads, 3, N] with 256 elements behind it and ta [M + 16, heads, 2, 16] given
+// (scratch): blocks of sixteen tokens; g is then written over.  Without them the tokens are walked one by one.  chunk_state [n_seqs * max_chunks, heads, N,
 // P + N] is scratch for steps whose longest sequence is cut into max_chunks > 1 chunks of `chunk` tokens (a multiple of 16).
 extern "C" int pta_delta_scan(float* y, const float* qkv, float* g, const float* beta, float* state, long state_ld, float* hat,
                               float* ta, float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new,

@@ -244,6 +244,65 @@ __global__ void conv_add_kernel(T* __restrict__ out, const float* __restrict__ i
     }
 }
 
+// The same for up to four taps and channels four at a time: a thread walks CONV_ADD_RUN tokens with the inputs before the
+// current one in registers, so that a row is read once (and the first K - 1 of the run twice).
+#define CONV_ADD_RUN 8
+
+__device__ __forceinline__ void store4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+__device__ __forceinline__ void store4(bf16_t* p, float4 v) {
+    bf16_t r[4] = {f32_to_bf16_bits(v.x), f32_to_bf16_bits(v.y), f32_to_bf16_bits(v.z), f32_to_bf16_bits(v.w)};
+    *reinterpret_cast<uint2*>(p) = make_uint2((uint32_t)r[0] | ((uint32_t)r[1] << 16), (uint32_t)r[2] | ((uint32_t)r[3] << 16));
+}
+
+template <typename T, int K>
+__global__ void conv_add4_kernel(T* __restrict__ out, const float* __restrict__ in, const float* __restrict__ w,
+                                 const float* __restrict__ tail, long tail_ld, const int* __restrict__ cu_tokens,
+                                 const int* __restrict__ token_seq, const int* __restrict__ seq_slot, int M, int C) {
+    const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+    if (c >= C) return;
+    const int m0 = blockIdx.x * CONV_ADD_RUN, m1 = min(M, m0 + CONV_ADD_RUN);
+    auto ld4 = [](const float* p) { return *reinterpret_cast<const float4*>(p); };
+    float4 wk[K], x[K];  // x[k]: the input of K - 1 - k tokens ago
+#pragma unroll
+    for (int k = 0; k < K; ++k) wk[k] = ld4(w + (long)k * C + c);
+    int s = -1, first = 0;
+    for (int m = m0; m < m1; ++m) {
+        if (token_seq[m] != s) {  // a new sequence, or the run's start
+            s = token_seq[m], first = cu_tokens[s];
+            const float* tl = tail + (K > 1 ? (long)seq_slot[s] * tail_ld : 0L);
+#pragma unroll
+            for (int k = 0; k + 1 < K; ++k) {
+                const int jj = m - first - (K - 1 - k);
+                x[k] = jj >= 0 ? ld4(in + (long)(first + jj) * C + c) : ld4(tl + (long)(K - 1 + jj) * C + c);
+            }
+        } else {
+#pragma unroll
+            for (int k = 0; k + 1 < K; ++k) x[k] = x[k + 1];
+        }
+        x[K - 1] = ld4(in + (long)m * C + c);
+        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int k = 0; k < K; ++k) {
+            acc.x += wk[k].x * x[k].x; acc.y += wk[k].y * x[k].y; acc.z += wk[k].z * x[k].z; acc.w += wk[k].w * x[k].w;
+        }
+        const float4 now = x[K - 1];
+        store4(out + (long)m * C + c, make_float4(now.x + acc.x, now.y + acc.y, now.z + acc.z, now.w + acc.w));
+    }
+}
+
+template <typename T>
+static void launch_conv_add4(T* out, const float* in, const float* w, const float* tail, long tail_ld, const int* cu_tokens,
+                             const int* token_seq, const int* seq_slot, int M, int C, int K, hipStream_t s) {
+    const dim3 block(C >= 1024 ? 256 : 64), grid((M + CONV_ADD_RUN - 1) / CONV_ADD_RUN, (C / 4 + block.x - 1) / block.x);
+#define CONV_ADD4(K_) hipLaunchKernelGGL((conv_add4_kernel<T, K_>), grid, block, 0, s, out, in, w, tail, tail_ld, cu_tokens, token_seq, \
+                                         seq_slot, M, C)
+    if (K == 1) CONV_ADD4(1);
+    else if (K == 2) CONV_ADD4(2);
+    else if (K == 3) CONV_ADD4(3);
+    else CONV_ADD4(4);
+#undef CONV_ADD4
+}
+
 extern "C" int pta_conv_add(void* out, const float* in, const float* w, float* tail, long tail_ld, const int* cu_tokens,
                             const int* token_seq, const int* seq_slot, int n_seqs, int M, int C, int K, int dtype, void* stream) {
     PTA_REQUIRE(M > 0 && n_seqs > 0 && C > 0, "conv_add: tokens=%d sequences=%d channels=%d must be positive", M, n_seqs, C);
@@ -254,7 +313,11 @@ extern "C" int pta_conv_add(void* out, const float* in, const float* w, float* t
     PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "conv_add: unknown dtype %d", dtype);
     hipStream_t s = (hipStream_t)stream;
     const dim3 block(C >= 256 ? 256 : 64), grid((M + CONV_ADD_TOKENS - 1) / CONV_ADD_TOKENS, (C + block.x - 1) / block.x);
-    if (dtype == PTA_F32)
+    if (K <= 4 && C % 4 == 0 && tail_ld % 4 == 0 && ((uintptr_t)in % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)w % 16) == 0 &&
+        ((uintptr_t)tail % 16) == 0) {
+        if (dtype == PTA_F32) launch_conv_add4<float>((float*)out, in, w, tail, tail_ld, cu_tokens, token_seq, seq_slot, M, C, K, s);
+        else launch_conv_add4<bf16_t>((bf16_t*)out, in, w, tail, tail_ld, cu_tokens, token_seq, seq_slot, M, C, K, s);
+    } else if (dtype == PTA_F32)
         hipLaunchKernelGGL(conv_add_kernel<float>, grid, block, 0, s, (float*)out, in, w, tail, tail_ld, cu_tokens, token_seq,
                            seq_slot, M, C, K);
     else

@@ -1955,8 +1955,9 @@ def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: to
     chunk, chunks = DELTA_CHUNK_TOKENS, 1
     hat = ta = chunk_state = None
     if longest >= DELTA_BLOCKS_FROM:
-        hat = torch.empty((M, heads, 3, key_dim), dtype=torch.float32, device=qkv.device)
-        ta = torch.empty((M, heads, 2, 16), dtype=torch.float32, device=qkv.device)
+        # (room behind the last token: its block's loads are of sixteen whole tokens, in vectors that may start inside the last)
+        hat = torch.empty((M + 16) * heads * 3 * key_dim + 256, dtype=torch.float32, device=qkv.device)
+        ta = torch.empty((M + 16, heads, 2, 16), dtype=torch.float32, device=qkv.device)
         if longest > 2 * chunk and n * heads * ((value_dim + 15) // 16) < DELTA_CHUNK_WAVES:
             chunks = (longest + chunk - 1) // chunk
     if chunks > 1:
