@@ -12,7 +12,7 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import Any, ClassVar, Dict
+from typing import Any, Callable, ClassVar, Dict
 
 CONFIG_NAME = "config.json"  # src/transformers/utils/__init__.py:254
 
@@ -49,9 +49,10 @@ class ModelConfig:
     def validate(self) -> None:
         """Raise ConfigError for values no model can be built from."""
 
-    def sizes_from_weights(self, shapes: Dict[str, Any]) -> None:
-        """Take sizes that ``config.json`` leaves to the weight file: ``shapes`` is tensor name -> shape of what the files
-        hold.  Called by whoever builds a model from a folder, before the model is put together."""
+    def sizes_from_weights(self, shapes: Callable[[], Dict[str, Any]]) -> None:
+        """Take sizes that ``config.json`` leaves to the weight file: ``shapes()`` is tensor name -> shape of what the files
+        hold (their headers are read then, so a configuration that says everything does not ask).  Called by whoever builds
+        a model from a folder, before the model is put together."""
 
     # dict / json -------------------------------------------------------
     @classmethod

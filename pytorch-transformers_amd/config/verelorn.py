@@ -79,12 +79,15 @@ class VerelornConfig(ModelConfig):
         return int(m.get(key) or m["vdim"])
 
     def sizes_from_weights(self, shapes) -> None:
+        if not any(l["type"] == "channel_delta" and l["mixer"].get(k) is None for l in self.layers for k in INNER_RANKS):
+            return
+        held = shapes()
         layers = [dict(l, mixer=dict(l["mixer"])) for l in self.layers]  # (entries of the list may be one object)
         for i, layer in enumerate(layers):
             if layer["type"] != "channel_delta":
                 continue
             for key, tensor in INNER_RANKS.items():
-                shape = shapes.get(f"l{i}.mix.{tensor}")
+                shape = held.get(f"l{i}.mix.{tensor}")
                 if layer["mixer"].get(key) is None and shape is not None and len(shape) == 2:
                     layer["mixer"][key] = int(shape[0])
         self.layers = layers

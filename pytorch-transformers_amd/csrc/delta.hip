@@ -44,11 +44,11 @@ enum { DELTA_WHOLE = 0, DELTA_LOCAL = 1, DELTA_OUTPUT = 2 };
 
 __device__ __forceinline__ float softplus_32(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
-// One wave per (PREP_TOKENS tokens, unit): units are the q heads, the k heads, the value heads and the heads' decays (with
+// One wave per (TOK tokens, unit): units are the q heads, the k heads, the value heads and the heads' decays (with
 // beta); a unit's convolution weights stay in registers over its tokens.
 #define PREP_TOKENS 4
 
-template <typename T, int KMAX>
+template <typename T, int KMAX, int TOK>
 __global__ __launch_bounds__(256) void delta_prep_kernel(
     float* __restrict__ qkv, float* __restrict__ g, float* __restrict__ beta, const T* __restrict__ q, const T* __restrict__ k,
     const T* __restrict__ v, long ld, const float* __restrict__ conv, const T* __restrict__ a, long a_ld,
@@ -56,7 +56,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
     float* __restrict__ tail, long tail_ld, const int* __restrict__ cu_tokens, const int* __restrict__ token_seq,
     const int* __restrict__ seq_slot, int move_tail, int M, int heads, int G, int N, int P, int K, float q_scale, float norm_eps) {
     const int unit = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    const int m0 = blockIdx.x * PREP_TOKENS, m1 = min(M, m0 + PREP_TOKENS);
+    const int m0 = blockIdx.x * TOK, m1 = min(M, m0 + TOK);
     if (unit >= 2 * G + 2 * heads) return;
     if (unit >= 2 * G + heads) {  // a head's decays and step size
         const int h = unit - 2 * G - heads;
@@ -76,7 +76,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
     const int c0 = is_v ? 2 * G * N + local * P : unit * N;  // first channel of the head in q | k | v
     const int C = 2 * G * N + heads * P;
     // whether every input of these tokens is a row of this step: they are then asked for all at once
-    const bool inside = m1 - m0 == PREP_TOKENS && token_seq[m0] == token_seq[m1 - 1] && m0 - cu_tokens[token_seq[m0]] >= K - 1;
+    const bool inside = TOK > 1 && m1 - m0 == TOK && token_seq[m0] == token_seq[m1 - 1] && m0 - cu_tokens[token_seq[m0]] >= K - 1;
     for (int e0 = 0; e0 < len; e0 += 4 * PTA_WAVE) {  // (heads of q and k fit one round)
         float w[4][KMAX];
 #pragma unroll
@@ -86,18 +86,18 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
             for (int kk = 0; kk < KMAX; ++kk)  // (fewer taps: zeros in front)
                 w[r][kk] = (e < len && kk >= KMAX - K) ? conv[(long)(kk - (KMAX - K)) * C + c0 + e] : 0.f;
         }
-        float x[4][PREP_TOKENS + KMAX - 1];  // row m0 - (KMAX - 1) + i
-        if (KMAX <= 4 && inside) {
+        float x[4][TOK + KMAX - 1];  // row m0 - (KMAX - 1) + i
+        if (TOK > 1 && KMAX <= 4 && inside) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int e = e0 + lane + r * PTA_WAVE;
                 if (e0 + r * PTA_WAVE >= len) continue;
 #pragma unroll
-                for (int i = 0; i < PREP_TOKENS + KMAX - 1; ++i)
+                for (int i = 0; i < TOK + KMAX - 1; ++i)
                     x[r][i] = Io<T>::ld(src + (long)max(m0 - (KMAX - 1) + i, 0) * ld + min(e, len - 1));
             }
 #pragma unroll
-            for (int t = 0; t < PREP_TOKENS; ++t) {
+            for (int t = 0; t < TOK; ++t) {
                 float y[4], ss = 0.f;
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
@@ -173,12 +173,18 @@ extern "C" int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, 
     PTA_REQUIRE(!several || ((const char*)k - (const char*)q == kv_heads * N * size && (const char*)v - (const char*)k == kv_heads * N * size && ld >= C),
                 "delta_prep: q, k and v must lie side by side");
     hipStream_t s = (hipStream_t)stream;
-    const dim3 grid((M + PREP_TOKENS - 1) / PREP_TOKENS, (2 * kv_heads + 2 * heads + 3) / 4);
+    const int each = several ? PREP_TOKENS : 1;  // (steps of one token per sequence are short of waves, not of registers)
+    const dim3 grid((M + each - 1) / each, (2 * kv_heads + 2 * heads + 3) / 4);
     const int move = several ? 0 : 1;
-#define DELTA_PREP(T_, KMAX_)                                                                                                    \
-    hipLaunchKernelGGL((delta_prep_kernel<T_, KMAX_>), grid, dim3(256), 0, s, qkv, g, beta, (const T_*)q, (const T_*)k, (const T_*)v, \
+#define DELTA_PREP_EACH(T_, KMAX_, TOK_)                                                                                                    \
+    hipLaunchKernelGGL((delta_prep_kernel<T_, KMAX_, TOK_>), grid, dim3(256), 0, s, qkv, g, beta, (const T_*)q, (const T_*)k, (const T_*)v, \
                        ld, conv, (const T_*)a, a_ld, (const T_*)b, b_ld, A_log, dt_bias, tail, tail_ld, cu_tokens, token_seq,         \
                        seq_slot, move, M, heads, kv_heads, N, P, taps, q_scale, norm_eps)
+#define DELTA_PREP(T_, KMAX_)                                   \
+    do {                                                        \
+        if (several) DELTA_PREP_EACH(T_, KMAX_, PREP_TOKENS);   \
+        else DELTA_PREP_EACH(T_, KMAX_, 1);                     \
+    } while (0)
     if (dtype == PTA_F32) {
         if (taps <= 4) DELTA_PREP(float, 4);
         else DELTA_PREP(float, DELTA_MAX_TAPS);
@@ -187,6 +193,7 @@ extern "C" int pta_delta_prep(float* qkv, float* g, float* beta, const void* q, 
         else DELTA_PREP(bf16_t, DELTA_MAX_TAPS);
     }
 #undef DELTA_PREP
+#undef DELTA_PREP_EACH
     if (several && taps > 1) {
         if (pta_check_launch("delta_prep")) return 1;
         return pta_conv_tail(q, ld, tail, tail_ld, cu_tokens, seq_slot, n_seqs, (int)C, taps, dtype, stream);

@@ -265,7 +265,7 @@ class CausalLM:
 
         device = _require_gpu(device)
         config = AutoConfig.from_pretrained(folder)
-        config.sizes_from_weights(tensor_shapes(folder))
+        config.sizes_from_weights(lambda: tensor_shapes(folder))
         dtype = auto_dtype(config, folder) if dtype == "auto" else resolve_dtype(dtype)
         _, builder = lookup(config.model_type)
         spec = builder(config)

@@ -1894,9 +1894,15 @@ def conv_add(x: torch.Tensor, w: torch.Tensor, tail: Optional[torch.Tensor], ctx
 
 
 # ---- the gated delta rule with a decay per key channel --------------------------------------------------------------
-DELTA_BLOCKS_FROM = 24  # a step in which some sequence brings so many tokens runs blocks of sixteen as matrix products
-DELTA_CHUNK_TOKENS = 256  # a sequence that brings more than twice as many is cut into chunks that run side by side ...
-DELTA_CHUNK_WAVES = 512  # ... where the launch would otherwise have fewer waves (sixteen columns of a head's state each)
+DELTA_BLOCKS_FROM = 20  # a step in which some sequence brings so many tokens runs blocks of sixteen as matrix products
+DELTA_CHUNK_WAVES = 512  # a launch of fewer waves (sixteen columns of a head's state each) cuts long sequences into chunks
+
+
+def delta_chunk(longest: int) -> int:
+    """Tokens of a chunk for a prompt of ``longest`` tokens: more chunks fill the chip, fewer make a shorter carry (16 heads
+    of 128 x 128: 600 tokens 95 us in chunks of 128, 120 of 256; 2,048 tokens 199, 180 and, of 512, 224; 8,192 tokens
+    695, 600, 540)."""
+    return 128 if longest <= 1024 else 256 if longest <= 4096 else 512
 
 
 def delta_prep(qkv: torch.Tensor, conv: torch.Tensor, a: torch.Tensor, b: torch.Tensor, a_log, dt_bias, tail, ctx, heads: int,
@@ -1952,7 +1958,7 @@ def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: to
     y = torch.empty((M, heads * value_dim), dtype=torch.float32, device=qkv.device)
     timing_hint["rows"] = M
     longest = int(max(ctx.new_tokens))
-    chunk, chunks = DELTA_CHUNK_TOKENS, 1
+    chunk, chunks = delta_chunk(longest), 1
     hat = ta = chunk_state = None
     if longest >= DELTA_BLOCKS_FROM:
         # (room behind the last token: its block's loads are of sixteen whole tokens, in vectors that may start inside the last)

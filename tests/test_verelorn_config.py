@@ -82,7 +82,7 @@ def _spec(cfg, shapes=None):
 
     c = AutoConfig.from_dict(cfg)
     if shapes is not None:
-        c.sizes_from_weights(shapes)
+        c.sizes_from_weights(lambda: shapes)
     spec = lookup(c.model_type)[1](c)
     spec.validate()
     return spec
