@@ -8,6 +8,7 @@ from .engine import bimepel as _bimepel  # registers model_type "bimepel"  # noq
 from .engine import kekapel as _kekapel  # registers model_type "kekapel"  # noqa: F401
 from .engine import nopuzen as _nopuzen  # registers model_type "nopuzen"  # noqa: F401
 from .engine import verelorn as _verelorn  # registers model_type "verelorn"  # noqa: F401
+from .engine import narezen as _narezen  # registers model_type "narezen"  # noqa: F401
 from .auto import AutoModelForCausalLM
 from .pipeline import TextGenerationPipeline, pipeline
 from .sampling.custom import LogitsProcessor, LogitsProcessorList, StoppingCriteria, StoppingCriteriaList

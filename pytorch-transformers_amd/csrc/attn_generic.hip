@@ -20,7 +20,7 @@ __global__ void attn_generic_kernel(T* __restrict__ out, const T* __restrict__ q
                                     int bt_stride, const int* __restrict__ token_seq,
                                     const int* __restrict__ token_pos, const float* __restrict__ slopes, int bias_mode, float bias_scale,
                                     int nh, int nkv, int d, float scale, int window, int chunk,
-                                    const float* __restrict__ sink) {
+                                    const float* __restrict__ sink, PtaHeadRows rows) {
     __shared__ float q_s[256];
     __shared__ float p_s[PTA_PAGE];
     const int m = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -74,7 +74,7 @@ __global__ void attn_generic_kernel(T* __restrict__ out, const T* __restrict__ q
         }
         m_run = m_new;
     }
-    T* orow = out + ((long)m * nh + h) * d;
+    T* orow = out + (long)m * rows.ld + (long)h * rows.head;
     // a learned number per head: its exponential joins the sum of the weights once, with no key and no value
     float last = 1.f;
     if (sink) {
@@ -82,11 +82,11 @@ __global__ void attn_generic_kernel(T* __restrict__ out, const T* __restrict__ q
         last = expf(m_run - m_new);
         l_run = l_run * last + expf(sink[h] - m_new);
     }
-    const float inv = last / l_run;
+    const float inv = last / l_run * rows.mult;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
         const int dim = lane + r * PTA_WAVE;
-        if (dim < d) Io<T>::st(orow + dim, acc[r] * inv);
+        if (dim < rows.keep) Io<T>::st(orow + dim, acc[r] * inv);
     }
 }
 
@@ -104,7 +104,7 @@ extern "C" int pta_attention_sizes_ok(int nh, int nkv, int d, int rotated) {
 extern "C" int pta_attn_generic(void* out, const void* q, const void* k_pool, const void* v_pool,
                                 const int* block_table, int bt_stride, const int* token_seq, const int* token_pos,
                                 const PtaScoreBias* score_bias, int M, int nh, int nkv, int d, float scale, int window, int chunk,
-                                const float* sink, int dtype, void* stream) {
+                                const float* sink, const PtaHeadRows* head_rows, int dtype, void* stream) {
     int bias_mode = 0;
     if (pta_score_bias_mode("attn_generic", score_bias, &bias_mode)) return 1;
     const float* slopes = score_bias ? score_bias->slopes : nullptr;
@@ -115,16 +115,18 @@ extern "C" int pta_attn_generic(void* out, const void* q, const void* k_pool, co
     PTA_REQUIRE(nh <= 65535, "attn_generic: at most 65535 heads, got %d", nh);
     PTA_REQUIRE(window >= 0, "attn_generic: window must be 0 (none) or positive, got %d", window);
     PTA_REQUIRE(chunk >= 0, "attn_generic: chunk must be 0 (none) or positive, got %d", chunk);
+    const PtaHeadRows rows = pta_head_rows_of(head_rows, nh, d);
+    if (pta_check_head_rows("attn_generic", rows, nh, d, out, 1)) return 1;
     hipStream_t s = (hipStream_t)stream;
     dim3 grid(M, nh);
     if (dtype == PTA_F32)
         hipLaunchKernelGGL(attn_generic_kernel<float>, grid, dim3(PTA_WAVE), 0, s, (float*)out, (const float*)q,
                            (const float*)k_pool, (const float*)v_pool, block_table, bt_stride, token_seq, token_pos,
-                           slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink);
+                           slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink, rows);
     else if (dtype == PTA_BF16)
         hipLaunchKernelGGL(attn_generic_kernel<bf16_t>, grid, dim3(PTA_WAVE), 0, s, (bf16_t*)out, (const bf16_t*)q,
                            (const bf16_t*)k_pool, (const bf16_t*)v_pool, block_table, bt_stride, token_seq,
-                           token_pos, slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink);
+                           token_pos, slopes, bias_mode, bias_scale, nh, nkv, d, scale, window, chunk, sink, rows);
     else
         return pta_fail("attn_generic: unknown dtype %d", dtype);
     return pta_check_launch("attn_generic");

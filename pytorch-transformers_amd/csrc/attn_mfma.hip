@@ -19,7 +19,7 @@ PTA_ATTN_HEAD(8) PTA_ATTN_HEAD(16)
 template <int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void attn_combine_kernel(bf16_t* __restrict__ out, const float* __restrict__ po,
                                                                   const float* __restrict__ pm, const float* __restrict__ pl,
-                                                                  int D, int n_splits, int lps, const float* __restrict__ sink, int nh) {
+                                                                  int D, int n_splits, int lps, const float* __restrict__ sink, int nh, PtaHeadRows rows) {
     __shared__ float part[WAVES][256 + 4];
     const long row = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -79,26 +79,29 @@ __global__ __launch_bounds__(64 * WAVES) void attn_combine_kernel(bf16_t* __rest
     }
     if (g == 0 && active) {
         if (sink) L += __builtin_amdgcn_exp2f(sink[row % nh] * PTA_LOG2E - mx);
-        const float inv = 1.0f / L;
+        const float inv = rows.mult / L;
         bf16_t r[4] = {f32_to_bf16_bits(acc.x * inv), f32_to_bf16_bits(acc.y * inv), f32_to_bf16_bits(acc.z * inv),
                        f32_to_bf16_bits(acc.w * inv)};
-        *reinterpret_cast<uint2*>(out + row * D + c) = *reinterpret_cast<const uint2*>(r);
+        if (c < rows.keep)
+            *reinterpret_cast<uint2*>(out + row / nh * rows.ld + row % nh * rows.head + c) = *reinterpret_cast<const uint2*>(r);
     }
 }
 
 extern "C" int pta_attn_combine(void* out, const float* po, const float* pm, const float* pl, long n_rows, int d,
-                                int n_splits, const float* sink, int nh, void* stream) {
-    PTA_REQUIRE(!sink || nh > 0, "attn_combine: numbers per head need the number of heads");
+                                int n_splits, const float* sink, int nh, const PtaHeadRows* head_rows, void* stream) {
+    PTA_REQUIRE(nh > 0 && n_rows % nh == 0, "attn_combine: %ld rows are no multiple of %d heads", n_rows, nh);
     PTA_REQUIRE(n_rows > 0 && n_rows <= 0x7fffffffL && d > 0 && d <= 256 && d % 4 == 0 && n_splits >= 1,
                 "attn_combine: %ld rows of %d elements in %d ranges", n_rows, d, n_splits);
     hipStream_t s = (hipStream_t)stream;
+    const PtaHeadRows to = pta_head_rows_of(head_rows, nh, d);
+    if (pta_check_head_rows("attn_combine", to, nh, d, out, 4)) return 1;
     int lps = 4;  // lanes that share a split's vector of d floats, a float4 each
     while (lps * 4 < d) lps *= 2;
     const dim3 rows((unsigned)n_rows);
     if (n_splits > 4 * (64 / lps))  // more splits than one wave has in flight at once
-        hipLaunchKernelGGL(attn_combine_kernel<4>, rows, dim3(256), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh);
+        hipLaunchKernelGGL(attn_combine_kernel<4>, rows, dim3(256), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh, to);
     else
-        hipLaunchKernelGGL(attn_combine_kernel<1>, rows, dim3(64), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh);
+        hipLaunchKernelGGL(attn_combine_kernel<1>, rows, dim3(64), 0, s, (bf16_t*)out, po, pm, pl, d, n_splits, lps, sink, nh, to);
     return pta_check_launch("attn_combine");
 }
 
@@ -118,7 +121,7 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
                              int bt_stride, const int* cu_tokens, const int* seq_start, const PtaScoreBias* score_bias,
                              int n_seqs, int max_new, int M, int nh, int nkv, int d, float scale, int split_size, int n_splits,
                              float* po, float* pm, float* pl, int window, int chunk, int decode_tiles, int decode_waves,
-                             int prompt_wide, const float* sink, void* stream) {
+                             int prompt_wide, const float* sink, const PtaHeadRows* head_rows, void* stream) {
     PTA_REQUIRE(n_seqs > 0 && max_new > 0 && M > 0 && nh > 0 && nkv > 0, "attn_mfma: sizes must be positive");
     int bias_mode = 0;
     if (pta_score_bias_mode("attn_mfma", score_bias, &bias_mode)) return 1;
@@ -134,6 +137,8 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
     PTA_REQUIRE((long)n_seqs * n_splits <= 65535 && nkv <= 65535, "attn_mfma: too many sequences x splits for one launch");
     PTA_REQUIRE(((uintptr_t)q % 16) == 0 && ((uintptr_t)k_pool % 16) == 0 && ((uintptr_t)v_pool % 16) == 0 &&
                     ((uintptr_t)out % 8) == 0, "attn_mfma: pointers must be 16-byte aligned");
+    const PtaHeadRows rows = pta_head_rows_of(head_rows, nh, d);
+    if (pta_check_head_rows("attn_mfma", rows, nh, d, out, 4)) return 1;
     hipStream_t s = (hipStream_t)stream;
     // Prompts: four waves of two column tiles share each stage of keys through LDS (head sizes up to 128;
     // beyond, one wave per workgroup).
@@ -181,7 +186,7 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
                 "(one wave, or four or eight with up to two tiles)", decode_waves, dct, d);
     const AttnLaunch a{(bf16_t*)out, po, pm, pl, (const bf16_t*)q, (const bf16_t*)k_pool, (const bf16_t*)v_pool,
                        block_table, bt_stride, cu_tokens, seq_start, slopes, bias_mode, bias_scale, sink, n_seqs, max_new, nh, nkv, scale,
-                       split_size, n_splits, window, chunk, paired, narrow ? decode_waves : 1, s};
+                       split_size, n_splits, window, chunk, paired, narrow ? decode_waves : 1, rows, s};
 #define PTA_ATTN_CASE(DT_)                                                                        \
     case DT_: {                                                                                   \
         const int none = attn_launch_head<DT_>(a, shared, narrow, wide, dct);                     \
@@ -206,6 +211,6 @@ extern "C" int pta_attn_mfma(void* out, const void* q, const void* k_pool, const
 #undef PTA_ATTN_CASE
     int rc = pta_check_launch("attn_mfma");
     if (rc) return rc;
-    if (n_splits > 1) rc = pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, sink, nh, stream);
+    if (n_splits > 1) rc = pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, sink, nh, head_rows, stream);
     return rc;
 }

@@ -119,7 +119,7 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
     const int* __restrict__ block_table, int bt_stride, const int* __restrict__ cu_tokens,
     const int* __restrict__ seq_start, const float* __restrict__ slopes, int bias_mode, int nh, int nkv, float scale,
     float alibi_mul,
-    int split_size, int n_splits, int window_arg, int chunk_arg, int paired, const float* __restrict__ sink) {
+    int split_size, int n_splits, int window_arg, int chunk_arg, int paired, const float* __restrict__ sink, PtaHeadRows rows) {
     constexpr int D = DT * 16;
     const int window = WIN ? window_arg : 0;
     const int chunk = WIN ? chunk_arg : 0;  // blocks of positions that a token does not see out of (0: none)
@@ -511,11 +511,12 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
                 const long row = (long)tok[ct] * nh + head[ct];
                 if (n_splits == 1) {
                     if (sink) l += __builtin_amdgcn_exp2f(sink[head[ct]] * PTA_LOG2E - mx);
-                    const float inv = 1.0f / l;
+                    const float inv = rows.mult / l;
                     uint2 w2;
                     w2.x = pack_bf16(acc.x * inv, acc.y * inv);
                     w2.y = pack_bf16(acc.z * inv, acc.w * inv);
-                    *reinterpret_cast<uint2*>(out + row * D + dt * 16 + gq * 4) = w2;
+                    if (dt * 16 + gq * 4 < rows.keep)
+                        *reinterpret_cast<uint2*>(out + (long)tok[ct] * rows.ld + (long)head[ct] * rows.head + dt * 16 + gq * 4) = w2;
                 } else {
                     *reinterpret_cast<float4*>(po + (row * n_splits + split) * D + dt * 16 + gq * 4) = acc;
                     if (dt == 0 && gq == 0) {
@@ -533,14 +534,14 @@ __global__ __launch_bounds__(64 * W * KS, OCC) void attn_mfma_kernel(
         const long row = (long)tok[ct] * nh + head[ct];
         if (n_splits == 1) {
             if (sink) l += __builtin_amdgcn_exp2f(sink[head[ct]] * PTA_LOG2E - m_run[ct]);
-            const float inv = 1.0f / l;
-            bf16_t* o = out + row * D;
+            const float inv = rows.mult / l;
+            bf16_t* o = out + (long)tok[ct] * rows.ld + (long)head[ct] * rows.head;
 #pragma unroll
             for (int dt = 0; dt < DT; ++dt) {
                 uint2 w;
                 w.x = pack_bf16(oacc[dt][ct][0] * inv, oacc[dt][ct][1] * inv);
                 w.y = pack_bf16(oacc[dt][ct][2] * inv, oacc[dt][ct][3] * inv);
-                *reinterpret_cast<uint2*>(o + dt * 16 + gq * 4) = w;
+                if (dt * 16 + gq * 4 < rows.keep) *reinterpret_cast<uint2*>(o + dt * 16 + gq * 4) = w;
             }
         } else {
             // a range past the column's keys has nothing to add: only its marker is written, and the combine
@@ -573,6 +574,7 @@ struct AttnLaunch {
     int chunk;   // 0, or the size of the blocks of positions that a token does not see out of
     int paired;  // workgroups take two column groups each, a late one and the early one that mirrors it
     int waves;   // one token per sequence: waves of a workgroup that divide its keys among them
+    PtaHeadRows rows;
     hipStream_t s;
 };
 
@@ -602,7 +604,7 @@ static void launch_attn(const AttnLaunch& a) {
     }
     hipLaunchKernelGGL(kern, grid, dim3(64 * W * KS), lds, a.s, a.out, a.po, a.pm, a.pl, a.q, a.k_pool, a.v_pool,
                        a.block_table, a.bt_stride, a.cu_tokens, a.seq_start, a.slopes, a.bias_mode, a.nh, a.nkv,
-                       a.scale * PTA_LOG2E, PTA_LOG2E * a.bias_scale, a.split_size, a.n_splits, a.window, a.chunk, paired, a.sink);
+                       a.scale * PTA_LOG2E, PTA_LOG2E * a.bias_scale, a.split_size, a.n_splits, a.window, a.chunk, paired, a.sink, a.rows);
 }
 
 // column tiles (of sixteen query heads of one KV head) that one wave of a decode launch holds at most:

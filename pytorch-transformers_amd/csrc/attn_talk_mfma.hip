@@ -95,5 +95,5 @@ extern "C" int pta_attn_talk_mfma(void* out, const void* q, const void* k_pool, 
     if (!built) return pta_fail("attn_talk_mfma: no kernel for %d heads a wave at head size %d", ct, d);
     int rc = pta_check_launch("attn_talk_mfma");
     if (rc || n_splits == 1) return rc;
-    return pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, nullptr, nh, stream);
+    return pta_attn_combine(out, po, pm, pl, (long)M * nh, d, n_splits, nullptr, nh, nullptr, stream);
 }

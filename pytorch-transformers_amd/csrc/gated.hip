@@ -10,8 +10,9 @@
 //                   PTA_GLU_SILU        silu(gate) * up
 //                   PTA_GLU_GELU_TANH   gelu_tanh(gate) * up
 //                   PTA_GLU_CLAMPED     g = min(gate, limit), u = clamp(up, -limit, limit): g * sigmoid(alpha g) * (u + 1)
-// pta_head_norm_gate: out[m, h * dv + e] = x / sqrt(mean over the head's dv elements (x^2) + eps) * w[e] * sigmoid(g),
-//                   every head by its own root mean square, one weight [dv] for all heads.
+// pta_head_norm_gate: out[m, h * dv + e] = x / sqrt(mean over the head's dv elements (x^2) + eps) * w[e] * gate(g) * mult,
+//                   every head by its own root mean square, one weight [dv] for all heads (null: ones); gate is the
+//                   sigmoid or silu.
 // Arithmetic in 32-bit, results in the compute type.
 #include "common.h"
 #include "pta_kernels.h"
@@ -86,7 +87,8 @@ __global__ void glu_kernel(T* __restrict__ out, const T* __restrict__ gate, cons
 }
 
 // bfloat16 rows of a multiple of eight elements at sixteen-byte addresses: eight elements a thread
-__global__ void glu_gelu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
+template <int KIND>
+__global__ void glu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
                                        long in_ld, int F8, long n8) {
     const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= n8) return;
@@ -96,6 +98,10 @@ __global__ void glu_gelu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* _
     unpack8(*reinterpret_cast<const uint4*>(up + m * in_ld + f), u);
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
+        if constexpr (KIND == PTA_GLU_SILU) {
+            g[j] = g[j] / (1.0f + __expf(-g[j])) * u[j];
+            continue;
+        }
         // tanh(z) = 1 - 2 / (1 + e^(2z)): both ends saturate without a branch (e^(2z) to infinity or to zero)
         const float z = 0.79788456080286535588f * (g[j] + 0.044715f * g[j] * g[j] * g[j]);
         g[j] = g[j] * (1.0f - 1.0f / (1.0f + __expf(2.0f * z))) * u[j];
@@ -112,9 +118,10 @@ extern "C" int pta_glu(void* out, const void* gate, const void* up, long in_ld, 
     hipStream_t s = (hipStream_t)stream;
     const long n = (long)M * F;
     const dim3 grid((unsigned)((n + 255) / 256));
-    if (dtype == PTA_BF16 && kind == PTA_GLU_GELU_TANH && F % 8 == 0 && in_ld % 8 == 0 && ((uintptr_t)gate % 16) == 0 &&
+    if (dtype == PTA_BF16 && kind != PTA_GLU_CLAMPED && F % 8 == 0 && in_ld % 8 == 0 && ((uintptr_t)gate % 16) == 0 &&
         ((uintptr_t)up % 16) == 0 && ((uintptr_t)out % 16) == 0) {
-        hipLaunchKernelGGL(glu_gelu_bf16x8_kernel, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0, s, (bf16_t*)out,
+        auto kern = kind == PTA_GLU_SILU ? glu_bf16x8_kernel<PTA_GLU_SILU> : glu_bf16x8_kernel<PTA_GLU_GELU_TANH>;
+        hipLaunchKernelGGL(kern, dim3((unsigned)((n / 8 + 255) / 256)), dim3(256), 0, s, (bf16_t*)out,
                            (const bf16_t*)gate, (const bf16_t*)up, in_ld, F / 8, n / 8);
         return pta_check_launch("glu");
     }
@@ -262,9 +269,9 @@ extern "C" int pta_polynorm(void* out, const void* z, long z_ld, const float* co
 
 // one wave per (token, head)
 template <typename T>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out, const float* __restrict__ x, const T* __restrict__ g,
-                                                             long g_ld, const float* __restrict__ w, float eps, long units,
-                                                             int heads, int dv) {
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out, long out_ld, const float* __restrict__ x,
+                                                             const T* __restrict__ g, long g_ld, const float* __restrict__ w,
+                                                             float eps, int silu, float mult, long units, int heads, int dv) {
     const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (unit >= units) return;
     const int lane = threadIdx.x & 63;
@@ -274,23 +281,28 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(T* __restrict__ out
     float ss = 0.f;
     for (int e = lane; e < dv; e += PTA_WAVE) ss += xr[e] * xr[e];
     const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
-    for (int e = lane; e < dv; e += PTA_WAVE)
-        Io<T>::st(out + unit * dv + e, xr[e] * inv * w[e] / (1.0f + expf(-Io<T>::ld(gr + e))));
+    for (int e = lane; e < dv; e += PTA_WAVE) {
+        const float gv = Io<T>::ld(gr + e);
+        const float gate = (silu ? gv : 1.0f) / (1.0f + expf(-gv));
+        Io<T>::st(out + m * out_ld + h * dv + e, xr[e] * inv * (w ? w[e] : 1.0f) * gate * mult);
+    }
 }
 
-// x [M, heads * dv] 32-bit, dense; g [M, heads * dv] rows g_ld apart, out dense, both in the compute type; w [dv]
-extern "C" int pta_head_norm_gate(void* out, const float* x, const void* g, long g_ld, const float* w, float eps, int M,
-                                  int heads, int dv, int dtype, void* stream) {
+// x [M, heads * dv] 32-bit, dense; g [M, heads * dv] rows g_ld apart and out, rows out_ld apart, in the compute type; w [dv]
+extern "C" int pta_head_norm_gate(void* out, long out_ld, const float* x, const void* g, long g_ld, const float* w, float eps,
+                                  int gate_act, float mult, int M, int heads, int dv, int dtype, void* stream) {
     PTA_REQUIRE(M > 0 && heads > 0 && dv > 0, "head_norm_gate: sizes must be positive");
-    PTA_REQUIRE(out && x && g && w, "head_norm_gate: null pointer");
-    PTA_REQUIRE(g_ld >= (long)heads * dv, "head_norm_gate: rows of the gate lie closer together than they are long");
+    PTA_REQUIRE(out && x && g, "head_norm_gate: null pointer");
+    PTA_REQUIRE(g_ld >= (long)heads * dv && out_ld >= (long)heads * dv, "head_norm_gate: rows lie closer together than they are long");
+    PTA_REQUIRE(gate_act == PTA_ACT_SIGMOID || gate_act == PTA_ACT_SILU, "head_norm_gate: a gate of kind %d is not built", gate_act);
     PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "head_norm_gate: unknown dtype %d", dtype);
     hipStream_t s = (hipStream_t)stream;
     const long units = (long)M * heads;
     const dim3 grid((unsigned)((units + 3) / 4));
+    const int silu = gate_act == PTA_ACT_SILU;
     if (dtype == PTA_F32)
-        hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, s, (float*)out, x, (const float*)g, g_ld, w, eps, units, heads, dv);
+        hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, s, (float*)out, out_ld, x, (const float*)g, g_ld, w, eps, silu, mult, units, heads, dv);
     else
-        hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, s, (bf16_t*)out, x, (const bf16_t*)g, g_ld, w, eps, units, heads, dv);
+        hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, s, (bf16_t*)out, out_ld, x, (const bf16_t*)g, g_ld, w, eps, silu, mult, units, heads, dv);
     return pta_check_launch("head_norm_gate");
 }

@@ -3,7 +3,7 @@
 //   z = W_r h (32-bit); s = score(z) (sigmoid, or softmax over the experts); the `top` largest s are taken;
 //   weights = s / (sum of the taken s + 1e-20) * scale   (or the taken s times scale, unnormalised);
 //   out = sum over the taken experts e of weight_e * D_e (act(G_e h) * (U_e h))
-//   (z may have a bias added; in place of act(g) * u an expert may have the clamped gate of PtaGate, pta_kernels.h;
+//   (the weight may stand on the input instead, out = sum over e of D_e (act(w_e G_e h) * (w_e U_e h)); z may have a bias added; in place of act(g) * u an expert may have the clamped gate of PtaGate, pta_kernels.h;
 //    an expert without a gate is D_e act(U_e h), its matrices stacked as up [E, F, H]; with groups the experts form
 //    `groups` equal runs of neighbours, a run's score is its largest s, and only experts of the `keep` best runs can
 //    be taken; the router's launch can also form sigmoid(X h) for a few more 32-bit rows X, e.g. the gate of an expert
@@ -190,10 +190,12 @@ extern "C" int pta_moe_route(int* ids, float* wts, const void* h, long h_ld, con
 template <typename T>
 __global__ __launch_bounds__(256) void moe_up_kernel(T* __restrict__ act_out, const T* __restrict__ h, long h_ld,
                                                      const T* __restrict__ gate_up, const int* __restrict__ ids, int H,
-                                                     int F, int top, int act, PtaGate gate, int gated) {
+                                                     int F, int top, int act, PtaGate gate, int gated,
+                                                     const float* __restrict__ in_wts) {
     extern __shared__ __attribute__((aligned(16))) float x_s[];  // [H]
     const int pair = blockIdx.x, m = pair / top, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int e = ids[pair];
+    const float in_w = in_wts ? in_wts[pair] : 1.f;  // (on the 32-bit sums: the same as on the input, rounded once less)
     for (int i = threadIdx.x; i < H; i += blockDim.x) x_s[i] = Io<T>::ld(h + (long)m * h_ld + i);
     __syncthreads();
     const T* G = gate_up + (long)e * (gated ? 2 : 1) * F * H;
@@ -209,7 +211,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(T* __restrict__ act_out, co
 #pragma unroll
             for (int r = 1; r < 4; ++r)
                 if (lane == r) gv = g[r];
-            Io<T>::st(act_out + (long)pair * F + f0 + lane, apply_act(Io<T>::round(gv), act));
+            Io<T>::st(act_out + (long)pair * F + f0 + lane, apply_act(Io<T>::round(in_w * gv), act));
         }
         return;
     }
@@ -220,7 +222,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(T* __restrict__ act_out, co
 #pragma unroll
         for (int r = 1; r < 4; ++r)
             if (lane == r) { gv = g[r]; uv = u[r]; }
-        Io<T>::st(act_out + (long)pair * F + f0 + lane, gate_value(Io<T>::round(gv), Io<T>::round(uv), act, gate));
+        Io<T>::st(act_out + (long)pair * F + f0 + lane, gate_value(Io<T>::round(in_w * gv), Io<T>::round(in_w * uv), act, gate));
     }
 }
 
@@ -240,7 +242,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(T* __restrict__ out, cons
     for (int k = 0; k < top; ++k) {
         float d[4];
         wave_dots<T, 4>(down + ((long)ids[(long)m * top + k] * H + n0) * F, F, rows, a_s + k * F, F, lane, d);
-        const float wk = wts[(long)m * top + k];
+        const float wk = wts ? wts[(long)m * top + k] : 1.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) acc[r] += wk * Io<T>::round(d[r]);
     }
@@ -249,14 +251,15 @@ __global__ __launch_bounds__(256) void moe_down_kernel(T* __restrict__ out, cons
 #pragma unroll
         for (int r = 1; r < 4; ++r)
             if (lane == r) v = acc[r];
-        if (extra) v += extra_gate[(long)m * gate_ld] * Io<T>::ld(extra + (long)m * H + n0 + lane);
+        if (extra) v += (extra_gate ? extra_gate[(long)m * gate_ld] : 1.f) * Io<T>::ld(extra + (long)m * H + n0 + lane);
         Io<T>::st(out + (long)m * H + n0 + lane, v);
     }
 }
 
-// act_out [M * top, F]; h [M, H] rows h_ld apart; gate_up [E, 2F, H] (gated) or [E, F, H]; ids [M, top]
+// act_out [M * top, F]; h [M, H] rows h_ld apart; gate_up [E, 2F, H] (gated) or [E, F, H]; ids [M, top]; in_wts [M, top] (null:
+// ones) multiplies the input
 extern "C" int pta_moe_up(void* act_out, const void* h, long h_ld, const void* gate_up, const int* ids, int M, int H, int F,
-                          int top, int act, const PtaGate* gate_how, int gated, int dtype, void* stream) {
+                          int top, int act, const PtaGate* gate_how, int gated, const float* in_wts, int dtype, void* stream) {
     const PtaGate gate = gate_how ? *gate_how : PtaGate{PTA_GLU_SILU, 1.f, 0.f};
     PTA_REQUIRE(gate.kind == PTA_GLU_SILU || gate.kind == PTA_GLU_CLAMPED, "moe_up: a gate of kind %d is not built", gate.kind);
     PTA_REQUIRE(M > 0 && H > 0 && F > 0 && top > 0 && act_out && h && gate_up && ids && h_ld >= H, "moe_up: sizes must be positive and pointers given");
@@ -266,18 +269,19 @@ extern "C" int pta_moe_up(void* act_out, const void* h, long h_ld, const void* g
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid((unsigned)((long)M * top), (F + MOE_ROWS - 1) / MOE_ROWS);
     if (dtype == PTA_F32)
-        hipLaunchKernelGGL(moe_up_kernel<float>, grid, dim3(256), (size_t)H * 4, s, (float*)act_out, (const float*)h, h_ld, (const float*)gate_up, ids, H, F, top, act, gate, gated);
+        hipLaunchKernelGGL(moe_up_kernel<float>, grid, dim3(256), (size_t)H * 4, s, (float*)act_out, (const float*)h, h_ld, (const float*)gate_up, ids, H, F, top, act, gate, gated, in_wts);
     else
-        hipLaunchKernelGGL(moe_up_kernel<bf16_t>, grid, dim3(256), (size_t)H * 4, s, (bf16_t*)act_out, (const bf16_t*)h, h_ld, (const bf16_t*)gate_up, ids, H, F, top, act, gate, gated);
+        hipLaunchKernelGGL(moe_up_kernel<bf16_t>, grid, dim3(256), (size_t)H * 4, s, (bf16_t*)act_out, (const bf16_t*)h, h_ld, (const bf16_t*)gate_up, ids, H, F, top, act, gate, gated, in_wts);
     return pta_check_launch("moe_up");
 }
 
 // out [M, H]; act_in [M * top, F]; down [E, H, F]
-// extra [M, H] (compute type) and extra_gate (32-bit, one number a token, gate_ld apart), both or neither: out += gate * extra
+// wts null: ones.  extra [M, H] (compute type) and extra_gate (32-bit, one number a token, gate_ld apart; null: ones): out +=
+// gate * extra
 extern "C" int pta_moe_down(void* out, const void* act_in, const void* down, const int* ids, const float* wts, int M, int H,
                             int F, int top, const void* extra, const float* extra_gate, int gate_ld, int dtype, void* stream) {
-    PTA_REQUIRE((extra != nullptr) == (extra_gate != nullptr), "moe_down: a further term and its gate come together");
-    PTA_REQUIRE(M > 0 && H > 0 && F > 0 && top > 0 && out && act_in && down && ids && wts, "moe_down: sizes must be positive and pointers given");
+    PTA_REQUIRE(extra || !extra_gate, "moe_down: a gate of a further term without the term");
+    PTA_REQUIRE(M > 0 && H > 0 && F > 0 && top > 0 && out && act_in && down && ids, "moe_down: sizes must be positive and pointers given");
     PTA_REQUIRE((size_t)top * F * 4 <= 160 * 1024 && (H + MOE_ROWS - 1) / MOE_ROWS <= 65535,
                 "moe_down: %d experts of %d rows a token are more than the kernel's LDS holds", top, F);
     PTA_REQUIRE(dtype == PTA_F32 || dtype == PTA_BF16, "moe_down: unknown dtype %d", dtype);
@@ -439,7 +443,7 @@ __global__ __launch_bounds__(256) void moe_grouped_up_kernel(bf16_t* __restrict_
                                                              long x_ld, const bf16_t* __restrict__ gate_up,
                                                              const int* __restrict__ sorted_pair,
                                                              const int* __restrict__ tile_expert, int H, int F, int top,
-                                                             int act, PtaGate gate, int tiles) {
+                                                             int act, PtaGate gate, int tiles, const float* __restrict__ in_wts) {
     __shared__ __attribute__((aligned(16))) bf16_t lds[2 * MOE_TILE * MOE_XROW];
     int tile, fb;
     if (!moe_item(tiles, (F + 127) / 128, &tile, &fb)) return;
@@ -461,12 +465,14 @@ __global__ __launch_bounds__(256) void moe_grouped_up_kernel(bf16_t* __restrict_
 #pragma unroll
     for (int tt = 0; tt < 4; ++tt) {
         const long slot = (long)tile * MOE_TILE + tt * 16 + c;
+        const int sp = in_wts ? sorted_pair[slot] : -1;
+        const float in_w = sp >= 0 ? in_wts[sp] : 1.f;
 #pragma unroll
         for (int half = 0; half < 2; ++half) {
             float y[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-                y[j] = gate_value(round_to_bf16(acc[half][tt][j]), round_to_bf16(acc[2 + half][tt][j]), act, gate);
+                y[j] = gate_value(round_to_bf16(in_w * acc[half][tt][j]), round_to_bf16(in_w * acc[2 + half][tt][j]), act, gate);
             const int f = f0 + half * 16 + 4 * gq;
             moe_store4(act_sorted + slot * F + f, f, F, y[0], y[1], y[2], y[3]);
         }
@@ -479,7 +485,7 @@ __global__ __launch_bounds__(256) void moe_grouped_up_plain_kernel(bf16_t* __res
                                                                    long x_ld, const bf16_t* __restrict__ up,
                                                                    const int* __restrict__ sorted_pair,
                                                                    const int* __restrict__ tile_expert, int H, int F, int top,
-                                                                   int act, int tiles) {
+                                                                   int act, int tiles, const float* __restrict__ in_wts) {
     __shared__ __attribute__((aligned(16))) bf16_t lds[2 * MOE_TILE * MOE_XROW];
     int tile, fb;
     if (!moe_item(tiles, (F + 255) / 256, &tile, &fb)) return;
@@ -498,11 +504,13 @@ __global__ __launch_bounds__(256) void moe_grouped_up_plain_kernel(bf16_t* __res
 #pragma unroll
     for (int tt = 0; tt < 4; ++tt) {
         const long slot = (long)tile * MOE_TILE + tt * 16 + c;
+        const int sp = in_wts ? sorted_pair[slot] : -1;
+        const float in_w = sp >= 0 ? in_wts[sp] : 1.f;
 #pragma unroll
         for (int a = 0; a < 4; ++a) {
             float y[4];
 #pragma unroll
-            for (int j = 0; j < 4; ++j) y[j] = apply_act(round_to_bf16(acc[a][tt][j]), act);
+            for (int j = 0; j < 4; ++j) y[j] = apply_act(round_to_bf16(in_w * acc[a][tt][j]), act);
             const int f = f0 + a * 16 + 4 * gq;
             moe_store4(act_sorted + slot * F + f, f, F, y[0], y[1], y[2], y[3]);
         }
@@ -547,21 +555,21 @@ __global__ void moe_combine_kernel(bf16_t* __restrict__ out, const bf16_t* __res
     for (int n = threadIdx.x; n < H; n += blockDim.x) {
         float acc = 0.f;
         for (int k = 0; k < top; ++k)
-            acc += wts[(long)m * top + k] * bf16_bits_to_f32(y_sorted[(long)slot_of_pair[(long)m * top + k] * H + n]);
-        if (extra) acc += extra_gate[(long)m * gate_ld] * bf16_bits_to_f32(extra[(long)m * H + n]);
+            acc += (wts ? wts[(long)m * top + k] : 1.f) * bf16_bits_to_f32(y_sorted[(long)slot_of_pair[(long)m * top + k] * H + n]);
+        if (extra) acc += (extra_gate ? extra_gate[(long)m * gate_ld] : 1.f) * bf16_bits_to_f32(extra[(long)m * H + n]);
         out[(long)m * H + n] = f32_to_bf16_bits(acc);
     }
 }
 
 extern "C" int pta_moe_grouped_slots(int pairs, int E) { return (pairs + E * (MOE_TILE - 1) + MOE_TILE - 1) / MOE_TILE * MOE_TILE; }
 
-// bfloat16 only; H and F multiples of 64.  sorted_pair [slots], slot_of_pair [M * top], tile_expert [slots / 64],
+// bfloat16 only; H and F multiples of 64.  weight_input: the weights multiply the experts' input, not their output.  sorted_pair [slots], slot_of_pair [M * top], tile_expert [slots / 64],
 // act_sorted [slots, F], y_sorted [slots, H] are the caller's scratch (slots = pta_moe_grouped_slots(M * top, E)).
 extern "C" int pta_moe_grouped(void* out, const void* x, long x_ld, const void* gate_up, const void* down, const int* ids,
                                const float* wts, int* sorted_pair, int* slot_of_pair, int* tile_expert, void* act_sorted,
                                void* y_sorted, int M, int H, int F, int E, int top, int act, const PtaGate* gate_how,
-                               int gated, const void* extra, const float* extra_gate, int gate_ld, void* stream) {
-    PTA_REQUIRE((extra != nullptr) == (extra_gate != nullptr), "moe_grouped: a further term and its gate come together");
+                               int gated, int weight_input, const void* extra, const float* extra_gate, int gate_ld, void* stream) {
+    PTA_REQUIRE(extra || !extra_gate, "moe_grouped: a gate of a further term without the term");
     const PtaGate gate = gate_how ? *gate_how : PtaGate{PTA_GLU_SILU, 1.f, 0.f};
     PTA_REQUIRE(gate.kind == PTA_GLU_SILU || gate.kind == PTA_GLU_CLAMPED, "moe_grouped: a gate of kind %d is not built", gate.kind);
     PTA_REQUIRE(M > 0 && H > 0 && F > 0 && E > 0 && top > 0, "moe_grouped: sizes must be positive");
@@ -575,19 +583,20 @@ extern "C" int pta_moe_grouped(void* out, const void* x, long x_ld, const void* 
     const long pairs = (long)M * top;
     const int slots = pta_moe_grouped_slots((int)pairs, E), tiles = slots / MOE_TILE;
     PTA_REQUIRE(pairs < (1L << 30) && tiles <= 2147483647 / 64, "moe_grouped: too many pairs");
+    const float* in_wts = weight_input ? wts : nullptr;
     hipStream_t s = (hipStream_t)stream;
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), (size_t)(3 * E + 1) * 4, s, sorted_pair, slot_of_pair, tile_expert,
                        ids, (int)pairs, E, slots, tiles);
     auto grid_for = [&](int blocks) { return dim3((unsigned)(((long)tiles * blocks + 7) / 8 * 8)); };
     if (gated)
         hipLaunchKernelGGL(moe_grouped_up_kernel, grid_for((F + 127) / 128), dim3(256), 0, s, (bf16_t*)act_sorted, (const bf16_t*)x,
-                           x_ld, (const bf16_t*)gate_up, sorted_pair, tile_expert, H, F, top, act, gate, tiles);
+                           x_ld, (const bf16_t*)gate_up, sorted_pair, tile_expert, H, F, top, act, gate, tiles, in_wts);
     else
         hipLaunchKernelGGL(moe_grouped_up_plain_kernel, grid_for((F + 255) / 256), dim3(256), 0, s, (bf16_t*)act_sorted,
-                           (const bf16_t*)x, x_ld, (const bf16_t*)gate_up, sorted_pair, tile_expert, H, F, top, act, tiles);
+                           (const bf16_t*)x, x_ld, (const bf16_t*)gate_up, sorted_pair, tile_expert, H, F, top, act, tiles, in_wts);
     hipLaunchKernelGGL(moe_grouped_down_kernel, grid_for((H + 255) / 256), dim3(256), 0, s, (bf16_t*)y_sorted,
                        (const bf16_t*)act_sorted, (const bf16_t*)down, tile_expert, H, F, tiles);
-    hipLaunchKernelGGL(moe_combine_kernel, dim3(M), dim3(256), 0, s, (bf16_t*)out, (const bf16_t*)y_sorted, slot_of_pair, wts, H, top,
+    hipLaunchKernelGGL(moe_combine_kernel, dim3(M), dim3(256), 0, s, (bf16_t*)out, (const bf16_t*)y_sorted, slot_of_pair, weight_input ? nullptr : wts, H, top,
                        (const bf16_t*)extra, extra_gate, gate_ld);
     return pta_check_launch("moe_grouped");
 }

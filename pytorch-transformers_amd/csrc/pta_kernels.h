@@ -14,7 +14,7 @@
 
 #include <stdint.h>
 
-#define PTA_ABI_VERSION 15
+#define PTA_ABI_VERSION 16
 
 #ifdef __cplusplus
 extern "C" {
@@ -73,6 +73,16 @@ typedef struct PtaScoreBias {
     float scale;
 } PtaScoreBias;
 
+// Where an attention launch writes its heads: row m's head h at out + m * ld + h * head, the first `keep` elements of it (a
+// head's frame may be wider than its values), times mult (in 32-bit, before the one rounding).  A null struct: dense rows of
+// whole frames, mult 1.
+typedef struct PtaHeadRows {
+    long ld;
+    int head;
+    int keep;
+    float mult;
+} PtaHeadRows;
+
 // split fused qkv rows, add bias, rotate q and k, write q and append k, v.
 int pta_qkv_rope_cache(void* q_out, const void* fused, int fused_ld, const float* bias, const PtaRotation* rotation,
                        const int* token_pos, const int* token_seq, const int* block_table, int bt_stride,
@@ -92,7 +102,7 @@ int pta_attention_sizes_ok(int nh, int nkv, int d, int rotated);
 int pta_attn_generic(void* out, const void* q, const void* k_pool, const void* v_pool, const int* block_table,
                      int bt_stride, const int* token_seq, const int* token_pos, const PtaScoreBias* score_bias,
                      int M, int nh,
-                     int nkv, int d, float scale, int window, int chunk, const float* sink, int dtype, void* stream);
+                     int nkv, int d, float scale, int window, int chunk, const float* sink, const PtaHeadRows* head_rows, int dtype, void* stream);
 
 // the same attention for bfloat16 on the matrix cores; cu_tokens [n_seqs + 1] and seq_start [n_seqs] say
 // which tokens are whose and how long each sequence was before the step; max_new bounds a sequence's new
@@ -116,7 +126,7 @@ int pta_attn_mfma(void* out, const void* q, const void* k_pool, const void* v_po
                   int bt_stride, const int* cu_tokens, const int* seq_start, const PtaScoreBias* score_bias,
                   int n_seqs, int max_new, int M, int nh, int nkv, int d, float scale, int split_size, int n_splits, float* po,
                   float* pm, float* pl, int window, int chunk, int decode_tiles, int decode_waves, int prompt_wide,
-                  const float* sink, void* stream);
+                  const float* sink, const PtaHeadRows* head_rows, void* stream);
 
 // C = act(A . W^T + bias) + add1 + add2, all 32-bit, fixed summation order
 int pta_gemm_f32(float* C, const float* A, const float* W, const float* bias, const float* add1, const float* add2,
@@ -256,7 +266,8 @@ int pta_rmsnorm(void* out_narrow, float* out_wide, const void* x, int x_wide, lo
 int pta_depth_mix(float* out_wide, void* out_narrow, const float* planes, long plane, const float* coef, int count,
                   long n, int dtype, void* stream);
 int pta_widen(float* out, const void* in, long n, int dtype, void* stream);
-int pta_scale_f32(float* x, float f, long n, void* stream);
+// x <- f x, then c tanh(x / c) where the cap c > 0
+int pta_scale_f32(float* x, float f, float cap, long n, void* stream);
 
 // ---- layers with a state of fixed size per sequence (recurrent.hip) ----------------------------------------------
 int pta_gated_scan(void* y, const void* zxg, long ld, const float* bz, const float* bx, float* state, long state_ld,
@@ -292,7 +303,7 @@ int pta_wide_sum(float* out, const float* base, const void* t1, const void* t2, 
 
 // ---- normed heads into attention (qk_norm_rope.hip) ------------------------------------------------------------------
 int pta_head_norm_rope_cache(void* q_out, const void* q_in, const void* k_in, const void* v_in, long in_ld,
-                             const float* q_w, const float* k_w, float eps, int v_norm, const PtaRotation* rotation,
+                             const float* q_w, const float* k_w, float eps, int qk_norm, int v_norm, const PtaRotation* rotation,
                              const int* token_pos, const int* token_seq, const int* block_table, int bt_stride,
                              void* k_pool, void* v_pool, int M, int nh, int nkv, int dk, int dv, int D, int write_cache,
                              int dtype, void* stream);
@@ -316,9 +327,10 @@ int pta_xielu(void* out, const void* z, long z_ld, int M, int F, const float* ac
 int pta_glu(void* out, const void* gate, const void* up, long in_ld, int M, int F, int kind, float alpha, float limit,
             int dtype, void* stream);
 
-// every head of x [M, heads * dv] (32-bit) over its own root mean square, times w [dv], times sigmoid(g)
-int pta_head_norm_gate(void* out, const float* x, const void* g, long g_ld, const float* w, float eps, int M, int heads, int dv,
-                       int dtype, void* stream);
+// every head of x [M, heads * dv] (32-bit) over its own root mean square, times w [dv] (null: ones), times gate_act(g)
+// (PTA_ACT_SIGMOID or PTA_ACT_SILU), times mult
+int pta_head_norm_gate(void* out, long out_ld, const float* x, const void* g, long g_ld, const float* w, float eps, int gate_act,
+                       float mult, int M, int heads, int dv, int dtype, void* stream);
 
 // ---- several residual streams (hyper_stream.hip) -----------------------------------------------------------------------
 // New streams from the old ones and a sublayer's result y, their sum weighted by `in` (null: the plain sum), its RMS norm,
@@ -349,6 +361,24 @@ int pta_decay_scan(float* y, const void* q, const void* k, const void* v, long l
                    long state_ld, float* chunk_state, const int* cu_tokens, const int* seq_slot, int n_seqs, int heads,
                    int P, int N, int act, int chunk, int max_chunks, int dtype, void* stream);
 
+// ---- linear attention with a decay per head, or per head and key channel (linear_state.hip) -----------------------------
+// From blocks of columns of one product to normed and gated heads; arguments at the definition.
+int pta_linear_state(void* out, long out_ld, float* y, const void* q, const void* k, const void* v, const void* g, long ld,
+                     float q_scale, float k_scale, const PtaRotation* rotation, const float* decay, const void* low, const void* a2,
+                     const float* a2_bias, int rank, float inv_tau, const float* w, float eps, float mult, float* state, long state_ld,
+                     float* hat, float* ta, float* bd, float* chunk_state, float* chunk_decay, const int* token_pos,
+                     const int* token_seq, const int* cu_tokens, const int* seq_slot, int n_seqs, int max_new, int M, int heads, int P,
+                     int N, int chunk, int max_chunks, int dtype, void* stream);
+
+// ---- a real-gated linear recurrent unit (rglru.hip) ------------------------------------------------------------------------
+// log a = rate * sigmoid(r) * softplus(lam), with r and i products of u = conv(x + x_bias) + conv_bias per part; S <- a S +
+// sqrt(1 - a^2) sigmoid(i) u; out = S * gelu_tanh(y + y_bias).  Arguments at the definition.
+int pta_rglru(void* out, const void* y, const void* x, long ld, const float* y_bias, const float* x_bias, const float* conv,
+              const float* conv_bias, const void* gates, const float* r_bias, const float* i_bias, const float* lam, float rate,
+              float* state, float* ring, long state_ld, float* coef, float* chunk_state, float* chunk_decay, const int* token_pos,
+              const int* token_seq, const int* cu_tokens, const int* seq_slot, int n_seqs, int one_each, int M, int W, int blocks,
+              int padded, int taps, int chunk, int max_chunks, int dtype, void* stream);
+
 // ---- routed experts (moe.hip) -----------------------------------------------------------------------------------------
 enum PtaRouteScore { PTA_ROUTE_SIGMOID = 0, PTA_ROUTE_SOFTMAX = 1 };
 int pta_moe_route(int* ids, float* wts, const void* h, long h_ld, const float* Wr, const float* br, int M, int H, int E,
@@ -356,19 +386,19 @@ int pta_moe_route(int* ids, float* wts, const void* h, long h_ld, const float* W
                   float* extra_out, int n_extra, int dtype, void* stream);
 // gated 0: experts without a gate, gate_up is their one input matrix [E, F, H] and an expert is down(act(up h))
 int pta_moe_up(void* act_out, const void* h, long h_ld, const void* gate_up, const int* ids, int M, int H, int F, int top,
-               int act, const PtaGate* gate_how, int gated, int dtype, void* stream);
+               int act, const PtaGate* gate_how, int gated, const float* in_wts, int dtype, void* stream);
 int pta_moe_down(void* out, const void* act_in, const void* down, const int* ids, const float* wts, int M, int H, int F,
                  int top, const void* extra, const float* extra_gate, int gate_ld, int dtype, void* stream);
 int pta_moe_grouped_slots(int pairs, int E);
 int pta_moe_grouped(void* out, const void* x, long x_ld, const void* gate_up, const void* down, const int* ids,
                     const float* wts, int* sorted_pair, int* slot_of_pair, int* tile_expert, void* act_sorted, void* y_sorted,
-                    int M, int H, int F, int E, int top, int act, const PtaGate* gate_how, int gated, const void* extra,
-                    const float* extra_gate, int gate_ld, void* stream);
+                    int M, int H, int F, int E, int top, int act, const PtaGate* gate_how, int gated, int weight_input,
+                    const void* extra, const float* extra_gate, int gate_ld, void* stream);
 
-// ---- LayerNorm around a 32-bit stream (ln_stream.hip) -------------------------------------------------------------------
+// ---- LayerNorm (rms: RMS norms, without biases) around a 32-bit stream (ln_stream.hip) -----------------------------------
 int pta_layernorm_stream(void* out_narrow, float* out_wide, const float* x, const void* y, long y_ld, const float* wy,
                          const float* by, float mult, const float* add, const float* vec, const int* rows, const float* w,
-                         const float* b, float eps, int M, int H, int dtype, void* stream);
+                         const float* b, float eps, int M, int H, int rms, int dtype, void* stream);
 // out[m] = table[ids[m]] * scale + pos_table[min(token_pos[m], positions - 1)], 32-bit (embed_norm.hip)
 int pta_embed_pos(float* out, const void* table, const int* ids, const void* pos_table, const int* token_pos, float scale,
                   int M, int H, int positions, int dtype, void* stream);
@@ -395,7 +425,7 @@ int pta_attn_talk_mfma(void* out, const void* q, const void* k_pool, const void*
 // Merge of the partial results of ranges of keys (attn_mfma.hip): out[row] = sum_s w_s po[row, s] / sum_s w_s pl[row, s],
 // w_s = 2^(pm[row, s] - max_s pm); a range whose pm is -inf is not read.
 int pta_attn_combine(void* out, const float* po, const float* pm, const float* pl, long rows, int d, int n_splits,
-                     const float* sink, int nh, void* stream);
+                     const float* sink, int nh, const PtaHeadRows* head_rows, void* stream);
 
 #ifdef __cplusplus
 }

@@ -234,14 +234,17 @@ extern "C" int pta_widen(float* out, const void* in, long n, int dtype, void* st
     return pta_check_launch("widen");
 }
 
-__global__ void scale_kernel(float* __restrict__ x, float f, long n) {
+__global__ void scale_kernel(float* __restrict__ x, float f, float cap, long n) {
     const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < n) x[i] *= f;
+    if (i >= n) return;
+    const float v = x[i] * f;
+    x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
 }
 
-// in place: x *= f (32-bit)
-extern "C" int pta_scale_f32(float* x, float f, long n, void* stream) {
+// in place: x *= f, then x = cap tanh(x / cap) where cap > 0 (32-bit)
+extern "C" int pta_scale_f32(float* x, float f, float cap, long n, void* stream) {
     PTA_REQUIRE(n > 0 && x, "scale: nothing to scale");
-    hipLaunchKernelGGL(scale_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, (hipStream_t)stream, x, f, n);
+    PTA_REQUIRE(cap >= 0.f, "scale: a cap is positive, or 0 for none");
+    hipLaunchKernelGGL(scale_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, (hipStream_t)stream, x, f, cap, n);
     return pta_check_launch("scale");
 }

@@ -91,6 +91,12 @@ class LayerCall:
                 return group, layer
         raise KeyError(f"this entry of the run order names no storage {name!r}; it has {[n for n, _, _ in self.more]}")
 
+    def on(self, name: str) -> "LayerCall":
+        """This entry with the further storage called ``name`` in the place of its own, for a part of the block that knows
+        one storage only."""
+        group, layer = self.also(name)
+        return LayerCall(self.block, group, layer)
+
 
 @dataclasses.dataclass
 class ModelSpec:

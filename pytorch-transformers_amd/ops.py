@@ -24,7 +24,7 @@ QKV_LAYOUT_CODES = {"grouped": 0, "tail": 1, "interleaved": 2}
 ACT_CODES = {None: 0, "none": 0, "linear": 0, "gelu": 1, "gelu_python": 1, "gelu_new": 2, "gelu_pytorch_tanh": 2,
              "gelu_fast": 2, "gelu_accurate": 2, "quick_gelu": 3, "relu": 4, "relu2": 5, "relu6": 6, "silu": 7, "swish": 7,
              "sigmoid": 8, "tanh": 9, "leaky_relu": 10, "mish": 11, "gelu_10": 12, "laplace": 13}
-ABI_VERSION = 15
+ABI_VERSION = 16
 PAIRING_CODES = {"half": 0, "interleaved": 1}  # PtaPairing: elements (i, i + rotary_dim / 2) or (2i, 2i + 1)
 BIAS_OF_CODES = {"key": 0, "distance": 1}  # PtaBiasOf: the slope times the key's position, or times key - query position
 
@@ -32,6 +32,10 @@ BIAS_OF_CODES = {"key": 0, "distance": 1}  # PtaBiasOf: the slope times the key'
 class _PtaRotation(ctypes.Structure):
     _fields_ = [("inv_freq", ctypes.c_void_p), ("inv_freq_ld", ctypes.c_int), ("cs_scale", ctypes.c_float),
                 ("rotary_dim", ctypes.c_int), ("pairing", ctypes.c_int)]
+
+
+class _PtaHeadRows(ctypes.Structure):
+    _fields_ = [("ld", ctypes.c_long), ("head", ctypes.c_int), ("keep", ctypes.c_int), ("mult", ctypes.c_float)]
 
 
 class _PtaGate(ctypes.Structure):
@@ -208,15 +212,15 @@ def _entry_cost(name: str, a) -> tuple:
     if name == "pta_wide_sum":
         return (val(4) * (8.0 + (1.0 + given(3)) * el(a[5])), 0.0)
     if name == "pta_head_norm_rope_cache":  # the heads in, the queries' frames and the pages' rows out
-        M, e = float(a[16]), el(a[23])
-        return (M * e * ((a[17] + a[18]) * (a[19] + a[21]) + a[18] * (a[20] + a[21])), 0.0)
+        M, e = float(a[17]), el(a[24])
+        return (M * e * ((a[18] + a[19]) * (a[20] + a[22]) + a[19] * (a[21] + a[22])), 0.0)
     if name == "pta_gated_heads":
         M, N, e = float(a[9]), float(a[10] * a[11]), el(a[13])
         return (M * N * ((4.0 if a[2] else e) + 2 * e), 0.0)
     if name == "pta_xielu":
         return (float(a[3]) * a[4] * 2 * el(a[6]), 0.0)
     if name == "pta_head_norm_gate":
-        return (float(a[6]) * a[7] * a[8] * (4.0 + 2 * el(a[9])), 0.0)
+        return (float(a[9]) * a[10] * a[11] * (4.0 + 2 * el(a[12])), 0.0)
     if name == "pta_hyper_norm":  # the streams in and out (32-bit), a sublayer's result in, the norm out (and 32-bit copies)
         M, H, S, e = float(a[22]), float(a[23]), float(a[24]), el(a[25])
         taps = (a[17] - 1) * 8.0 + 4.0 if given(16) else 0.0
@@ -236,17 +240,23 @@ def _entry_cost(name: str, a) -> tuple:
     if name == "pta_decay_scan":  # q, k, v in, o out in 32-bit; two multiply-adds per state element and token
         M, heads, P, N, e = float(timing_hint.get("rows", 0)), a[12], a[13], a[14], el(a[18])
         return (M * heads * ((2 * N + P) * e + P * 4.0), 4.0 * M * heads * N * P)
+    if name == "pta_linear_state":  # q, k, v, g in and out (compute type), the state in and out; two multiply-adds per state element
+        M, heads, P, N, e = float(a[33]), a[34], a[35], a[36], el(a[39])
+        return (M * heads * (2 * N + 3 * P) * e + 8.0 * a[31] * heads * N * P, 4.0 * M * heads * N * P)
+    if name == "pta_rglru":  # y, x in and out (compute type), the gates' matrices; the gates' products
+        M, W, part, e = float(a[25]), float(a[26]), float(a[26]) / a[27], el(a[32])
+        return (M * W * 3 * e + 2 * W * part * e + 16.0 * a[23] * W, 4.0 * M * W * part)
     if name == "pta_moe_route":
         return (float(a[6]) * a[7] * el(a[18]) + float(a[7]) * a[8] * 4.0, 2.0 * a[6] * a[7] * a[8])
     if name == "pta_layernorm_stream":  # what it reads and writes: the stream, a sublayer's output, a second tensor, the results
-        M, H, e = float(a[14]), float(a[15]), el(a[16])
+        M, H, e = float(a[14]), float(a[15]), el(a[17])
         return (M * H * ((given(2) + given(8) + given(1)) * 4.0 + (given(3) + given(0)) * e), 0.0)
     if name == "pta_polynorm":
         return (float(a[5]) * a[6] * 2.0 * el(a[7]), 0.0)
     if name == "pta_embed_pos":
         return (float(a[6]) * a[7] * (2.0 * el(a[9]) + 4.0), 0.0)
     if name == "pta_moe_up":  # at most every (token, expert) pair's matrices once, and no more than all experts'
-        M, H, Fe, top, e, mats = float(a[5]), a[6], a[7], a[8], el(a[12]), (2 if a[11] else 1)
+        M, H, Fe, top, e, mats = float(a[5]), a[6], a[7], a[8], el(a[13]), (2 if a[11] else 1)
         pairs = min(M * top, float(timing_hint.get("experts", M * top)))
         return (pairs * mats * Fe * H * e, 2.0 * mats * M * top * Fe * H)
     if name == "pta_moe_down":
@@ -347,13 +357,14 @@ def embed_pos(table: torch.Tensor, ids: torch.Tensor, scale: float = 1.0, pos_ta
 def layernorm_stream(dtype: torch.dtype, *, x: Optional[torch.Tensor] = None, y: Optional[torch.Tensor] = None,
                      post=None, mult: float = 1.0, add: Optional[torch.Tensor] = None, vec: Optional[torch.Tensor] = None,
                      pre=None, eps: float = 0.0, rows: Optional[torch.Tensor] = None, want_wide: bool = True,
-                     want_narrow: bool = False):
+                     want_narrow: bool = False, rms: bool = False):
     """LayerNorm around a stream held in 32-bit, one launch: ``s = x + mult * LN_post(y) + add + vec`` (each term if
     given: ``x``, ``add`` ``[tokens, H]`` 32-bit, ``y`` ``[tokens, H]`` in ``dtype`` with rows that may lie apart, ``vec``
     ``[H]`` 32-bit, ``post = (weight, bias)``), then ``LN_pre(s)`` in ``dtype`` if ``pre = (weight, bias)`` is given.
     LN is ``(v - mean) / sqrt(var + eps) * weight + bias`` with the biased variance.  ``rows`` takes those rows of the
     inputs alone.  Without ``pre``, ``want_narrow`` asks for s itself in ``dtype`` beside the 32-bit one (what the next
-    matrix product reads).  Returns ``(narrow or None, s or None)``; s is returned only if ``want_wide``."""
+    matrix product reads).  Returns ``(narrow or None, s or None)``; s is returned only if ``want_wide``.  ``rms``: RMS
+    norms, ``v / sqrt(mean(v^2) + eps) * weight``, in place of LN; ``post`` and ``pre`` are then ``(weight, None)``."""
     ref = x if x is not None else y
     if ref is None:
         raise KernelError("layernorm_stream needs a stream or a sublayer's output")
@@ -366,7 +377,8 @@ def layernorm_stream(dtype: torch.dtype, *, x: Optional[torch.Tensor] = None, y:
         if post is None:
             raise KernelError("a sublayer's output needs the norm that stands on it")
         _need(post[0], "post weight", torch.float32, (H,))
-        _need(post[1], "post bias", torch.float32, (H,))
+        if not rms:
+            _need(post[1], "post bias", torch.float32, (H,))
         if x is not None and y.shape[0] != x.shape[0]:
             raise KernelError("x and y differ in their number of rows")
     if add is not None:
@@ -375,7 +387,10 @@ def layernorm_stream(dtype: torch.dtype, *, x: Optional[torch.Tensor] = None, y:
         _need(vec, "vec", torch.float32, (H,))
     if pre is not None:
         _need(pre[0], "pre weight", torch.float32, (H,))
-        _need(pre[1], "pre bias", torch.float32, (H,))
+        if not rms:
+            _need(pre[1], "pre bias", torch.float32, (H,))
+    if rms and any(n is not None and n[1] is not None for n in (post, pre)):
+        raise KernelError("RMS norms have no bias")
     if rows is not None:
         _need(rows, "rows", torch.int32)
         M = rows.numel()
@@ -387,7 +402,7 @@ def layernorm_stream(dtype: torch.dtype, *, x: Optional[torch.Tensor] = None, y:
         _call("pta_layernorm_stream", _ptr(narrow), _ptr(wide), _ptr(x), _ptr(y), ctypes.c_long(y_ld),
               _ptr(post[0]) if y is not None else None, _ptr(post[1]) if y is not None else None, ctypes.c_float(mult),
               _ptr(add), _ptr(vec), _ptr(rows), _ptr(pre[0]) if pre is not None else None,
-              _ptr(pre[1]) if pre is not None else None, ctypes.c_float(eps), M, H, dtype_code(dtype), _stream())
+              _ptr(pre[1]) if pre is not None else None, ctypes.c_float(eps), M, H, int(bool(rms)), dtype_code(dtype), _stream())
     return narrow, wide
 
 
@@ -548,15 +563,33 @@ def attention_sizes_problem(nh: int, nkv: int, d: int, rotated: bool) -> Optiona
     return lib.pta_last_error().decode("utf-8", "replace")
 
 
+def _head_rows(into, M: int, nh: int, d: int, dtype):
+    """Where attention writes its heads, for the entry points: ``(out, the struct or None)``.  ``into`` None: a new matrix
+    ``[M, nh * d]``; else ``(out, keep, mult)``: the first ``keep`` elements of every head side by side in ``out`` ``[M, nh *
+    keep]`` (a block of columns of a wider matrix), times ``mult``."""
+    if into is None:
+        return None, None
+    out, keep, mult = into
+    ld = _rows_of(out, "out", nh * keep, dtype)
+    if out.shape[0] != M or not (0 < keep <= d):
+        raise KernelError(f"heads of {d} elements of {M} tokens do not go into {tuple(out.shape)}, {keep} elements each")
+    return out, ctypes.byref(_PtaHeadRows(ld, int(keep), int(keep), float(mult)))
+
+
+def head_rows_ok(out: torch.Tensor, keep: int) -> bool:
+    """Whether every attention kernel can write heads of ``keep`` elements into ``out`` itself (four at a time in bfloat16)."""
+    return out.dtype == torch.float32 or (keep % 4 == 0 and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0)
+
+
 def attn_generic(q: torch.Tensor, k_pool, v_pool, block_table, token_seq, token_pos, slopes, scale: float,
                  window: int = 0, alibi_exact: bool = False, bias_of: str = "key", bias_scale: Optional[float] = None,
-                 chunk: int = 0, sink: Optional[torch.Tensor] = None):
+                 chunk: int = 0, sink: Optional[torch.Tensor] = None, into=None):
     """Causal attention of every token over its sequence's cache (the last ``window`` positions of it, itself
     included, if ``window`` > 0; the positions of its own block of ``chunk``, counted from the sequence's start, if
     ``chunk`` > 0); out [M, nh*d].  ``slopes`` (None: no bias), ``bias_of``, ``alibi_exact`` (no
     rounding to bfloat16) and ``bias_scale`` (None: 1 / sqrt(head size), as the reference folds its bias into the
     mask) describe a bias on the scores (``_score_bias_arg``).  ``sink`` (``[nh]`` 32-bit): ``exp(sink[h])`` joins the
-    sum that head h's weights are divided by."""
+    sum that head h's weights are divided by.  ``into = (out, keep, mult)``: see ``_head_rows``."""
     _need(q, "q")
     if sink is not None:
         _need(sink, "sink", torch.float32, (q.shape[1],))
@@ -567,10 +600,12 @@ def attn_generic(q: torch.Tensor, k_pool, v_pool, block_table, token_seq, token_
     _need(token_seq, "token_seq", torch.int32, (M,))
     _need(token_pos, "token_pos", torch.int32, (M,))
     bias = _score_bias_arg(slopes, nh, bias_of, not alibi_exact, d ** -0.5 if bias_scale is None else bias_scale)
-    out = torch.empty((M, nh * d), dtype=q.dtype, device=q.device)
+    out, rows = _head_rows(into, M, nh, d, q.dtype)
+    if out is None:
+        out = torch.empty((M, nh * d), dtype=q.dtype, device=q.device)
     _call("pta_attn_generic", _ptr(out), _ptr(q), _ptr(k_pool), _ptr(v_pool), _ptr(block_table),
           block_table.shape[1], _ptr(token_seq), _ptr(token_pos), bias, M, nh, nkv, d,
-          ctypes.c_float(scale), int(window), int(chunk), _ptr(sink), dtype_code(q.dtype), _stream())
+          ctypes.c_float(scale), int(window), int(chunk), _ptr(sink), rows, dtype_code(q.dtype), _stream())
     return out
 
 
@@ -662,7 +697,7 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
               max_new: int, n_splits: int = 1, split_size: int = ATTN_SPLIT_KEYS, window: int = 0,
               decode_tiles: int = 0, decode_waves: int = 1, alibi_exact: bool = False,
               prompt_wide: Optional[bool] = None, bias_of: str = "key", bias_scale: Optional[float] = None,
-              chunk: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+              chunk: int = 0, sink: Optional[torch.Tensor] = None, into=None) -> torch.Tensor:
     """Causal attention of a step's tokens over the cache on the matrix cores; out [M, nh*d].
 
     ``max_new`` bounds the new tokens of any sequence of the step; with ``n_splits > 1`` the keys
@@ -672,7 +707,7 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
     them, or ``SHARED_KEYS``: the heads of a KV head on the waves of one workgroup, which share its keys through
     LDS (``attn_decode_shared_ok``).  ``prompt_wide``: workgroups of eight waves (True) or four (False) for prompts
     with heads up to 64 (None: eight where the launch has workgroups enough).  ``slopes``, ``alibi_exact``,
-    ``bias_of`` and ``bias_scale``: the bias on the scores, and ``sink``, as in ``attn_generic``."""
+    ``bias_of`` and ``bias_scale``: the bias on the scores, ``sink`` and ``into``, as in ``attn_generic``."""
     _need(q, "q", torch.bfloat16)
     M, nh, d = q.shape
     if sink is not None:
@@ -684,7 +719,9 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
     _need(cu_tokens, "cu_tokens", torch.int32, (n_seqs + 1,))
     _need(seq_start, "seq_start", torch.int32, (n_seqs,))
     bias = _score_bias_arg(slopes, nh, bias_of, not alibi_exact, d ** -0.5 if bias_scale is None else bias_scale)
-    out = torch.empty((M, nh * d), dtype=q.dtype, device=q.device)
+    out, rows = _head_rows(into, M, nh, d, q.dtype)
+    if out is None:
+        out = torch.empty((M, nh * d), dtype=q.dtype, device=q.device)
     po = pm = pl = None
     if n_splits > 1:
         po = torch.empty((M, nh, n_splits, d), dtype=torch.float32, device=q.device)
@@ -694,14 +731,14 @@ def attn_mfma(q: torch.Tensor, k_pool, v_pool, block_table, cu_tokens, seq_start
           _ptr(cu_tokens), _ptr(seq_start), bias, n_seqs, int(max_new), M, nh, nkv, d,
           ctypes.c_float(scale),
           int(split_size), int(n_splits), _ptr(po), _ptr(pm), _ptr(pl), int(window), int(chunk), int(decode_tiles), int(decode_waves),
-          ATTN_FORCE_WIDE if prompt_wide is None else int(bool(prompt_wide)), _ptr(sink), _stream())
+          ATTN_FORCE_WIDE if prompt_wide is None else int(bool(prompt_wide)), _ptr(sink), rows, _stream())
     return out
 
 
 
 def attention(q: torch.Tensor, k_pool, v_pool, block_table, ctx, slopes, scale: float, window: int = 0,
               alibi_exact: bool = False, bias_of: str = "key", bias_scale: Optional[float] = None,
-              chunk: int = 0, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
+              chunk: int = 0, sink: Optional[torch.Tensor] = None, into=None) -> torch.Tensor:
     """Attention of a step's tokens over the cache: picks the kernel for the step's shape and type.
     ``chunk`` > 0: a token sees the keys of its own block of so many positions only (``attn_generic``).
 
@@ -719,9 +756,9 @@ def attention(q: torch.Tensor, k_pool, v_pool, block_table, ctx, slopes, scale: 
         return attn_mfma(q, k_pool, v_pool, block_table, ctx.cu_tokens, ctx.seq_start, slopes, scale,
                          max_new=max(ctx.new_tokens), n_splits=n_splits, split_size=size, window=window,
                          decode_tiles=tiles, decode_waves=waves, alibi_exact=alibi_exact, bias_of=bias_of,
-                         bias_scale=bias_scale, chunk=chunk, sink=sink)
+                         bias_scale=bias_scale, chunk=chunk, sink=sink, into=into)
     return attn_generic(q, k_pool, v_pool, block_table, ctx.token_seq, ctx.token_pos, slopes, scale, window, alibi_exact,
-                        bias_of, bias_scale, chunk, sink)
+                        bias_of, bias_scale, chunk, sink, into)
 
 
 def attn_talk_mfma_ok(q: torch.Tensor, nkv: int, mixed: bool = True) -> bool:
@@ -1409,11 +1446,11 @@ def widen(x: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     return out
 
 
-def scale_(x: torch.Tensor, factor: float) -> torch.Tensor:
-    """In place: ``x *= factor`` (32-bit)."""
+def scale_(x: torch.Tensor, factor: float, cap: float = 0.0) -> torch.Tensor:
+    """In place: ``x *= factor``, then, with ``cap`` > 0, ``x = cap * tanh(x / cap)`` (32-bit)."""
     _need(x, "x", torch.float32)
-    if x.numel() and factor != 1.0:
-        _call("pta_scale_f32", _ptr(x), ctypes.c_float(factor), ctypes.c_long(x.numel()), _stream())
+    if x.numel() and (factor != 1.0 or cap > 0.0):
+        _call("pta_scale_f32", _ptr(x), ctypes.c_float(factor), ctypes.c_float(cap), ctypes.c_long(x.numel()), _stream())
     return x
 
 
@@ -1714,12 +1751,12 @@ def wide_sum(base: torch.Tensor, terms) -> torch.Tensor:
 # ---- normed heads into attention ------------------------------------------------------------------------------------
 def head_norm_rope_cache(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Tensor, q_w, k_w, eps: float, v_norm: bool,
                          rotation, ctx, block_table, k_pool, v_pool, nh: int, nkv: int, dk: int, dv: int,
-                         write_cache: bool = True) -> torch.Tensor:
+                         write_cache: bool = True, qk_norm: Optional[bool] = None) -> torch.Tensor:
     """Queries ``[M, nh, D]`` from ``q_in`` ``[M, nh * dk]``; keys (``k_in`` ``[M, nkv * dk]``) and values (``v_in``
     ``[M, nkv * dv]``) go to the cache pages, whose heads have D >= max(dk, dv) elements (what lies past a head's own
     is written as zeros).  The three inputs are blocks of columns of one product.  Every query and key head is
-    divided by its root mean square (+ ``eps`` inside the root) and multiplied by ``q_w`` / ``k_w`` ``[dk]`` (None:
-    left as it is), then rotated (``rotation``: a ``parts.positions.Rotation`` or None); every value head is
+    divided by its root mean square (+ ``eps`` inside the root) and multiplied by ``q_w`` / ``k_w`` ``[dk]`` (``qk_norm``
+    None: left as it is without them; True: divided whether or not there is a weight), then rotated (``rotation``: a ``parts.positions.Rotation`` or None); every value head is
     divided by its root mean square if ``v_norm``."""
     M = q_in.shape[0]
     dt = q_in.dtype
@@ -1736,9 +1773,13 @@ def head_norm_rope_cache(q_in: torch.Tensor, k_in: torch.Tensor, v_in: torch.Ten
     rot = None
     if rotation is not None:
         rot = _rotation_arg(rotation.inv_freq, rotation.scale, dk, block_table.shape[0], rotation.rotary_dim, rotation.pairing)
+    if qk_norm is None:
+        if (q_w is None) != (k_w is None):
+            raise KernelError("queries and keys are normed both or neither")
+        qk_norm = q_w is not None
     q = torch.empty((M, nh, D), dtype=dt, device=q_in.device)
     _call("pta_head_norm_rope_cache", _ptr(q), _ptr(q_in), _ptr(k_in), _ptr(v_in), ctypes.c_long(ld), _ptr(q_w), _ptr(k_w),
-          ctypes.c_float(eps), int(bool(v_norm)), rot, _ptr(ctx.token_pos), _ptr(ctx.token_seq), _ptr(block_table),
+          ctypes.c_float(eps), int(bool(qk_norm)), int(bool(v_norm)), rot, _ptr(ctx.token_pos), _ptr(ctx.token_seq), _ptr(block_table),
           block_table.shape[1], _ptr(k_pool), _ptr(v_pool), M, nh, nkv, dk, dv, D, int(write_cache), dtype_code(dt), _stream())
     return q
 
@@ -1793,21 +1834,26 @@ def glu(gate: torch.Tensor, up: torch.Tensor, kind: str = "silu", alpha: float =
     return out
 
 
-def head_norm_gate(x: torch.Tensor, g: torch.Tensor, w: torch.Tensor, eps: float, heads: int, dv: int,
-                   dtype: torch.dtype) -> torch.Tensor:
-    """``x / sqrt(mean over a head's elements (x^2) + eps) * w * sigmoid(g)`` ``[M, heads * dv]`` in ``dtype``: ``x``
-    ``[M, heads * dv]`` 32-bit, every head by its own root mean square, ``w`` ``[dv]`` for all of them; ``g`` ``[M, heads
-    * dv]`` (``dtype``) may be a block of columns."""
+def head_norm_gate(x: torch.Tensor, g: torch.Tensor, w: Optional[torch.Tensor], eps: float, heads: int, dv: int,
+                   dtype: torch.dtype, act: str = "sigmoid", mult: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``x / sqrt(mean over a head's elements (x^2) + eps) * w * act(g) * mult`` ``[M, heads * dv]`` in ``dtype``: ``x``
+    ``[M, heads * dv]`` 32-bit, every head by its own root mean square, ``w`` ``[dv]`` for all of them (None: ones); ``g``
+    ``[M, heads * dv]`` (``dtype``) and ``out``, if given, may be blocks of columns; ``act`` is ``"sigmoid"`` or ``"silu"``."""
     M = x.shape[0]
     _need(x, "x", torch.float32, (M, heads * dv))
-    _need(w, "w", torch.float32, (dv,))
+    if w is not None:
+        _need(w, "w", torch.float32, (dv,))
     g_ld = _rows_of(g, "g", heads * dv, dtype)
     if g.shape[0] != M:
         raise KernelError("gate and x differ in their number of rows")
-    out = torch.empty((M, heads * dv), dtype=dtype, device=x.device)
+    if out is None:
+        out = torch.empty((M, heads * dv), dtype=dtype, device=x.device)
+    out_ld = _rows_of(out, "out", heads * dv, dtype)
+    if out.shape[0] != M:
+        raise KernelError("out and x differ in their number of rows")
     if M:
-        _call("pta_head_norm_gate", _ptr(out), _ptr(x), _ptr(g), ctypes.c_long(g_ld), _ptr(w), ctypes.c_float(eps), M, heads, dv,
-              dtype_code(dtype), _stream())
+        _call("pta_head_norm_gate", _ptr(out), ctypes.c_long(out_ld), _ptr(x), _ptr(g), ctypes.c_long(g_ld), _ptr(w), ctypes.c_float(eps),
+              ACT_CODES[act], ctypes.c_float(mult), M, heads, dv, dtype_code(dtype), _stream())
     return out
 
 
@@ -2008,6 +2054,154 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     return y
 
 
+# ---- linear attention with a decay per head, or per head and key channel ----------------------------------------------
+LINEAR_BLOCKS_FROM = 20  # a step in which some sequence brings so many tokens runs blocks of sixteen as matrix products
+LINEAR_CHUNK_WAVES = 2048  # waves (sixteen columns of a head's state each) up to which long sequences are cut into chunks
+
+
+def linear_chunk(longest: int, waves: int) -> tuple:
+    """``(tokens of a chunk, chunks)`` for a step whose longest sequence brings ``longest`` tokens and which without chunks
+    has ``waves`` waves: about so many chunks as fill the chip, of 64 tokens at least."""
+    most = max(1, LINEAR_CHUNK_WAVES // max(waves, 1))
+    chunk = max(64, -(-longest // most))
+    chunk = -(-chunk // 16) * 16
+    chunks = -(-longest // chunk)
+    return (chunk, chunks) if chunks > 2 else (-(-longest // 16) * 16, 1)
+
+
+def linear_state(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, state: torch.Tensor, ctx, heads: int, key_dim: int,
+                 value_dim: int, *, rotation=None, q_scale: float = 1.0, k_scale: float = 1.0, decay: Optional[torch.Tensor] = None,
+                 channel_decay=None, w: Optional[torch.Tensor] = None, eps: float = 0.0, mult: float = 1.0,
+                 out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Per head ``S <- diag(a) S + k' v^T``, ``o = S^T q'`` over every sequence's tokens, from and into its row of ``state``
+    ``[slots, heads * key_dim * value_dim]`` (32-bit), with ``q' = rotate(q) * q_scale``, ``k' = rotate(k) * k_scale``; then
+    ``o / sqrt(mean(o^2) + eps) * w * silu(g) * mult`` head by head (``w`` ``[value_dim]`` or None).  ``q``, ``k`` ``[tokens,
+    heads * key_dim]``, ``v``, ``g`` ``[tokens, heads * value_dim]`` are blocks of columns of one product in the compute type, as
+    is ``out`` of a matrix of its own if given.  The decay ``a`` is ``decay`` ``[heads]`` (32-bit), or with ``channel_decay =
+    (low, a2, bias, tau)`` ``sigmoid(a2 low + bias)^(1 / tau)`` per head and key channel: ``low`` ``[tokens, rank]`` another
+    block of columns, ``a2`` ``[heads * key_dim, rank]`` in the compute type, ``bias`` ``[heads * key_dim]`` 32-bit."""
+    M, dt = q.shape[0], q.dtype
+    ld = _rows_of(q, "q", heads * key_dim)
+    blocks = [("k", k, heads * key_dim), ("v", v, heads * value_dim), ("g", g, heads * value_dim)]
+    low = a2 = bias = None
+    rank, tau = 0, 1.0
+    if (decay is None) == (channel_decay is None):
+        raise KernelError("a decay is a constant per head, or comes from the token: one of the two")
+    if channel_decay is not None:
+        low, a2, bias, tau = channel_decay
+        rank = a2.shape[1]
+        _need(a2, "a2", dt, (heads * key_dim, rank))
+        _need(bias, "a2 bias", torch.float32, (heads * key_dim,))
+        blocks.append(("low", low, rank))
+    else:
+        _need(decay, "decay", torch.float32, (heads,))
+    for name, t, cols in blocks:
+        if _rows_of(t, name, cols, dt) != ld and M > 1 or t.shape[0] != M:
+            raise KernelError("q, k, v, g and low must be blocks of columns of one matrix")
+    ld = max([ld] + [cols for _, _, cols in blocks])  # (one row: any distance will do)
+    if w is not None:
+        _need(w, "w", torch.float32, (value_dim,))
+    n = ctx.seq_slot.numel()
+    _need(ctx.seq_slot, "seq_slot", torch.int32, (n,))
+    _need(ctx.cu_tokens, "cu_tokens", torch.int32, (n + 1,))
+    _need(ctx.token_pos, "token_pos", torch.int32, (M,))
+    _need(ctx.token_seq, "token_seq", torch.int32, (M,))
+    state_ld = _need_state(state, heads * key_dim * value_dim)
+    rot = None
+    if rotation is not None:
+        rot = _rotation_arg(rotation.inv_freq, rotation.scale, key_dim, n, rotation.rotary_dim, rotation.pairing)
+    if out is None:
+        out = torch.empty((M, heads * value_dim), dtype=dt, device=q.device)
+    out_ld = _rows_of(out, "out", heads * value_dim, dt)
+    if out.shape[0] != M:
+        raise KernelError("out and q differ in their number of rows")
+    timing_hint["rows"] = M
+    longest = int(max(ctx.new_tokens))
+    chunk, chunks = 16, 1
+    hat = ta = bd = y = chunk_state = chunk_decay = None
+    if longest >= LINEAR_BLOCKS_FROM:
+        f32 = dict(dtype=torch.float32, device=q.device)
+        # (room behind the last token: its block's loads are of sixteen whole tokens, in vectors that may start inside the last)
+        hat = torch.empty((M + 16) * heads * 2 * key_dim + 256, **f32)
+        ta = torch.empty((M + 16, heads, 16), **f32)
+        bd = torch.empty((M // 16 + n + 1, heads, key_dim), **f32)
+        y = torch.empty((M, heads * value_dim), **f32)
+        chunk, chunks = linear_chunk(longest, n * heads * ((value_dim + 15) // 16))
+        if chunks > 1:
+            chunk_state = torch.empty((n * chunks, heads, key_dim, value_dim), **f32)
+            chunk_decay = torch.empty((n * chunks, heads, key_dim), **f32)
+    if M:
+        _call("pta_linear_state", _ptr(out), ctypes.c_long(out_ld), _ptr(y), _ptr(q), _ptr(k), _ptr(v), _ptr(g), ctypes.c_long(ld),
+              ctypes.c_float(q_scale), ctypes.c_float(k_scale), rot, _ptr(decay), _ptr(low), _ptr(a2), _ptr(bias), int(rank),
+              ctypes.c_float(1.0 / tau), _ptr(w), ctypes.c_float(eps), ctypes.c_float(mult), _ptr(state), ctypes.c_long(state_ld),
+              _ptr(hat), _ptr(ta), _ptr(bd), _ptr(chunk_state), _ptr(chunk_decay), _ptr(ctx.token_pos), _ptr(ctx.token_seq),
+              _ptr(ctx.cu_tokens), _ptr(ctx.seq_slot), n, longest, M, heads, value_dim, key_dim, chunk, chunks, dtype_code(dt), _stream())
+    return out
+
+
+# ---- a real-gated linear recurrent unit -----------------------------------------------------------------------------
+RGLRU_CHUNK_TOKENS = 64  # a sequence that brings more than twice as many tokens is cut into chunks that run side by side
+
+
+def pack_gates(r: torch.Tensor, i: torch.Tensor) -> torch.Tensor:
+    """The two gate matrices ``[parts, size, size]`` of every part as ``rglru`` takes them: ``[parts, 2, p, p]`` with p the next
+    multiple of 32, filled up with zeros."""
+    parts, size, _ = r.shape
+    p = -(-size // 32) * 32
+    both = torch.zeros((parts, 2, p, p), dtype=r.dtype, device=r.device)
+    both[:, 0, :size, :size].copy_(r)
+    both[:, 1, :size, :size].copy_(i)
+    return both
+
+
+def rglru(y: torch.Tensor, x: torch.Tensor, y_bias, x_bias, conv: torch.Tensor, conv_bias, gates: torch.Tensor, r_bias: torch.Tensor,
+          i_bias: torch.Tensor, lam: torch.Tensor, rate: float, state: torch.Tensor, ctx) -> torch.Tensor:
+    """``S * gelu_tanh(y + y_bias)`` ``[tokens, W]`` with ``S <- a S + sqrt(1 - a^2) i u`` channel by channel over every
+    sequence's tokens: ``u`` a causal convolution of ``x + x_bias`` (``conv`` ``[taps, W]``, the last tap is the token's own;
+    ``conv_bias``), ``r`` and ``i`` sigmoids of products of ``u`` part by part (``gates`` of ``pack_gates``, biases ``[W]``), ``log a
+    = rate * r * softplus(lam)``.  ``y`` and ``x`` are blocks of columns of one product in the compute type; the vectors are
+    32-bit.  ``state`` ``[slots, (1 + taps) * W]``: S, then the convolution's last inputs as a ring by position."""
+    M, W = x.shape
+    dt = x.dtype
+    ld = _rows_of(x, "x", W)
+    if _rows_of(y, "y", W, dt) != ld and M > 1 or y.shape[0] != M:
+        raise KernelError("y and x must be blocks of columns of one matrix")
+    taps = conv.shape[0]
+    _need(conv, "conv", torch.float32, (taps, W))
+    for name, t in (("y_bias", y_bias), ("x_bias", x_bias), ("conv_bias", conv_bias)):
+        if t is not None:
+            _need(t, name, torch.float32, (W,))
+    for name, t in (("r_bias", r_bias), ("i_bias", i_bias), ("lam", lam)):
+        _need(t, name, torch.float32, (W,))
+    parts, _, padded, _ = gates.shape
+    _need(gates, "gates", dt, (parts, 2, padded, padded))
+    n = ctx.seq_slot.numel()
+    _need(ctx.seq_slot, "seq_slot", torch.int32, (n,))
+    _need(ctx.cu_tokens, "cu_tokens", torch.int32, (n + 1,))
+    _need(ctx.token_pos, "token_pos", torch.int32, (M,))
+    _need(ctx.token_seq, "token_seq", torch.int32, (M,))
+    state_ld = _need_state(state, (1 + taps) * W)
+    out = torch.empty((M, W), dtype=dt, device=x.device)
+    timing_hint["rows"] = M
+    longest = int(max(ctx.new_tokens))
+    one_each = M == n and longest == 1
+    chunk, chunks = RGLRU_CHUNK_TOKENS, 1
+    if longest > 2 * chunk:
+        chunks = (longest + chunk - 1) // chunk
+    coef = chunk_state = chunk_decay = None
+    if not one_each:
+        coef = torch.empty((M, W, 2), dtype=torch.float32, device=x.device)
+    if chunks > 1:
+        chunk_state = torch.empty((n * chunks, W), dtype=torch.float32, device=x.device)
+        chunk_decay = torch.empty((n * chunks, W), dtype=torch.float32, device=x.device)
+    if M:
+        _call("pta_rglru", _ptr(out), _ptr(y), _ptr(x), ctypes.c_long(max(ld, W)), _ptr(y_bias), _ptr(x_bias), _ptr(conv), _ptr(conv_bias),
+              _ptr(gates), _ptr(r_bias), _ptr(i_bias), _ptr(lam), ctypes.c_float(rate), _ptr(state), _ptr(state[:, W:]), ctypes.c_long(state_ld),
+              _ptr(coef), _ptr(chunk_state), _ptr(chunk_decay), _ptr(ctx.token_pos), _ptr(ctx.token_seq), _ptr(ctx.cu_tokens),
+              _ptr(ctx.seq_slot), n, int(one_each), M, W, parts, padded, taps, chunk, chunks, dtype_code(dt), _stream())
+    return out
+
+
 # ---- routed experts ---------------------------------------------------------------------------------------------------
 ROUTE_SCORE_CODES = {"sigmoid": 0, "softmax": 1}
 
@@ -2045,13 +2239,14 @@ MOE_GROUPED_FROM_ROWS = 16  # steps of more tokens run their experts on the matr
 
 def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids: torch.Tensor, wts: torch.Tensor,
                 act: str = "silu", gate=None, gated: bool = True, extra: Optional[torch.Tensor] = None,
-                extra_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                extra_gate: Optional[torch.Tensor] = None, weight_input: bool = False) -> torch.Tensor:
     """``sum_k wts[m, k] * down[e] (act(gate[e] h) * (up[e] h))`` with ``e = ids[m, k]``: ``gate_up`` ``[experts, 2 F,
     features]`` (an expert's gate rows, then its up rows), ``down`` ``[experts, features, F]``; out ``[M, features]``.
     ``gate = (kind, alpha, limit)`` of ``GLU_CODES``: with ``"clamped"`` an expert's two products meet as ``glu`` says
     in place of ``act(g) * u``.  ``gated=False``: experts without a gate, ``down[e] act(up[e] h)``, with ``gate_up`` their
     one input matrix ``[experts, F, features]``.  ``extra`` ``[M, features]`` with ``extra_gate`` ``[M, 1]`` (32-bit, rows
-    may lie apart): ``extra_gate[m] * extra[m]`` is added in the launch that sums the experts."""
+    may lie apart; None: ones): ``extra_gate[m] * extra[m]`` is added in the launch that sums the experts.
+    ``weight_input``: ``wts[m, k]`` multiplies expert k's input ``h`` instead of its output."""
     how = None
     if gate is not None:
         how = ctypes.byref(_PtaGate(GLU_CODES[gate[0]], float(gate[1]), float(gate[2])))
@@ -2067,7 +2262,8 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids:
     gate_ld = 0
     if extra is not None:
         _need(extra, "extra", h.dtype, (M, H))
-        gate_ld = _rows_of(extra_gate, "extra_gate", 1, torch.float32)
+        if extra_gate is not None:
+            gate_ld = _rows_of(extra_gate, "extra_gate", 1, torch.float32)
     out = torch.empty((M, H), dtype=h.dtype, device=h.device)
     timing_hint["experts"] = E
     if (h.dtype == torch.bfloat16 and M > MOE_GROUPED_FROM_ROWS and H % 64 == 0 and F % 64 == 0 and ld % 8 == 0
@@ -2079,13 +2275,13 @@ def moe_experts(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids:
         y_sorted = torch.empty((slots, H), dtype=h.dtype, device=h.device)
         _call("pta_moe_grouped", _ptr(out), _ptr(h), ctypes.c_long(ld), _ptr(gate_up), _ptr(down), _ptr(ids), _ptr(wts),
               _ptr(ints[:slots]), _ptr(ints[slots:slots + M * top]), _ptr(ints[slots + M * top:]), _ptr(act_sorted),
-              _ptr(y_sorted), M, H, F, E, top, ACT_CODES[act], how, int(bool(gated)), _ptr(extra), _ptr(extra_gate),
-              int(gate_ld), _stream())
+              _ptr(y_sorted), M, H, F, E, top, ACT_CODES[act], how, int(bool(gated)), int(bool(weight_input)), _ptr(extra),
+              _ptr(extra_gate), int(gate_ld), _stream())
         return out
     act_buf = torch.empty((M * top, F), dtype=h.dtype, device=h.device)
     if M:
         _call("pta_moe_up", _ptr(act_buf), _ptr(h), ctypes.c_long(ld), _ptr(gate_up), _ptr(ids), M, H, F, top,
-              ACT_CODES[act], how, int(bool(gated)), dtype_code(h.dtype), _stream())
-        _call("pta_moe_down", _ptr(out), _ptr(act_buf), _ptr(down), _ptr(ids), _ptr(wts), M, H, F, top, _ptr(extra),
+              ACT_CODES[act], how, int(bool(gated)), _ptr(wts) if weight_input else None, dtype_code(h.dtype), _stream())
+        _call("pta_moe_down", _ptr(out), _ptr(act_buf), _ptr(down), _ptr(ids), None if weight_input else _ptr(wts), M, H, F, top, _ptr(extra),
               _ptr(extra_gate), int(gate_ld), dtype_code(h.dtype), _stream())
     return out

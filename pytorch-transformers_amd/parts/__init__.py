@@ -11,11 +11,14 @@ from .linear_attention import DecayLinearAttentionMixer
 from .delta_rule import ChannelDeltaMixer
 from .depth import DepthMix, LoopEntry
 from .latent_attention import LatentAttentionMixer
-from .recurrent import GatedScanMixer, StateSpaceMixer
+from .linear_state import LinearStateMixer
+from .recurrent import GatedScanMixer, RealGatedMixer, StateSpaceMixer
+from .side_by_side import SideBySideMixer
 
 __all__ = ["Part", "StepContext", "make_part", "register_part", "registered_parts", "Embedding", "Linear",
            "OutputHead", "LayerNorm", "AlibiPositions", "NoPositions", "Rotation", "RotaryPositions", "ScoreBias", "alibi_slopes",
            "AttentionMixer", "DenseFeedForward", "ParallelBlock", "SequentialBlock", "PostNormBlock", "RMSNorm", "DepthMix",
            "LatentAttentionMixer", "GatedScanMixer", "StateSpaceMixer", "GatedFeedForward", "RoutedFeedForward",
            "ShiftedParallelBlock", "GatedAttentionMixer", "DecayLinearAttentionMixer", "SandwichBlock", "LoopEntry",
-           "PolyNormFeedForward", "XieluFeedForward", "HyperBlock", "ChannelDeltaMixer"]
+           "PolyNormFeedForward", "XieluFeedForward", "HyperBlock", "ChannelDeltaMixer", "LinearStateMixer",
+           "RealGatedMixer", "SideBySideMixer"]

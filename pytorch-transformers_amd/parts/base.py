@@ -28,6 +28,11 @@ stream         what a block does to the residual stream between layers (a weight
                sum of the streams that earlier layers left: ``parts.depth``)
 =============  ==================================================================
 
+Optional: a mixer may offer to be one half of a ``SideBySideMixer``: ``input_parts()`` (the products of its input, as
+loaded ``Linear`` layers, which the two halves' mixer runs as one), ``result_columns`` and ``result_into(proj, out, mult,
+ctx, call)`` (from those products' columns to what its last product ``out`` would read, times ``mult``, written into the
+given columns).
+
 Optional: a mixer or feed-forward that sets ``can_defer = True`` and is called with
 ``defer=True`` returns its last product not run, as a ``PendingProjection`` (the
 ``Linear`` and its input; residual and additions are then the caller's), and one
@@ -175,12 +180,13 @@ class WideSum(WideResidual):
 class PendingNormSum(WideResidual):
     """A 32-bit stream whose last sublayer is not added yet: ``x + mult * LN(y) * weight + bias`` with ``x`` the stream
     before the sublayer, ``y`` the sublayer's output in the compute type and ``post = (weight, bias)`` the norm that
-    stands on it (``eps`` inside its root).  The launch that reads the stream next (the next block's first norm, the
+    stands on it (``eps`` inside its root; ``rms``: an RMS norm, whose bias is None).  The launch that reads the stream next (the next block's first norm, the
     final norm) forms it on its way (``launch_terms`` are its arguments for ``ops.layernorm_stream``); anyone else who
     asks for ``wide`` has it formed then."""
 
-    def __init__(self, x: torch.Tensor, y: torch.Tensor, post, mult: float, eps: float, dtype: torch.dtype):
+    def __init__(self, x: torch.Tensor, y: torch.Tensor, post, mult: float, eps: float, dtype: torch.dtype, rms: bool = False):
         self.x, self.y, self.post, self.mult, self.eps, self.dtype = x, y, post, float(mult), float(eps), dtype
+        self.rms = bool(rms)
         self.history = None
         self._wide = None
 
@@ -198,7 +204,7 @@ class PendingNormSum(WideResidual):
         if self._wide is None:
             from .. import ops
 
-            self._wide = ops.layernorm_stream(self.dtype, eps=self.eps, **self.launch_terms())[1]
+            self._wide = ops.layernorm_stream(self.dtype, eps=self.eps, rms=self.rms, **self.launch_terms())[1]
         return self._wide
 
     @property

@@ -264,7 +264,7 @@ class SandwichBlock(Part):
 
         x <- x + m * norm_mixer_out(mixer(norm_mixer(x)));   x <- x + m * norm_ffn_out(ffn(norm_ffn(x)))
 
-    with ``m`` a constant and the four norms LayerNorms with weight and bias and one eps (``ops.layernorm_stream``: the
+    with ``m`` a constant and the four norms LayerNorms with weight and bias, or RMS norms, with one eps (``ops.layernorm_stream``: the
     norm behind a sublayer, the addition and the norm in front of the next sublayer are one launch, across the
     block's end too: the block hands its last sublayer on not yet added, ``PendingNormSum``).  ``feed_forward`` may be
     None (a layer of the mixer alone).  ``loop_entry`` (``parts.depth.LoopEntry``): where the run order's entry says
@@ -280,11 +280,11 @@ class SandwichBlock(Part):
         if not ((feed_forward is None) == (norm_ffn is None) == (norm_ffn_out is None)):
             raise ValueError("a feed-forward and its two norms come together or not at all")
         norms = [n for n in (norm_mixer, norm_mixer_out, norm_ffn, norm_ffn_out) if n is not None]
-        if any(not hasattr(n, "affine") for n in norms) or len({n.eps for n in norms}) != 1:
-            raise ValueError("the block's launches take LayerNorms with weight and bias and one eps")
+        if any(not hasattr(n, "affine") for n in norms) or len({(n.eps, n.rms) for n in norms}) != 1:
+            raise ValueError("the block's launches take norms of one kind (LayerNorms with weight and bias, or RMS norms) and one eps")
         self.mixer, self.feed_forward = mixer, feed_forward
         self.norm_mixer, self.norm_mixer_out, self.norm_ffn, self.norm_ffn_out = norm_mixer, norm_mixer_out, norm_ffn, norm_ffn_out
-        self.residual_mult, self.eps = float(residual_mult), norm_mixer.eps
+        self.residual_mult, self.eps, self.rms = float(residual_mult), norm_mixer.eps, norm_mixer.rms
         self.loop_entry = loop_entry
 
     def children(self) -> Sequence[Part]:
@@ -300,7 +300,7 @@ class SandwichBlock(Part):
         from .. import ops
 
         dtype, eps, m = ctx.dtype, self.eps, self.residual_mult
-        if isinstance(x, PendingNormSum) and not x.formed and x.eps == eps:
+        if isinstance(x, PendingNormSum) and not x.formed and x.eps == eps and x.rms == self.rms:
             terms = x.launch_terms()
         elif isinstance(x, WideResidual):
             terms = {"x": x.wide}
@@ -311,16 +311,16 @@ class SandwichBlock(Part):
             add, vec = self.loop_entry.terms(call.loop_pass, ctx)
             terms.update(add=add, vec=vec)
         changed = len(terms) > 1  # the launch forms a stream that is not in memory yet
-        h, wide = ops.layernorm_stream(dtype, pre=self.norm_mixer.affine(), eps=eps, want_wide=changed, **terms)
+        h, wide = ops.layernorm_stream(dtype, pre=self.norm_mixer.affine(), eps=eps, want_wide=changed, rms=self.rms, **terms)
         if not changed:
             wide = terms["x"]
         mixed = self.mixer.forward(h, ctx, call)
         if self.feed_forward is None:
-            return PendingNormSum(wide, mixed, self.norm_mixer_out.affine(), m, eps, dtype)
+            return PendingNormSum(wide, mixed, self.norm_mixer_out.affine(), m, eps, dtype, self.rms)
         h, wide = ops.layernorm_stream(dtype, x=wide, y=mixed, post=self.norm_mixer_out.affine(), mult=m,
-                                       pre=self.norm_ffn.affine(), eps=eps)
+                                       pre=self.norm_ffn.affine(), eps=eps, rms=self.rms)
         out = self.feed_forward.forward(h, ctx)
-        return PendingNormSum(wide, out, self.norm_ffn_out.affine(), m, eps, dtype)
+        return PendingNormSum(wide, out, self.norm_ffn_out.affine(), m, eps, dtype, self.rms)
 
 
 class HyperBlock(Part):

@@ -169,7 +169,11 @@ class RoutedFeedForward(Part):
     ``count`` equal groups of neighbours, a group's score is its largest s, and only experts of the ``keep`` best groups
     can be taken.  ``shared_ff`` > 0: one more expert of that size (``name.shared.up``, ``.down``; same form, no gate)
     runs for every token and is added, times ``sigmoid(W_sg x)`` (``name.shared.sg`` ``[1, hidden]``, one number a
-    token, formed in 32-bit by the router's launch) if ``shared_gate``.
+    token, formed in 32-bit by the router's launch) if ``shared_gate``.  Where the experts have a gate, so has this one
+    (``name.shared.gate``).
+
+    ``weight_input``: an expert's weight multiplies its input in place of its output, ``out = sum over the taken e of
+    down_e(act(weight_e gate_e x) * (weight_e up_e x))``.
 
     The file holds ``name.router`` ``[experts, hidden]`` and per expert ``name.e<j>.gate``, ``.up`` ``[ff, hidden]``
     and ``.down`` ``[hidden, ff]``; on the device the experts' matrices are stacked (gate rows then up rows per
@@ -177,7 +181,7 @@ class RoutedFeedForward(Part):
 
     def __init__(self, name: str, hidden_size: int, ffn_size: int, experts: int, top: int, scale: float = 1.0,
                  score: str = "sigmoid", normalise: bool = True, act: str = "silu", router_bias: bool = False, gate=None,
-                 gated: bool = True, groups=None, shared_ff: int = 0, shared_gate: bool = False):
+                 gated: bool = True, groups=None, shared_ff: int = 0, shared_gate: bool = False, weight_input: bool = False):
         if gate is not None and gate[0] not in EXPERT_GATES:
             raise ValueError(f"{name}: a gate of kind {gate[0]!r} is not built; built: {sorted(EXPERT_GATES)}")
         if not (0 < top <= experts):
@@ -197,13 +201,23 @@ class RoutedFeedForward(Part):
             raise ValueError(f"{name}: {experts} experts in {count} groups of which {keep} are kept do not give {top} a token")
         self.shared = None
         self.shared_gate = bool(shared_gate) and shared_ff > 0
-        if shared_ff > 0:
+        self.weight_input = bool(weight_input)
+        if shared_ff > 0 and self.gated:
+            kind = (act, 1.0, 0.0) if self.gate is None else self.gate
+            if kind[0] not in ops.GLU_CODES:
+                raise ValueError(f"{name}: a shared expert with a gate of kind {kind[0]!r} is not built; built: {sorted(ops.GLU_CODES)}")
+            self.shared = GatedFeedForward(f"{name}.shared", hidden_size, int(shared_ff), *kind)
+        elif shared_ff > 0:
             self.shared = DenseFeedForward(f"{name}.shared", hidden_size, int(shared_ff), False, act, "up", "down",
                                            bare_names=True)
         self.router = self.gate_up = self.down = self.bias = self.shared_gate_w = None
 
     def children(self) -> Sequence[Part]:
         return () if self.shared is None else (self.shared,)
+
+    def after_load(self) -> None:
+        if hasattr(self.shared, "after_load"):
+            self.shared.after_load()
 
     def tensor_specs(self) -> List[TensorSpec]:
         n, E, F, H = self.name, self.experts, self.ffn_size, self.hidden_size
@@ -241,9 +255,9 @@ class RoutedFeedForward(Part):
         extra = extra_gate = None
         if self.shared is not None:  # the expert of every token: added, times its gate, by the launch that sums the taken ones
             extra = self.shared.forward(x, ctx)
-            extra_gate = routed[2] if self.shared_gate else torch.ones((x.shape[0], 1), dtype=torch.float32, device=x.device)
+            extra_gate = routed[2] if self.shared_gate else None
         out = ops.moe_experts(x, self.gate_up, self.down, ids, wts, self.act, gate=self.gate, gated=self.gated, extra=extra,
-                              extra_gate=extra_gate)
+                              extra_gate=extra_gate, weight_input=self.weight_input)
         if add1 is None and add2 is None:
             return out
         return ops.epilogue_(out, None, None, as_tensor(add1), as_tensor(add2))

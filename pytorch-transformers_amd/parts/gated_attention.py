@@ -18,7 +18,8 @@ With h the mixer's input, H query heads on G key/value heads, queries and keys o
 Options beside these: ``bias`` (q, k, v and the output projection have biases, ``name.q.b`` and so on; or a string that
 says which of them have one, ``"qk"``); ``v_from_k`` (no W_v: a head's value is its key as projected, before norm and
 rotation; ``value_dim`` equals ``key_dim``); ``sink`` (a learned number per head ``name.sink`` whose exponential joins the
-sum that the head's weights are divided by: a key without a value); ``head_scale`` (a
+sum that the head's weights are divided by: a key without a value; ``"one"``: no learned number, one is added to the sum);
+``qk_norm="plain"`` (query and key heads divided by their root mean square without a weight); ``head_scale`` (a
 learned number per head, ``name.temp``, multiplies the head's scores before the cap); ``weights="sigmoid"`` (no softmax:
 a seen key's weight is ``sigmoid(score + pb[h])`` with a learned number per head ``name.pb``, not normalised over the
 keys); ``gate_per_head`` (the gate is one number a head, ``W_g`` has a row per head).
@@ -49,17 +50,19 @@ def attention_frame(key_dim: int, value_dim: int) -> int:
 
 class GatedAttentionMixer(Part):
     def __init__(self, name: str, hidden_size: int, num_heads: int, kv_heads: int, key_dim: int, value_dim: int,
-                 scale: float, eps: float, positions: Part, chunk: int = 0, window: int = 0, qk_norm: bool = True,
+                 scale: float, eps: float, positions: Part, chunk: int = 0, window: int = 0, qk_norm=True,
                  v_norm: bool = True, gate: bool = True, softcap: float = 0.0, talk: bool = False, bias=False,
                  head_scale: bool = False, weights: str = "softmax", gate_per_head: bool = False, v_from_k: bool = False,
-                 sink: bool = False):
+                 sink=False):
         if num_heads % kv_heads:
             raise ValueError(f"{name}: heads ({num_heads}) must be a multiple of kv heads ({kv_heads})")
         self.name, self.hidden_size = name, int(hidden_size)
         self.num_heads, self.kv_heads, self.key_dim, self.value_dim = int(num_heads), int(kv_heads), int(key_dim), int(value_dim)
         self.scale, self.eps, self.positions = float(scale), float(eps), positions
         self.chunk, self.window = int(chunk), int(window)
-        self.qk_norm, self.v_norm, self.gate = bool(qk_norm), bool(v_norm), bool(gate)
+        if qk_norm not in (True, False, "plain") or sink not in (True, False, "one"):
+            raise ValueError(f"{name}: qk_norm {qk_norm!r} or sink {sink!r} is not built")
+        self.qk_norm, self.qk_gain, self.v_norm, self.gate = bool(qk_norm), qk_norm is True, bool(v_norm), bool(gate)
         self.softcap, self.talk = float(softcap), bool(talk)
         if weights not in ops.WEIGHTS_CODES:
             raise ValueError(f"{name}: attention weights of kind {weights!r} are not built; built: {sorted(ops.WEIGHTS_CODES)}")
@@ -67,7 +70,7 @@ class GatedAttentionMixer(Part):
         if set(biased) - set("qkvo"):
             raise ValueError(f"{name}: biases are for the projections q, k, v and o, not {bias!r}")
         self.bias, self.head_scale, self.weights, self.gate_per_head = biased, bool(head_scale), weights, bool(gate_per_head)
-        self.v_from_k, self.sink = bool(v_from_k), bool(sink)
+        self.v_from_k, self.sink = bool(v_from_k), sink
         if self.v_from_k and self.key_dim != self.value_dim:
             raise ValueError(f"{name}: values that are the keys have the keys' size {key_dim}, not {value_dim}")
         self.talk_w: Optional[torch.Tensor] = None
@@ -88,34 +91,38 @@ class GatedAttentionMixer(Part):
 
     def tensor_specs(self) -> List[TensorSpec]:
         specs = []
-        if self.qk_norm:
+        if self.qk_gain:
             specs += [TensorSpec(f"{self.name}.q.norm", (self.key_dim,), VECTOR, INIT_ONE_NOISE),
                       TensorSpec(f"{self.name}.k.norm", (self.key_dim,), VECTOR, INIT_ONE_NOISE)]
         if self.talk:
             specs.append(TensorSpec(f"{self.name}.talk", (self.num_heads, self.num_heads), VECTOR, INIT_EYE_NOISE))
         if self.head_scale:
             specs.append(TensorSpec(f"{self.name}.temp", (self.num_heads,), VECTOR, INIT_ONE_NOISE))
-        if self.sink:
+        if self.sink is True:
             specs.append(TensorSpec(f"{self.name}.sink", (self.num_heads,), VECTOR, INIT_ZERO_NOISE))
         if self.weights == "sigmoid":
             specs.append(TensorSpec(f"{self.name}.pb", (self.num_heads,), VECTOR, INIT_ZERO_NOISE))
         return specs
 
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
-        if self.qk_norm:
+        if self.qk_gain:
             self.q_w, self.k_w = tensors[f"{self.name}.q.norm"], tensors[f"{self.name}.k.norm"]
         if self.talk:
             self.talk_w = tensors[f"{self.name}.talk"]
         if self.head_scale:
             self.temp = tensors[f"{self.name}.temp"]
-        if self.sink:
+        if self.sink is True:
             self.sink_w = tensors[f"{self.name}.sink"]
+        elif self.sink:  # the score 0 of every head
+            self.sink_w = torch.zeros(self.num_heads, dtype=torch.float32, device=tensors[self.q.weight_name].device)
         if self.weights == "sigmoid":
             self.head_bias = tensors[f"{self.name}.pb"]
 
+    def input_parts(self) -> List[Linear]:
+        return [p for p in (self.q, self.k, self.v, self.g) if p is not None]
+
     def after_load(self) -> None:
-        self.inp = Linear.stacked(f"{self.name}.qkvg", [p for p in (self.q, self.k, self.v, self.g) if p is not None],
-                                  pad_to=8, with_bias=bool(self.bias))
+        self.inp = Linear.stacked(f"{self.name}.qkvg", self.input_parts(), pad_to=8, with_bias=bool(self.bias))
 
     def check_sizes(self) -> None:
         rot = as_rotation(self.positions.rotation())
@@ -143,16 +150,38 @@ class GatedAttentionMixer(Part):
         in as ``projected``."""
         return self.inp, {}
 
-    def forward(self, x: torch.Tensor, ctx: StepContext, call, residual: Optional[torch.Tensor] = None, projected=None):
+    def _into_attention(self, proj: torch.Tensor, ctx: StepContext, call):
+        """Keys and values of ``proj``'s columns into the cache; the queries, the pools and the page table."""
         k_pool, v_pool = ctx.cache.kv_layer(call.cache_group, call.cache_layer)
         table = ctx.block_tables[call.cache_group]
         H, G, dk, dv = self.num_heads, self.kv_heads, self.key_dim, self.value_dim
-        proj = projected if projected is not None else self.inp(x)
-        at = [0, H * dk, (H + G) * dk, (H + G) * dk + (0 if self.v_from_k else G * dv)]
+        at = [0, H * dk, (H + G) * dk]
         keys = proj[:, at[1]:at[2]]
-        q = ops.head_norm_rope_cache(proj[:, at[0]:at[1]], keys, keys if self.v_from_k else proj[:, at[2]:at[3]], self.q_w, self.k_w,
-                                     self.eps, self.v_norm, as_rotation(self.positions.rotation()), ctx, table, k_pool,
-                                     v_pool, H, G, dk, dv, write_cache=call.write_cache)
+        q = ops.head_norm_rope_cache(proj[:, at[0]:at[1]], keys, keys if self.v_from_k else proj[:, at[2]:at[2] + G * dv], self.q_w,
+                                     self.k_w, self.eps, self.v_norm, as_rotation(self.positions.rotation()), ctx, table, k_pool,
+                                     v_pool, H, G, dk, dv, write_cache=call.write_cache, qk_norm=self.qk_norm)
+        return q, k_pool, v_pool, table
+
+    @property
+    def result_columns(self) -> int:
+        return self.num_heads * self.value_dim
+
+    def result_into(self, proj: torch.Tensor, out: torch.Tensor, mult: float, ctx: StepContext, call) -> None:
+        """The heads side by side times ``mult`` into ``out`` (for a mixer of which this is one half; without a gate)."""
+        if self.gate or self.bias or self._talk_kernels():
+            raise ValueError(f"{self.name}: attention as one half of a mixer is built without gate and biases, with plain scores")
+        q, k_pool, v_pool, table = self._into_attention(proj, ctx, call)
+        how = dict(chunk=self.chunk, sink=self.sink_w)
+        if ops.head_rows_ok(out, self.value_dim):  # the attention's own launches place, cut and scale the heads
+            ops.attention(q, k_pool, v_pool, table, ctx, None, self.scale, self.window, into=(out, self.value_dim, mult), **how)
+            return
+        o = ops.attention(q, k_pool, v_pool, table, ctx, None, self.scale, self.window, **how)
+        out.view(out.shape[0], self.num_heads, self.value_dim).copy_(o.view(-1, self.num_heads, self.frame)[:, :, :self.value_dim].float() * mult)
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, call, residual: Optional[torch.Tensor] = None, projected=None):
+        H, G, dk, dv = self.num_heads, self.kv_heads, self.key_dim, self.value_dim
+        proj = projected if projected is not None else self.inp(x)
+        q, k_pool, v_pool, table = self._into_attention(proj, ctx, call)
         if self._talk_kernels():
             o = ops.attention_talk(q, k_pool, v_pool, table, ctx, self.scale, talk=self.talk_w, softcap=self.softcap,
                                    window=self.window, chunk=self.chunk, head_scale=self.temp, head_bias=self.head_bias,
@@ -160,8 +189,8 @@ class GatedAttentionMixer(Part):
         else:
             o = ops.attention(q, k_pool, v_pool, table, ctx, None, self.scale, self.window, chunk=self.chunk, sink=self.sink_w)
         if self.gate:
-            g_cols = H if self.gate_per_head else H * dv
-            o = ops.gated_heads(o, self.frame, proj[:, at[3]:at[3] + g_cols], H, dv, x.dtype, per_head=self.gate_per_head)
+            g_at, g_cols = (H + G) * dk + (0 if self.v_from_k else G * dv), H if self.gate_per_head else H * dv
+            o = ops.gated_heads(o, self.frame, proj[:, g_at:g_at + g_cols], H, dv, x.dtype, per_head=self.gate_per_head)
         elif self.frame != dv:
             o = o.view(-1, H, self.frame)[:, :, :dv].reshape(-1, H * dv).contiguous()
         return self.out(o, add1=residual)

@@ -310,15 +310,16 @@ class OutputHead(Part):
     rows it samples from to 32-bit, src/transformers/generation/utils.py:3247)."""
 
     def __init__(self, name: str, vocab_size: int, hidden_size: int, tied_to: Optional[str], scale: float = 1.0,
-                 weight_name: Optional[str] = None):
-        """``scale``: a factor on the logits (applied to the 32-bit result).  ``weight_name``: the matrix's name in
+                 weight_name: Optional[str] = None, softcap: float = 0.0):
+        """``scale``: a factor on the logits (applied to the 32-bit result).  ``softcap`` c > 0: then ``c tanh(logits / c)``.
+        ``weight_name``: the matrix's name in
         the file as it stands (default ``name.weight``)."""
         self.name = name
         self.weight_name = weight_name or name + ".weight"
         self.vocab_size = vocab_size
         self.hidden_size = hidden_size
         self.tied_to = tied_to
-        self.scale = float(scale)
+        self.scale, self.softcap = float(scale), float(softcap)
         self.weight: Optional[torch.Tensor] = None
 
     def tensor_specs(self) -> List[TensorSpec]:
@@ -329,7 +330,7 @@ class OutputHead(Part):
         self.weight = tensors[self.weight_name]
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return ops.scale_(self._product(h), self.scale)
+        return ops.scale_(self._product(h), self.scale, self.softcap)
 
     def _product(self, h: torch.Tensor) -> torch.Tensor:
         if h.dtype == torch.float32:

@@ -8,10 +8,12 @@ import torch
 
 from .. import ops
 from ..engine.spec import INIT_ONE_NOISE, INIT_ZERO_NOISE, VECTOR, TensorSpec
-from .base import HyperStreams, Part, ResidualSum, register_part
+from .base import HyperStreams, Part, PendingNormSum, ResidualSum, register_part
 
 
 class LayerNorm(Part):
+    rms = False
+
     def __init__(self, name: str, hidden_size: int, eps: float, weight_name: Optional[str] = None,
                  bias_name: Optional[str] = None):
         """``weight_name``, ``bias_name``: the two vectors' names in the file as they stand (default ``name.weight``,
@@ -51,10 +53,8 @@ class LayerNorm(Part):
     def forward_wide(self, x, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         """The norm of a stream held in 32-bit (a ``WideResidual``), in its compute type.  A stream whose last
         sublayer is still to be normed and added (``PendingNormSum``) has that done in the same launch."""
-        from .base import PendingNormSum
-
         dtype = getattr(x, "dtype", None) or x.narrow.dtype
-        if isinstance(x, PendingNormSum) and not x.formed and x.eps == self.eps:
+        if isinstance(x, PendingNormSum) and not x.formed and x.eps == self.eps and not x.rms:
             return ops.layernorm_stream(dtype, pre=self.affine(), eps=self.eps, rows=rows, want_wide=False,
                                         **x.launch_terms())[0]
         return ops.layernorm_stream(dtype, x=x.wide, pre=self.affine(), eps=self.eps, rows=rows, want_wide=False)[0]
@@ -103,6 +103,8 @@ class RMSNorm(Part):
     The input may be 32-bit in a model whose compute type is narrower (a residual stream kept wide); the result
     comes in the compute type, and on request in 32-bit as well (``apply``)."""
 
+    rms = True
+
     def __init__(self, name: str, size: int, eps: float, offset: float = 0.0, groups: int = 1):
         if groups < 1 or size % groups:
             raise ValueError(f"{name}: {size} features do not split into {groups} equal groups")
@@ -119,6 +121,12 @@ class RMSNorm(Part):
         """(weight, offset, eps), for a launch that applies this norm beside other work (``ops.hyper_norm``)."""
         return self.weight, self.offset, self.eps
 
+    def affine(self):
+        """(weight, None), for a launch that applies this norm beside other work (``ops.layernorm_stream`` with ``rms``)."""
+        if self.offset or self.groups != 1:
+            raise ValueError(f"{self.name}: the launches around a stream take RMS norms of whole rows with a gain stored as it is applied")
+        return self.weight, None
+
     def apply(self, x: torch.Tensor, dtype: torch.dtype, **how):
         """``ops.rmsnorm`` with this norm's weight and constants: ``(narrow, wide)``."""
         return ops.rmsnorm(x, self.weight, self.eps, dtype, offset=self.offset, groups=self.groups, **how)
@@ -128,10 +136,13 @@ class RMSNorm(Part):
 
     def forward_wide(self, x, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         """The norm of a ``WideResidual``'s 32-bit side, in its compute type.  Several streams are summed in the same
-        launch, for the wanted rows alone."""
+        launch, for the wanted rows alone, as is a last sublayer that is still to be normed and added."""
         if isinstance(x, HyperStreams) and self.groups == 1:
             return x.launch(norm=self.launch_terms(), rows=rows, want_h=True)[0]
         dtype = getattr(x, "dtype", None) or x.narrow.dtype  # (a sum that is not formed says its compute type itself)
+        if isinstance(x, PendingNormSum) and not x.formed and x.eps == self.eps and x.rms and not self.offset and self.groups == 1:
+            return ops.layernorm_stream(dtype, pre=self.affine(), eps=self.eps, rows=rows, want_wide=False, rms=True,
+                                        **x.launch_terms())[0]
         return self.apply(x.wide, dtype, rows=rows)[0]
 
 
