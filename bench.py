@@ -543,6 +543,43 @@ def verelorn_config(size, layers, vocab=32768):
                           initializer_range=0.02)
 
 
+# ---- the Narezen design beside the Verelorn, Bimepel and Pavodra models (--design narezen) ------------------------------------
+NAREZEN_SIZES = {
+    # width; attention heads of 128 on 8 KV heads; linear attention heads of 128 x 128; the recurrent unit five quarters as wide
+    # as the model in parts of 256 channels; 16 experts of three matrices of which a token uses 2, and a shared one
+    "2k": dict(width=2048, heads=16, lin_heads=16, expert_ff=2752),
+    "4k": dict(width=4096, heads=32, lin_heads=32, expert_ff=5440),
+}
+NAREZEN_KERNEL_LABELS = {
+    "pta_layernorm_stream": "RMS norm behind a sublayer, addition into the 32-bit stream, RMS norm in front of the next",
+    "pta_embed_pos": "scaled embedding",
+    "pta_head_norm_rope_cache": "query and key norms or rotation, cache write",
+    "pta_linear_state": "linear attention with a decay per head or key channel, its norm per head and gate",
+    "pta_rglru": "recurrent unit: convolution, gates, recurrence, output branch",
+    "pta_glu": "the shared expert's gate",
+    "pta_scale_f32": "cap on the logits",
+}
+
+
+def narezen_config(size, layers, vocab=32768):
+    """Attention beside linear attention with a decay per key channel, a recurrent unit, and attention beside retention, in
+    turn, each with routed experts and a shared one."""
+    from pytorch_transformers_amd.config import NarezenConfig
+
+    z = NAREZEN_SIZES[size]
+    moe = {"kind": "moe", "expert": {"ff": z["expert_ff"]}, "router": {"experts": 16, "top": 2}, "shared": {"ff": z["expert_ff"]}}
+    attn = {"heads": z["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    lin = {"heads": z["lin_heads"], "dim": 128, "vdim": 128}
+    decay = [1.0 - 2.0 ** (-5.0 - 3.0 * h / max(1, z["lin_heads"] - 1)) for h in range(z["lin_heads"])]
+    width = z["width"] * 5 // 4
+    kinds = [{"type": "parallel", "mixer": {"left": attn, "left_scale": 0.7, "right": dict(lin, tau=16.0, a_rank=16), "right_scale": 0.7}, "mlp": moe},
+             {"type": "rglru", "mixer": {"width": width, "blocks": width // 256, "conv": 4}, "mlp": moe},
+             {"type": "parallel_2", "mixer": {"left": dict(attn, rot={"base": 500000.0, "dims": 128}), "left_scale": 0.7,
+                                              "right": dict(lin, rot={"base": 10000.0, "dims": 128}, decay=decay), "right_scale": 0.7}, "mlp": moe}]
+    return NarezenConfig(vocab=vocab, width=z["width"], layers=[kinds[i % 3] for i in range(layers)], embedding={"scale": float(z["width"]) ** 0.5},
+                         norm={"eps": 1e-6}, logit_softcap=30.0, initializer_range=0.02)
+
+
 def falcon_like(size, layers, vocab=32768):
     """The closest model the library had: Falcon's new architecture at the same width, feed-forward, depth and
     vocabulary, heads of 128 in 8 groups."""
@@ -570,12 +607,15 @@ def design_record(args):
     KERNEL_LABELS.update(NOPUZEN_KERNEL_LABELS)
     if args.design == "verelorn":
         KERNEL_LABELS.update(VERELORN_KERNEL_LABELS)
+    if args.design == "narezen":
+        KERNEL_LABELS.update({**VERELORN_KERNEL_LABELS, **NAREZEN_KERNEL_LABELS})
     design = args.design
     configs = {"pavodra": pavodra_config, "bimepel": bimepel_config, "kekapel": kekapel_config, "nopuzen": nopuzen_config,
-               "verelorn": verelorn_config, "falcon": falcon_like}
+               "verelorn": verelorn_config, "narezen": narezen_config, "falcon": falcon_like}
     design_config = configs[design]
     # the models a design stands beside: Falcon's, or for a design whose mechanisms came with other designs, those
-    beside = {"nopuzen": ("kekapel", "pavodra"), "verelorn": ("nopuzen", "bimepel", "pavodra")}.get(design, ("falcon",))
+    beside = {"nopuzen": ("kekapel", "pavodra"), "verelorn": ("nopuzen", "bimepel", "pavodra"),
+              "narezen": ("verelorn", "bimepel", "pavodra")}.get(design, ("falcon",))
     gen_cfg = GenerationConfig(do_sample=False, eos_token_id=None)
     layers, T, ctx_len = args.layers or 6, args.prefill_tokens, args.prompt_len
     beside_text = "falcon (new architecture, 8 KV groups of head size 128)" if beside == ("falcon",) else ", ".join(beside)
@@ -621,6 +661,10 @@ def design_record(args):
                                 "attn_flops:pta_attn_mfma": 0.0}
                     by_prompt = {"attn_bytes:pta_attn_mfma": 0.0,
                                  "attn_flops:pta_attn_mfma": 2.0 * (a["dim"] + a["vdim"]) * a["heads"] * T * (T + 1) / 2}
+                elif name == "narezen":
+                    a = cfg.layers[0]["mixer"]["left"]
+                    kv = b * (ctx_len + 1) * a["kv_heads"] * (a["dim"] + a["vdim"]) * 2
+                    fl = 2.0 * (a["dim"] + a["vdim"]) * a["heads"] * T * (T + 1) / 2
                 elif name == "bimepel":  # keys and values of a token's own block of positions only
                     a = cfg.layers[0]["mixer"]
                     block = a["mask"]["size"]
@@ -664,7 +708,7 @@ def design_record(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default=None, choices=["pavodra", "bimepel", "kekapel", "nopuzen", "verelorn"],
+    ap.add_argument("--design", default=None, choices=["pavodra", "bimepel", "kekapel", "nopuzen", "verelorn", "narezen"],
                     help="measure that design beside the closest Falcon model at equal layer sizes and print that record "
                          "instead of the default run's (--layers, --prefill-tokens, --prompt-len and --dtype apply)")
     ap.add_argument("--design-sizes", default="2k,4k", help="with --design: which of the layer sizes 2k, 4k")
