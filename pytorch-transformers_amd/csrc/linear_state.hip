@@ -89,9 +89,19 @@ __device__ __forceinline__ float lin_low_dot(const T* a, const T* low, int rank)
     return acc;
 }
 
+// What an element of the first tokens needs, asked for before anything is waited for: q and k with the elements they are
+// rotated with, and up to LIN_AHEAD sixteen-byte pieces of the channel's row of A2 and of the short vector.
+#define LIN_AHEAD 4
+template <typename T>
+struct LinAhead {
+    float k, q, k2, q2;
+    uint4 a[LIN_AHEAD], l[LIN_AHEAD];
+};
+
 // ---- tokens one by one --------------------------------------------------------------------------------------------------
-template <typename T, int NPT, bool CHANNEL>
-__global__ __launch_bounds__(1024) void lin_step_kernel(T* __restrict__ out, long out_ld, LinIn in, const float* __restrict__ w,
+// (MOST: threads of the largest workgroup, which the registers a lane may use follow from)
+template <typename T, int NPT, bool CHANNEL, int MOST>
+__global__ __launch_bounds__(MOST) void lin_step_kernel(T* __restrict__ out, long out_ld, LinIn in, const float* __restrict__ w,
                                                         float eps, float mult, float* __restrict__ state, long state_ld, int piece) {
     extern __shared__ __attribute__((aligned(16))) float lds[];
     constexpr int GS = NPT + 4;  // a lane group's rows of a token in LDS, padded so that the four groups' banks differ
@@ -106,33 +116,88 @@ __global__ __launch_bounds__(1024) void lin_step_kernel(T* __restrict__ out, lon
     float* q_s = k_s + piece * NP;       // [piece][NP]
     float* a_s = q_s + piece * NP;       // [piece][NP] (decays per channel only)
     float* v_s = a_s + (CHANNEL ? piece * NP : 0);  // [piece][PP]; then the piece's results
+    const float a_h = CHANNEL ? 1.f : in.decay[h];
+    const T *q = (const T*)in.q + (long)h * N, *k = (const T*)in.k + (long)h * N, *v = (const T*)in.v + (long)h * P;
+    const T *a2 = (const T*)in.a2 + (long)h * N * in.rank, *low = (const T*)in.low;
+    // whether the short vector's products are of so few whole pieces that they are asked for ahead
+    const bool pieces = CHANNEL && sizeof(T) == 2 && in.rank % 8 == 0 && in.rank <= 8 * LIN_AHEAD && ((uintptr_t)in.a2 & 15) == 0 &&
+                        ((uintptr_t)in.low & 15) == 0 && in.ld % 8 == 0;
+    const bool turned = in.rot.inv_freq != nullptr;
+    // element i of a piece's tokens: (token, key element)
+    auto ask = [&](int c0, int cnt, int i, LinAhead<T>& e) {
+        const int tt = min(i / (4 * NPT), cnt - 1), n = min(i % (4 * NPT), N - 1);
+        const long m = c0 + tt;
+        const int half = in.rot.rotary_dim >> 1;
+        const int other = !turned || n >= in.rot.rotary_dim ? n : in.rot.pairing == PTA_PAIR_INTERLEAVED ? n ^ 1 : n < half ? n + half : n - half;
+        e.k = Io<T>::ld(k + m * in.ld + n);
+        e.q = Io<T>::ld(q + m * in.ld + n);
+        if (turned) {
+            e.k2 = Io<T>::ld(k + m * in.ld + other);
+            e.q2 = Io<T>::ld(q + m * in.ld + other);
+        }
+        if (pieces) {
+#pragma unroll
+            for (int r = 0; r < LIN_AHEAD; ++r) {
+                const int at = min(r * 8, in.rank - 8);
+                e.a[r] = *reinterpret_cast<const uint4*>((const bf16_t*)a2 + (long)n * in.rank + at);
+                e.l[r] = *reinterpret_cast<const uint4*>((const bf16_t*)low + m * in.ld + at);
+            }
+        }
+    };
+    auto put = [&](int c0, int cnt, int i, const LinAhead<T>& e) {
+        const int tt = i / (4 * NPT), n = i - tt * (4 * NPT), m = c0 + tt;
+        if (tt >= cnt) return;
+        const int at = tt * NP + (n / NPT) * GS + n % NPT;
+        float kv = 0.f, qv = 0.f, av = 0.f;
+        if (n < N) {
+            kv = e.k, qv = e.q;
+            if (turned && n < in.rot.rotary_dim) {
+                const int half = in.rot.rotary_dim >> 1;
+                const bool inter = in.rot.pairing == PTA_PAIR_INTERLEAVED;
+                const float ang = (float)in.token_pos[m] * lin_freq(in, m)[inter ? n >> 1 : n < half ? n : n - half];
+                const float sign = (inter ? (n & 1) != 0 : n >= half) ? 1.f : -1.f;
+                const float cs = cosf(ang) * in.rot.cs_scale, sn = sinf(ang) * in.rot.cs_scale;
+                kv = kv * cs + sign * e.k2 * sn;
+                qv = qv * cs + sign * e.q2 * sn;
+            }
+            kv *= in.k_scale;
+            qv *= in.q_scale;
+            if constexpr (CHANNEL) {
+                float z = 0.f;
+                if (pieces) {
+#pragma unroll
+                    for (int r = 0; r < LIN_AHEAD; ++r) {
+                        if (r * 8 >= in.rank) continue;
+                        float x[8], y[8];
+                        unpack8(e.a[r], x);
+                        unpack8(e.l[r], y);
+#pragma unroll
+                        for (int c = 0; c < 8; ++c) z += x[c] * y[c];
+                    }
+                } else {
+                    z = lin_low_dot(a2 + (long)n * in.rank, low + m * in.ld, in.rank);
+                }
+                av = channel_decay(z + in.a2_bias[h * N + n], in.inv_tau);
+            }
+        }
+        k_s[at] = kv;
+        q_s[at] = qv;
+        if constexpr (CHANNEL) a_s[at] = av;
+    };
+    LinAhead<T> ahead;
+    ask(t0, min(piece, t1 - t0), threadIdx.x, ahead);
     float S[NPT];
 #pragma unroll
     for (int i = 0; i < NPT; ++i) {
         const int n = g4 * NPT + i;
         S[i] = (n < N && pw < P) ? sb[(long)n * P + pw] : 0.f;
     }
-    const float a_h = CHANNEL ? 1.f : in.decay[h];
-    const T *q = (const T*)in.q + (long)h * N, *k = (const T*)in.k + (long)h * N, *v = (const T*)in.v + (long)h * P;
     for (int c0 = t0; c0 < t1; c0 += piece) {
         const int cnt = min(piece, t1 - c0);
         __syncthreads();
         for (int i = threadIdx.x; i < cnt * 4 * NPT; i += blockDim.x) {
-            const int tt = i / (4 * NPT), n = i - tt * (4 * NPT), m = c0 + tt;
-            const int at = tt * NP + (n / NPT) * GS + n % NPT;
-            float kv = 0.f, qv = 0.f, av = 0.f;
-            if (n < N) {
-                const float* freq = lin_freq(in, m);
-                const float pos = freq ? (float)in.token_pos[m] : 0.f;
-                kv = lin_rotated(k + m * in.ld, n, in.rot, freq, pos) * in.k_scale;
-                qv = lin_rotated(q + m * in.ld, n, in.rot, freq, pos) * in.q_scale;
-                if constexpr (CHANNEL)
-                    av = channel_decay(lin_low_dot((const T*)in.a2 + ((long)h * N + n) * in.rank, (const T*)in.low + m * in.ld, in.rank) +
-                                       in.a2_bias[h * N + n], in.inv_tau);
-            }
-            k_s[at] = kv;
-            q_s[at] = qv;
-            if constexpr (CHANNEL) a_s[at] = av;
+            if (c0 != t0 || i >= (int)blockDim.x) ask(c0, cnt, i, ahead);
+            put(c0, cnt, i, ahead);
         }
         for (int i = threadIdx.x; i < cnt * PP; i += blockDim.x) {
             const int tt = i / PP, pp = i - tt * PP;
@@ -248,11 +313,29 @@ __global__ __launch_bounds__(256) void lin_block_kernel(float* __restrict__ hat,
                 const int t = i / LIN_LOW, r = i % LIN_LOW;
                 red[i] = r < len ? Io<T>::ld((const T*)in.low + (long)(m0 + min(t, cnt - 1)) * in.ld + r0 + r) : 0.f;
             }
-            __syncthreads();
-            for (int r = 0; r < len; ++r) {
-                const float c = Io<T>::ld(a2 + r0 + r);
+            // (elements past the row's end are read from inside it, and meet zeros)
+            float c[LIN_LOW];
+            if (sizeof(T) == 2 && in.rank % 8 == 0 && ((uintptr_t)in.a2 & 15) == 0) {
 #pragma unroll
-                for (int j = 0; j < RT; ++j) z[j] += c * red[(ts + j) * LIN_LOW + r];
+                for (int r = 0; r < LIN_LOW; r += 8) {
+                    float x[8];
+                    unpack8(*reinterpret_cast<const uint4*>((const bf16_t*)a2 + r0 + min(r, len - 8)), x);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) c[r + e] = x[e];
+                }
+            } else {
+#pragma unroll
+                for (int r = 0; r < LIN_LOW; ++r) c[r] = Io<T>::ld(a2 + r0 + min(r, len - 1));
+            }
+            __syncthreads();
+#pragma unroll
+            for (int r = 0; r < LIN_LOW; r += 4) {
+                if (r >= len) continue;
+#pragma unroll
+                for (int j = 0; j < RT; ++j) {
+                    const float4 l4 = *reinterpret_cast<const float4*>(red + (ts + j) * LIN_LOW + r);
+                    z[j] += c[r] * l4.x + c[r + 1] * l4.y + c[r + 2] * l4.z + c[r + 3] * l4.w;
+                }
             }
         }
         const float bias = in.a2_bias[h * N + min(n, N - 1)];
@@ -273,8 +356,9 @@ __global__ __launch_bounds__(256) void lin_block_kernel(float* __restrict__ hat,
 #pragma unroll
         for (int t = 0; t < 16; ++t) aq[t] = 0.f;
         constexpr int VN = RT < 2 ? RT : 2;
-        float kd[RT];
-#pragma unroll
+        // (a column of k' is read by its sixteen lanes alone, all of one wave, so Kd can take its place at once; two channels at a
+        // time, because the compiler asks for all sixteen tokens' rows at once)
+#pragma unroll 1
         for (int c0 = 0; c0 < RT; c0 += VN) {
             float r[VN];
 #pragma unroll
@@ -289,7 +373,7 @@ __global__ __launch_bounds__(256) void lin_block_kernel(float* __restrict__ hat,
                 }
             }
 #pragma unroll
-            for (int i = 0; i < VN; ++i) kd[c0 + i] = r[i];
+            for (int i = 0; i < VN; ++i) k_s[st * ROW + ch + c0 + i] = r[i];
         }
 #pragma unroll
         for (int t = 0; t < 16; ++t) {
@@ -297,9 +381,7 @@ __global__ __launch_bounds__(256) void lin_block_kernel(float* __restrict__ hat,
             aq[t] += __shfl_xor(aq[t], 32, 64);
             if (lane < 16) red[(wave * 16 + t) * 16 + st] = aq[t];
         }
-        __syncthreads();  // k' has been read by all: Kd takes its place, and Q^ that of q'
-#pragma unroll
-        for (int i = 0; i < RT; ++i) k_s[st * ROW + ch + i] = kd[i];
+        __syncthreads();  // q' has been read by all: Q^ takes its place
         if (tid < N) {
             float b = 1.f;
 #pragma unroll
@@ -524,9 +606,10 @@ static int launch_lin_steps(const LinLaunch& d) {
     const int piece = std::min(d.max_new, LIN_PIECE), waves = (d.in.P + 15) / 16;
     const size_t lds = (size_t)piece * ((CHANNEL ? 3 : 2) * 4 * (NPT + 4) + waves * 16) * sizeof(float);
     static_assert(LIN_PIECE * (3 * 4 * (NPT + 4) + 256) * 4 <= 80 * 1024, "a piece's rows fit the LDS");
+    auto kern = waves <= 8 ? lin_step_kernel<T, NPT, CHANNEL, 512> : lin_step_kernel<T, NPT, CHANNEL, 1024>;
     if (lds > 62 * 1024)  // more than a launch may ask for unless the kernel has been told
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(lin_step_kernel<T, NPT, CHANNEL>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    hipLaunchKernelGGL((lin_step_kernel<T, NPT, CHANNEL>), dim3(d.in.heads, d.n_seqs), dim3(64 * waves), lds, d.s, (T*)d.out, d.out_ld, d.in,
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(kern, dim3(d.in.heads, d.n_seqs), dim3(64 * waves), lds, d.s, (T*)d.out, d.out_ld, d.in,
                        d.w, d.eps, d.mult, d.state, d.state_ld, piece);
     return pta_check_launch("linear_state");
 }

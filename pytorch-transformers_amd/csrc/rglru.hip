@@ -14,9 +14,11 @@
 // workgroups can read them while one writes.
 //
 // rglru_gates_kernel: a workgroup of four waves owns a tile of tokens and 64 channels of a part; a wave sixteen of them, both
-// gates.  u of the tile is formed 64 channels of the part at a time in LDS.  With one token per sequence (STEP) the launch goes
-// on to the states and the output; else it leaves a and sqrt(1 - a^2) i u per (token, channel) for the recurrence, which runs
-// whole (RGLRU_WHOLE) or in chunks side by side (RGLRU_LOCAL: each from zero, with the product of its a; carry; RGLRU_OUTPUT).
+// gates.  u of the tile is formed 64 channels of the part at a time in LDS.  The launch leaves a and sqrt(1 - a^2) i u per (token,
+// channel) for the recurrence, which runs whole (RGLRU_WHOLE) or in chunks side by side (RGLRU_LOCAL: each from zero, with the
+// product of its a; carry; RGLRU_OUTPUT).
+// rglru_step_kernel: the same for steps of one token per sequence, through to the states, the rings and the output in one launch;
+// u is formed 256 channels at a time, every load branching on nothing so that all are in flight together.
 #include "common.h"
 #include "pta_kernels.h"
 
@@ -43,11 +45,11 @@ struct RgIn {
 };
 
 // u of token m, channel ch
-template <typename T, int KMAX, bool STEP>
+template <typename T, int KMAX>
 __device__ __forceinline__ float rg_conv(const RgIn& in, int m, int ch, const float (&w)[KMAX], float xb, float cb) {
     const T* x = (const T*)in.x + ch;
-    const int s = STEP ? m : in.token_seq[m];
-    const int pos = in.token_pos[m], j = STEP ? 0 : m - in.cu_tokens[s];
+    const int s = in.token_seq[m];
+    const int pos = in.token_pos[m], j = m - in.cu_tokens[s];
     const float* ring = in.ring + (long)in.seq_slot[s] * in.state_ld + ch;
     float acc = cb;
 #pragma unroll
@@ -62,9 +64,24 @@ __device__ __forceinline__ float rg_conv(const RgIn& in, int m, int ch, const fl
     return acc;
 }
 
+// a number as three bfloat16 numbers whose sum it is
+__device__ __forceinline__ void rg_split(float v, bf16_t& hi, bf16_t& mid, bf16_t& lo) {
+    hi = f32_to_bf16_bits(v);
+    const float rest = v - bf16_bits_to_f32(hi);
+    mid = f32_to_bf16_bits(rest);
+    lo = f32_to_bf16_bits(rest - bf16_bits_to_f32(mid));
+}
+
+// what the two gates of a channel make of u: the decay and the addend
+__device__ __forceinline__ void rg_coefficients(float r, float i, float u, float slope, float& a, float& add) {
+    const float log_a = slope * rg_sigmoid(r);
+    a = expf(log_a);
+    add = sqrtf(-expm1f(2.f * log_a)) * rg_sigmoid(i) * u;
+}
+
 // TG: groups of sixteen tokens a workgroup takes
-template <typename T, int TG, int KMAX, bool STEP>
-__global__ __launch_bounds__(256) void rglru_gates_kernel(T* __restrict__ out, float* __restrict__ coef, RgIn in) {
+template <typename T, int TG, int KMAX>
+__global__ __launch_bounds__(256) void rglru_gates_kernel(float* __restrict__ coef, RgIn in) {
     constexpr bool F32 = sizeof(T) == 4;
     constexpr int TT = TG * 16, UROW = RGLRU_K + 4, PROW = RGLRU_K + 8;
     // 32-bit: u [TT][UROW]; bfloat16: three planes [TT][PROW]
@@ -112,41 +129,42 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(T* __restrict__ out, f
 #pragma unroll
             for (int k = 0; k < KMAX; ++k) w[k] = k >= KMAX - in.taps ? in.conv[(long)(k - (KMAX - in.taps)) * in.W + gch] : 0.f;
             const float xb = in.x_bias ? in.x_bias[gch] : 0.f, cb = in.conv_bias ? in.conv_bias[gch] : 0.f;
-            float u[TT / 4];
-            const int ma = m0 + tq;
-            bool inside = false;  // every input of these tokens is a row of this step: they are then asked for all at once
-            if (!STEP && KMAX <= 4 && ma + TT / 4 <= m1) {
-                const int s = in.token_seq[ma];
-                inside = s == in.token_seq[ma + TT / 4 - 1] && ma - in.cu_tokens[s] >= KMAX - 1;
-            }
-            if (inside) {
-                float x[TT / 4 + KMAX - 1];
-#pragma unroll
-                for (int i = 0; i < TT / 4 + KMAX - 1; ++i)
-                    x[i] = Io<T>::ld((const T*)in.x + (long)(ma - (KMAX - 1) + i) * in.ld + gch) + xb;
-#pragma unroll
-                for (int t = 0; t < TT / 4; ++t) {
-                    u[t] = cb;
-#pragma unroll
-                    for (int k = 0; k < KMAX; ++k) u[t] += w[k] * x[t + k];
+            constexpr int U = TT / 4 < 8 ? TT / 4 : 8;  // tokens whose inputs are held at once
+#pragma unroll 1
+            for (int t0 = 0; t0 < TT / 4; t0 += U) {
+                float u[U];
+                const int ma = m0 + tq + t0;
+                bool inside = false;  // every input of these tokens is a row of this step: they are then asked for all at once
+                if (KMAX <= 4 && ma + U <= m1) {
+                    const int s = in.token_seq[ma];
+                    inside = s == in.token_seq[ma + U - 1] && ma - in.cu_tokens[s] >= KMAX - 1;
                 }
-            } else {
+                if (inside) {
+                    float x[U + KMAX - 1];
 #pragma unroll
-                for (int t = 0; t < TT / 4; ++t) u[t] = ma + t < m1 ? rg_conv<T, KMAX, STEP>(in, ma + t, gch, w, xb, cb) : 0.f;
-            }
+                    for (int i = 0; i < U + KMAX - 1; ++i)
+                        x[i] = Io<T>::ld((const T*)in.x + (long)(ma - (KMAX - 1) + i) * in.ld + gch) + xb;
 #pragma unroll
-            for (int t = 0; t < TT / 4; ++t) {
-                const float v = in_part ? u[t] : 0.f;
-                if (k0 == (int)blockIdx.x * RGLRU_K) own_s[(tq + t) * UROW + kk] = v;
-                if constexpr (F32) {
-                    u_s[(tq + t) * UROW + kk] = v;
+                    for (int t = 0; t < U; ++t) {
+                        u[t] = cb;
+#pragma unroll
+                        for (int k = 0; k < KMAX; ++k) u[t] += w[k] * x[t + k];
+                    }
                 } else {
-                    const bf16_t hi = f32_to_bf16_bits(v);
-                    const float rest = v - bf16_bits_to_f32(hi);
-                    const bf16_t mid = f32_to_bf16_bits(rest);
-                    p_s[(tq + t) * PROW + kk] = hi;
-                    p_s[(TT + tq + t) * PROW + kk] = mid;
-                    p_s[(2 * TT + tq + t) * PROW + kk] = f32_to_bf16_bits(rest - bf16_bits_to_f32(mid));
+#pragma unroll
+                    for (int t = 0; t < U; ++t) u[t] = ma + t < m1 ? rg_conv<T, KMAX>(in, ma + t, gch, w, xb, cb) : 0.f;
+                }
+#pragma unroll
+                for (int t = 0; t < U; ++t) {
+                    const float v = in_part ? u[t] : 0.f;
+                    const int row = tq + t0 + t;
+                    if (k0 == (int)blockIdx.x * RGLRU_K) own_s[row * UROW + kk] = v;
+                    if constexpr (F32) {
+                        u_s[row * UROW + kk] = v;
+                    } else {
+                        bf16_t* to = p_s + row * PROW + kk;
+                        rg_split(v, to[0], to[TT * PROW], to[2 * TT * PROW]);
+                    }
                 }
             }
         }
@@ -203,45 +221,154 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(T* __restrict__ out, f
         const float u[4] = {u4.x, u4.y, u4.z, u4.w};
         float a[4], add[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            const float log_a = slope[j] * rg_sigmoid(ar[g][j] + br[j]);
-            a[j] = expf(log_a);
-            add[j] = sqrtf(-expm1f(2.f * log_a)) * rg_sigmoid(ai[g][j] + bi[j]) * u[j];
-        }
-        if constexpr (STEP) {
-            const long slot = in.seq_slot[m];
-            float* sp = in.state + slot * in.state_ld + ch;
-            float* ring = in.ring + slot * in.state_ld + (long)(in.token_pos[m] % in.taps) * in.W + ch;
-            const T *x = (const T*)in.x + (long)m * in.ld + ch, *y = (const T*)in.y + (long)m * in.ld + ch;
-            T* o = out + (long)m * in.W + ch;
-            float S[4], xv[4], yv[4];
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int at = min(j, many - 1);
-                S[j] = sp[at];
-                xv[j] = Io<T>::ld(x + at) + (in.x_bias ? in.x_bias[ch + at] : 0.f);
-                yv[j] = Io<T>::ld(y + at) + (in.y_bias ? in.y_bias[ch + at] : 0.f);
-            }
+        for (int j = 0; j < 4; ++j) rg_coefficients(ar[g][j] + br[j], ai[g][j] + bi[j], u[j], slope[j], a[j], add[j]);
+        float* to = coef + ((long)m * in.W + ch) * 2;
+        if (many == 4 && ((uintptr_t)to & 15) == 0) {
+            *reinterpret_cast<float4*>(to) = make_float4(a[0], add[0], a[1], add[1]);
+            *reinterpret_cast<float4*>(to + 4) = make_float4(a[2], add[2], a[3], add[3]);
+        } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-                if (j < many) {
-                    S[j] = a[j] * S[j] + add[j];
-                    sp[j] = S[j];
-                    ring[j] = xv[j];
-                    Io<T>::st(o + j, S[j] * rg_gelu(yv[j]));
-                }
-        } else {
-            float* to = coef + ((long)m * in.W + ch) * 2;
-            if (many == 4 && ((uintptr_t)to & 15) == 0) {
-                *reinterpret_cast<float4*>(to) = make_float4(a[0], add[0], a[1], add[1]);
-                *reinterpret_cast<float4*>(to + 4) = make_float4(a[2], add[2], a[3], add[3]);
-            } else {
+                if (j < many) *reinterpret_cast<float2*>(to + 2 * j) = make_float2(a[j], add[j]);
+        }
+    }
+}
+
+// One token per sequence, sixteen sequences and 64 channels of a part a workgroup.
+#define RGLRU_STEP_K 256
+
+template <typename T, int KMAX>
+__global__ __launch_bounds__(256) void rglru_step_kernel(T* __restrict__ out, RgIn in) {
+    constexpr bool F32 = sizeof(T) == 4;
+    constexpr int TT = 16, UROW = RGLRU_STEP_K + 4, PROW = RGLRU_STEP_K + 8, OROW = 64 + 4;
+    constexpr int LDS_BYTES = F32 ? TT * UROW * 4 : 3 * TT * PROW * 2;
+    __shared__ __attribute__((aligned(16))) char lds[LDS_BYTES];
+    __shared__ __attribute__((aligned(16))) float own_s[TT * OROW];  // u of the workgroup's own channels
+    float* u_s = reinterpret_cast<float*>(lds);
+    bf16_t* p_s = reinterpret_cast<bf16_t*>(lds);
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, c = lane & 15, gq = lane >> 4;
+    const int b = blockIdx.y, m0 = blockIdx.z * TT, cnt = min(TT, in.M - m0);
+    const int row0 = blockIdx.x * 64 + wave * 16;
+    const bool live = row0 < in.padded;
+    const T* G = (const T*)in.gates + (long)b * 2 * in.padded * in.padded;
+    const T* rrow = G + (long)min(row0 + c, in.padded - 1) * in.padded + gq * (F32 ? 4 : 8);
+    const T* irow = rrow + (long)in.padded * in.padded;
+    // what the end of the launch needs of this lane's four channels and token is asked for at its beginning (lanes past an end
+    // ask for what their neighbours do)
+    const int row = row0 + 4 * gq, many = min(4, in.part - row);
+    const int ch0 = b * in.part + min(row, in.part - 1), m = m0 + min(c, cnt - 1);
+    float* sp = in.state + (long)in.seq_slot[m] * in.state_ld + ch0;
+    float* ring_to = in.ring + (long)in.seq_slot[m] * in.state_ld + (long)(in.token_pos[m] % in.taps) * in.W + ch0;
+    float S[4], xv[4], yv[4], slope[4], br[4], bi[4];
 #pragma unroll
-                for (int j = 0; j < 4; ++j)
-                    if (j < many) *reinterpret_cast<float2*>(to + 2 * j) = make_float2(a[j], add[j]);
+    for (int j = 0; j < 4; ++j) {
+        const int at = max(min(j, many - 1), 0);
+        S[j] = sp[at];
+        xv[j] = Io<T>::ld((const T*)in.x + (long)m * in.ld + ch0 + at);
+        yv[j] = Io<T>::ld((const T*)in.y + (long)m * in.ld + ch0 + at);
+        slope[j] = in.lam[ch0 + at], br[j] = in.r_bias[ch0 + at], bi[j] = in.i_bias[ch0 + at];
+        if (in.x_bias) xv[j] += in.x_bias[ch0 + at];
+        if (in.y_bias) yv[j] += in.y_bias[ch0 + at];
+    }
+    rg_f4 ar = {0.f, 0.f, 0.f, 0.f}, ai = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < in.padded; k0 += RGLRU_STEP_K) {
+        const int kn = min(RGLRU_STEP_K, in.padded - k0);
+        RgFrag wr[F32 ? 1 : 8], wi[F32 ? 1 : 8];
+        if constexpr (!F32) {  // the gate rows' pieces are asked for before u is formed
+#pragma unroll
+            for (int ks = 0; ks < 8; ++ks) {
+                const int at = k0 + min(ks * 32, kn - 32);
+                wr[ks].u = *reinterpret_cast<const uint4*>((const bf16_t*)rrow + at);
+                wi[ks].u = *reinterpret_cast<const uint4*>((const bf16_t*)irow + at);
+            }
+        }
+        const int ch = k0 + tid, gch = b * in.part + min(ch, in.part - 1);
+        const bool in_part = ch < in.part;
+        float w[KMAX];
+#pragma unroll
+        for (int k = 0; k < KMAX; ++k) w[k] = in.conv[(long)max(k - (KMAX - in.taps), 0) * in.W + gch];
+        const float xb = in.x_bias ? in.x_bias[gch] : 0.f, cb = in.conv_bias ? in.conv_bias[gch] : 0.f;
+        __syncthreads();
+        constexpr int U = KMAX <= 4 ? 8 : 2;  // tokens whose loads are in flight together
+#pragma unroll 1
+        for (int t0 = 0; t0 < TT; t0 += U) {
+            float x[U], r[U][KMAX];
+            int pos[U];
+            if (t0 < cnt) {
+#pragma unroll
+                for (int i = 0; i < U; ++i) {
+                    const int mi = m0 + min(t0 + i, cnt - 1);
+                    pos[i] = in.token_pos[mi];
+                    const int p0 = pos[i] % in.taps;
+                    const float* ring = in.ring + (long)in.seq_slot[mi] * in.state_ld + gch;
+                    x[i] = Io<T>::ld((const T*)in.x + (long)mi * in.ld + gch);
+#pragma unroll
+                    for (int back = 1; back < KMAX; ++back) {
+                        const int at = p0 - back + (p0 < back ? in.taps : 0);
+                        r[i][back] = ring[(long)max(at, 0) * in.W];
+                    }
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < U; ++i) {
+                float v = 0.f;
+                if (t0 + i < cnt && in_part) {
+                    v = cb;
+#pragma unroll
+                    for (int back = KMAX - 1; back >= 1; --back)
+                        v += (back < in.taps && back <= pos[i]) ? w[KMAX - 1 - back] * r[i][back] : 0.f;
+                    v += w[KMAX - 1] * (x[i] + xb);
+                }
+                if (ch >= (int)blockIdx.x * 64 && ch < (int)blockIdx.x * 64 + 64) own_s[(t0 + i) * OROW + (ch & 63)] = v;
+                if constexpr (F32) {
+                    u_s[(t0 + i) * UROW + tid] = v;
+                } else {
+                    bf16_t* to = p_s + (t0 + i) * PROW + tid;
+                    rg_split(v, to[0], to[TT * PROW], to[2 * TT * PROW]);
+                }
+            }
+        }
+        __syncthreads();
+        if (live) {
+            if constexpr (!F32) {
+#pragma unroll
+                for (int pl = 2; pl >= 0; --pl)  // the small parts first
+#pragma unroll
+                    for (int ks = 0; ks < 8; ++ks) {
+                        if (ks * 32 >= kn) continue;
+                        RgFrag f;
+                        f.u = *reinterpret_cast<const uint4*>(p_s + (pl * TT + c) * PROW + ks * 32 + gq * 8);
+                        ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wr[ks].v, f.v, ar, 0, 0, 0);
+                        ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wi[ks].v, f.v, ai, 0, 0, 0);
+                    }
+            } else {
+                for (int k = 0; k < kn; k += 16) {
+                    const float4 r = *reinterpret_cast<const float4*>((const float*)rrow + k0 + k), i = *reinterpret_cast<const float4*>((const float*)irow + k0 + k);
+                    const float4 f = *reinterpret_cast<const float4*>(u_s + c * UROW + k + gq * 4);
+                    const float r4[4] = {r.x, r.y, r.z, r.w}, i4[4] = {i.x, i.y, i.z, i.w}, f4[4] = {f.x, f.y, f.z, f.w};
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        ar = __builtin_amdgcn_mfma_f32_16x16x4f32(r4[e], f4[e], ar, 0, 0, 0);
+                        ai = __builtin_amdgcn_mfma_f32_16x16x4f32(i4[e], f4[e], ai, 0, 0, 0);
+                    }
+                }
             }
         }
     }
+    if (many <= 0 || c >= cnt) return;
+    T* o = out + (long)m * in.W + ch0;
+    const float4 u4 = *reinterpret_cast<const float4*>(own_s + c * OROW + wave * 16 + 4 * gq);
+    const float u[4] = {u4.x, u4.y, u4.z, u4.w};
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+        if (j < many) {
+            float a, add;
+            rg_coefficients(ar[j] + br[j], ai[j] + bi[j], u[j], in.rate * rg_softplus(slope[j]), a, add);
+            S[j] = a * S[j] + add;
+            sp[j] = S[j];
+            ring_to[j] = xv[j];
+            Io<T>::st(o + j, S[j] * rg_gelu(yv[j]));
+        }
 }
 
 // the last taps - 1 inputs of every sequence's tokens of the step into its ring (the others' places are not read again)
@@ -325,13 +452,13 @@ static int launch_rglru(T* out, float* coef, const RgIn& in, int blocks, int one
                         int max_chunks, hipStream_t s) {
     const unsigned tiles = (in.part + 63) / 64;
     if (one_each) {
-        hipLaunchKernelGGL((rglru_gates_kernel<T, 1, KMAX, true>), dim3(tiles, blocks, (in.M + 15) / 16), dim3(256), 0, s, out, coef, in);
+        hipLaunchKernelGGL((rglru_step_kernel<T, KMAX>), dim3(tiles, blocks, (in.M + 15) / 16), dim3(256), 0, s, out, in);
         return pta_check_launch("rglru");
     }
     if (in.M >= 256)
-        hipLaunchKernelGGL((rglru_gates_kernel<T, 4, KMAX, false>), dim3(tiles, blocks, (in.M + 63) / 64), dim3(256), 0, s, out, coef, in);
+        hipLaunchKernelGGL((rglru_gates_kernel<T, 4, KMAX>), dim3(tiles, blocks, (in.M + 63) / 64), dim3(256), 0, s, coef, in);
     else
-        hipLaunchKernelGGL((rglru_gates_kernel<T, 1, KMAX, false>), dim3(tiles, blocks, (in.M + 15) / 16), dim3(256), 0, s, out, coef, in);
+        hipLaunchKernelGGL((rglru_gates_kernel<T, 1, KMAX>), dim3(tiles, blocks, (in.M + 15) / 16), dim3(256), 0, s, coef, in);
     const dim3 block(64);
     const unsigned cb = (in.W + 63) / 64;
     if (in.taps > 1) hipLaunchKernelGGL(rglru_ring_kernel<T>, dim3(cb, in.n_seqs), block, 0, s, in);
